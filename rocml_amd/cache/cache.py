@@ -125,7 +125,7 @@ class PagedGroup(CacheGroup):
     paged = True
 
     def __init__(self, name: str, request, n_lines: int, n_pages: int, page_size: int, window: Optional[int],
-                 chunk: Optional[int] = None):
+                 chunk: Optional[int] = None, keep_first: int = 0):
         super().__init__(name, request, n_lines)
         self.n_pages = n_pages
         self.page_size = page_size
@@ -135,6 +135,9 @@ class PagedGroup(CacheGroup):
         self.window = window
         self.chunk = chunk
         self.span = window if window is not None else chunk
+        # ``keep_first``: with a window, the first so many positions stay visible; the leading pages that hold them are
+        # never given back before the sequence ends
+        self.pinned = pages_for(keep_first, page_size) if window is not None else 0
         self._free = list(range(n_pages - 1, -1, -1))
         self._pages: Dict[int, List[int]] = {}   # slot -> logical page -> pool page, -1 once released
 
@@ -145,15 +148,16 @@ class PagedGroup(CacheGroup):
         return window if window is not None else chunk
 
     @staticmethod
-    def pool_pages(window: Optional[int], geo: Geometry) -> int:
+    def pool_pages(window: Optional[int], geo: Geometry, keep_first: int = 0) -> int:
         """Pages of the pool.  A group with a window holds, per sequence, the pages its window
         spans (one more than the window's pages, as it rarely starts on a page's edge) and the
         page being filled; while a step runs it also holds the pages of the step's own tokens,
         which are only given back when the step's piece is committed.  With a bound on the
         sequences and on the tokens of a piece the group needs no more than that, however long
-        the sequences grow; without them it is sized like a group that keeps everything."""
+        the sequences grow (and the pages of kept first positions, where the layer has such); without them
+        it is sized like a group that keeps everything."""
         if window is not None and geo.max_seqs is not None and geo.step_tokens is not None:
-            return min(geo.n_pages, geo.max_seqs * (pages_for(window, geo.page_size) + 2)
+            return min(geo.n_pages, geo.max_seqs * (pages_for(window, geo.page_size) + 2 + pages_for(keep_first, geo.page_size))
                        + pages_for(geo.step_tokens, geo.page_size))
         return geo.n_pages
 
@@ -200,14 +204,20 @@ class PagedGroup(CacheGroup):
             return length - length % self.chunk
         return 0
 
+    def released_before(self, length: int) -> Tuple[int, int]:
+        """The pages ``first .. stop - 1`` that no query at position ``length`` or later can see."""
+        if self.span is None:
+            return 0, 0
+        return self.pinned, max(self.pinned, self.first_visible(length) // self.page_size)
+
     def trim(self, slot: int, length: int) -> None:
         """After a sequence reached ``length``: a group with a window or blocks releases the pages
         whose positions no query at ``length`` or later can see."""
         if self.span is None:
             return
-        first_needed = self.first_visible(length) // self.page_size
+        first, stop = self.released_before(length)
         table = self._pages[slot]
-        for i in range(min(first_needed, len(table))):
+        for i in range(first, min(stop, len(table))):
             if table[i] >= 0:
                 self._free.append(table[i])
                 table[i] = -1
@@ -236,8 +246,9 @@ class KVGroup(PagedGroup):
     """Paged keys and values of the cache lines that share one ``KVCacheRequest``."""
 
     def __init__(self, name: str, request: KVCacheRequest, n_lines: int, geo: Geometry):
-        super().__init__(name, request, n_lines, self.pool_pages(self.span_of(request), geo), geo.page_size,
-                         request.window, getattr(request, "chunk", None))
+        keep = getattr(request, "keep_first", 0)
+        super().__init__(name, request, n_lines, self.pool_pages(self.span_of(request), geo, keep), geo.page_size,
+                         request.window, getattr(request, "chunk", None), keep)
         # Values are transposed inside a page, which is the order the attention kernels
         # multiply them in.  Zeroed once: rows beyond a sequence's length are never counted,
         # but they are multiplied by a zero weight and so must stay finite.
@@ -250,7 +261,7 @@ class KVGroup(PagedGroup):
     def planned_bytes(request: KVCacheRequest, n_lines: int, geo: Geometry) -> int:
         size = torch.empty((), dtype=geo.dtype).element_size()
         dv = request.head_dim if getattr(request, "v_head_dim", None) is None else request.v_head_dim
-        return (n_lines * PagedGroup.pool_pages(PagedGroup.span_of(request), geo) * geo.page_size
+        return (n_lines * PagedGroup.pool_pages(PagedGroup.span_of(request), geo, getattr(request, "keep_first", 0)) * geo.page_size
                 * request.n_kv_heads * (request.head_dim + dv) * size)
 
     def view(self, line: int, step) -> "CacheLineView":
@@ -504,10 +515,11 @@ class Cache:
                 free -= need
                 if w is not None:        # what the commit of this piece gives back
                     for key, n in piece:
-                        first_needed = min(g.first_visible(n) // g.page_size, size[key])
-                        if first_needed > released[key]:
-                            free += first_needed - released[key]
-                            released[key] = first_needed
+                        first, stop = g.released_before(n)
+                        gone = max(0, min(stop, size[key]) - first)
+                        if gone > released[key]:
+                            free += gone - released[key]
+                            released[key] = gone
             if final:
                 # a token at a time: a sequence of a windowed group then never holds more than
                 # the pages its window spans and the one being filled
@@ -516,7 +528,7 @@ class Cache:
                     held = size.get(key, 0) - released.get(key, 0)
                     want = pages_for(n, g.page_size) - released.get(key, 0)
                     if w is not None:
-                        want = min(want, max(held, pages_for(w, g.page_size) + 2))
+                        want = min(want, max(held, pages_for(w, g.page_size) + 2 + g.pinned))
                     need += max(0, want - held)
                 if need > free:
                     return (f"cache group {g.name}: the sequences would need {need} more pages of "

@@ -136,6 +136,13 @@ def _register_builtin() -> None:
         checkpoint_names=roravik.checkpoint_names,
         unused_tensors=roravik.unused_tensors,
         refine_config=lambda cfg, shapes: cfg.with_shapes(shapes)))
+    from . import kakalorn
+    register_architecture(Architecture(
+        name=kakalorn.ARCHITECTURE,
+        read_config=kakalorn.KakalornConfig.from_dict,
+        to_spec=lambda cfg: cfg.to_model_spec(),
+        checkpoint_names=kakalorn.checkpoint_names,
+        unused_tensors=kakalorn.unused_tensors))
 
 
 _register_builtin()

@@ -56,12 +56,14 @@ class RopeStretch:
 class RopeSpec:
     """Rotary position encoding with NEOX pairing ``(i, i + rot_dim/2)`` over the
     first ``rot_dim`` values of a head; ``theta`` is the frequency base.  ``stretch``: the
-    frequencies are slowed down as ``RopeStretch`` says."""
+    frequencies are slowed down as ``RopeStretch`` says.  ``pairing`` ``"neighbours"``: the pairs are
+    ``(2 i, 2 i + 1)`` instead."""
     head_dim: int
     rot_dim: int
     theta: float
     kind: str = "rope_neox"
     stretch: Optional[RopeStretch] = None
+    pairing: str = "halves"
 
 
 @dataclass(frozen=True)
@@ -89,7 +91,9 @@ class AttentionSpec:
     ``softcap``: the scaled score ``s`` becomes ``softcap * tanh(s / softcap)`` before the mask.
     ``conv``: q, k and v pass a causal convolution of so many taps per channel (no bias, no
     activation) right after their projection; the last ``conv - 1`` projected rows of a sequence
-    are part of its state."""
+    are part of its state.  ``keep_first`` (with a window): the first so many positions stay visible
+    whatever their distance.  ``values_are_keys``: there is no value projection, the values are the keys
+    as projected (with their bias), before norm and rotation."""
     hidden: int
     n_heads: int
     n_kv_heads: int
@@ -112,6 +116,8 @@ class AttentionSpec:
     sink_learned: bool = False
     softcap: Optional[float] = None
     conv: Optional[int] = None
+    keep_first: int = 0
+    values_are_keys: bool = False
 
 
 @dataclass(frozen=True)
@@ -124,7 +130,9 @@ class LatentAttentionSpec:
     ``W_dkv h`` gives ``kv_rank`` values, normed into the latent ``c``, and ``rot_dim`` more, the
     shared rotated key part; per head the unrotated key is ``W_uk c`` and the value ``W_uv c``
     (``v_head_dim`` wide).  ``gate``: the concatenated heads are multiplied by
-    ``sigmoid(W_g h)`` before the output projection."""
+    ``sigmoid(W_g h)`` before the output projection; with ``gate_per_head`` the gate is one number per
+    head.  ``own_rows`` false: the layer has no ``W_dkv`` and runs on the rows another layer keeps (an entry
+    of the schedule with ``reads_cache_of``), with expansions of its own."""
     hidden: int
     n_heads: int
     head_dim: int
@@ -139,6 +147,8 @@ class LatentAttentionSpec:
     window: Optional[int] = None
     gate: bool = False
     kind: str = "latent_attention"
+    gate_per_head: bool = False
+    own_rows: bool = True
 
 
 @dataclass(frozen=True)
@@ -152,6 +162,15 @@ class GatedMlpSpec:
     kind: str = "gated_mlp"
     limit: Optional[float] = None
     up_offset: float = 0.0
+
+
+@dataclass(frozen=True)
+class MlpSpec:
+    """Dense feed-forward without a gate: ``down(act(up(x)))``; ``relu2`` is ``max(z, 0)^2``."""
+    hidden: int
+    intermediate: int
+    activation: str = "relu2"
+    kind: str = "mlp"
 
 
 @dataclass(frozen=True)
@@ -262,6 +281,21 @@ class TimeMixSpec:
 
 
 @dataclass(frozen=True)
+class Hgrn2Spec:
+    """Linear attention in which the forget gate also decides what is written (HGRN2): ``q = silu(W_q h)``,
+    ``v = W_v h`` and per head and key channel ``f = l + (1 - l) sigmoid(W_f h + b)`` with a learned lower bound
+    ``l``; per head ``S <- diag(f) S + (1 - f) v^T``, ``o = S^T q`` with the new ``S``.  Every head's output is
+    normed over ``v_head_dim`` with one gain for all heads, the heads side by side are projected back.  The
+    state (``head_dim x v_head_dim`` per head) is 32-bit."""
+    hidden: int
+    n_heads: int
+    head_dim: int
+    v_head_dim: int
+    eps: float
+    kind: str = "hgrn2"
+
+
+@dataclass(frozen=True)
 class TokenSideSpec:
     """A per-token input that depends on the token's id: with ``e`` the columns ``column0 ..
     column0 + dim - 1`` of the token's row of the model's table ``table``, the result is
@@ -345,7 +379,9 @@ class BlockSpec:
     is applied to a sublayer's output alone.  ``side`` (with ``side_norm``): one more sublayer
     that runs last in the same way (only in ``sublayer_norm``).  ``sandwich_norm`` is
     ``x += mixer_out_norm(mixer(mixer_norm(x))); x += ffn_out_norm(ffn(ffn_norm(x)))``: a norm before
-    and one after every sublayer."""
+    and one after every sublayer.  ``input_conv``: what the mixer reads, ``h``, is first replaced by ``h`` plus
+    a causal convolution of so many taps over it per channel (no bias); the last ``input_conv - 1`` rows of
+    ``h`` are part of a sequence's state (only in ``pre_norm`` and ``sandwich_norm``)."""
     mixer: Any
     ffn: Any
     mixer_norm: Any
@@ -356,6 +392,7 @@ class BlockSpec:
     side_norm: Optional[Any] = None
     mixer_out_norm: Optional[Any] = None
     ffn_out_norm: Optional[Any] = None
+    input_conv: Optional[int] = None
 
 
 @dataclass(frozen=True)

@@ -195,8 +195,8 @@ ROCML_EXPORT int rocml_attention(const void* q, void* out, const void* kcache, c
                                  const int* cu_seqlens, int n_seqs, int max_new, const int* q_counts,
                                  int max_len, int n_splits, void* workspace, long long workspace_bytes,
                                  int dv, int v_in_k, int chunk, const float* slopes, int sink,
-                                 const float* sinks, float softcap, hipStream_t stream) {
-    // dv (0: the key head's size), v_in_k, chunk, slopes, sink, sinks and softcap: see AttnExtra in attention_generic.h.
+                                 const float* sinks, float softcap, int keep_first, hipStream_t stream) {
+    // dv (0: the key head's size), v_in_k, chunk, slopes, sink, sinks, softcap and keep_first: see AttnExtra in attention_generic.h.
     ROCML_REQUIRE(!sinks || sink, "attention: learned sinks need the sink switched on");
     ROCML_REQUIRE(softcap >= 0.f, "attention: negative soft cap %g", (double)softcap);
     if (dv <= 0) dv = d;
@@ -206,7 +206,10 @@ ROCML_EXPORT int rocml_attention(const void* q, void* out, const void* kcache, c
     ROCML_REQUIRE(dv <= AG_BLOCK * AG_MAX_D_PER_THREAD, "attention: value head size %d exceeds %d", dv,
                   AG_BLOCK * AG_MAX_D_PER_THREAD);
     bool plain_features = dv == d && !v_in_k;          // what the matrix-core kernels need
-    bool has_extra = chunk > 0 || slopes || sink || softcap > 0.f;
+    ROCML_REQUIRE(keep_first >= 0, "attention: %d kept first positions", keep_first);
+    if (window == 0) keep_first = 0;                   // (everything is seen anyway)
+    ROCML_REQUIRE(keep_first == 0 || chunk == 0, "attention: kept first positions go with a window");
+    bool has_extra = chunk > 0 || slopes || sink || softcap > 0.f || keep_first > 0;
     ROCML_REQUIRE(n_tokens >= 0 && hq > 0 && hkv > 0 && d > 0 && page_size > 0 && bt_width > 0,
                   "attention: bad sizes T=%d Hq=%d Hkv=%d D=%d page=%d width=%d", n_tokens, hq, hkv,
                   d, page_size, bt_width);
@@ -264,7 +267,7 @@ ROCML_EXPORT int rocml_attention(const void* q, void* out, const void* kcache, c
         AttnArgs a{(const bf16_t*)q, (bf16_t*)out, (const bf16_t*)kcache, (const bf16_t*)vcache, block_table,
                    bt_width, token_seq, token_pos, cu_seqlens, n_seqs, n_tokens, (int)total_q_tiles, max_len, hq, hkv,
                    scale, window, workspace, workspace_bytes, n_splits, nullptr};
-        a.extra = MaskExtra{chunk, slopes, sink, sinks, softcap};
+        a.extra = MaskExtra{chunk, slopes, sink, sinks, softcap, keep_first};
         a.has_extra = has_extra;
         int rc = decode ? BY_HEAD_DIM(launch_decode_plain, d, a, stream) : BY_HEAD_DIM(launch_prefill, d, a, stream);
         if (rc) return rc;
@@ -273,7 +276,7 @@ ROCML_EXPORT int rocml_attention(const void* q, void* out, const void* kcache, c
     }
     dim3 grid(n_tokens, hq);
     size_t lds = (size_t)(d + AG_BLOCK) * sizeof(float);
-    AttnExtra ex{dv, v_in_k, chunk, slopes, sink, sinks, softcap};
+    AttnExtra ex{dv, v_in_k, chunk, slopes, sink, sinks, softcap, keep_first};
     if (dtype == ROCML_F32)
         attn_generic_kernel<float><<<grid, AG_BLOCK, lds, stream>>>(
             (const float*)q, (float*)out, (const float*)kcache, (const float*)vcache, block_table,
@@ -307,8 +310,16 @@ ROCML_EXPORT int rocml_attention_decode_fused(const float* qkv, int ld, int qkv_
                                               int max_len, int n_splits, void* workspace,
                                               long long workspace_bytes, const float* row_ssq, int row_parts,
                                               float row_eps, int row_width, const float* bias, int chunk,
-                                              const float* slopes, int sink, hipStream_t stream) {
-    // bias (may be null): [ld] numbers added to the projection's sums; chunk, slopes, sink: see MaskExtra.
+                                              const float* slopes, int sink, const float* sinks, int keep_first, int rot,
+                                              int v_is_k, hipStream_t stream) {
+    // bias (may be null): [ld] numbers added to the projection's sums; chunk, slopes, sink, sinks, keep_first: see
+    // MaskExtra.  rot: leading values of a head that turn (with tables [tokens, rot/2]; D or 0: all of them).  v_is_k:
+    // the rows hold no value columns, a value is the projected key.
+    if (rot <= 0) rot = d;
+    ROCML_REQUIRE(rot <= d && rot % 2 == 0, "fused decode attention: %d of %d values of a head turn", rot, d);
+    ROCML_REQUIRE(keep_first >= 0 && (keep_first == 0 || chunk == 0), "fused decode attention: kept first positions go with a window");
+    ROCML_REQUIRE(!sinks || sink, "fused decode attention: learned sinks need the sink switched on");
+    if (window == 0) keep_first = 0;
     ROCML_REQUIRE(chunk >= 0 && (chunk == 0 || window == 0), "fused decode attention: a window or blocks of positions, not both");
     ROCML_REQUIRE(n_tokens >= 0 && hq > 0 && hkv > 0 && bt_width > 0 && qkv_splits >= 1,
                   "fused decode attention: bad sizes T=%d Hq=%d Hkv=%d width=%d splits=%d", n_tokens, hq, hkv,
@@ -319,7 +330,7 @@ ROCML_EXPORT int rocml_attention_decode_fused(const float* qkv, int ld, int qkv_
                   "fused decode attention: needs pages of 64 positions and a head size of 64, 128, 192 or 256 "
                   "(page=%d D=%d)", page_size, d);
     ROCML_REQUIRE(window >= 0, "fused decode attention: negative window %d", window);
-    int rows = write_kv ? hq + 2 * hkv : hq;
+    int rows = write_kv ? hq + (v_is_k ? 1 : 2) * hkv : hq;
     ROCML_REQUIRE(ld >= rows * d && ld % 4 == 0 && ((uintptr_t)qkv & 15) == 0 &&
                       (qkv_splits == 1 || (qkv_split_stride >= (long long)n_tokens * ld && qkv_split_stride % 4 == 0)),
                   "fused decode attention: projection rows of %d values (need %d, a multiple of 4, 16-byte aligned), "
@@ -330,12 +341,13 @@ ROCML_EXPORT int rocml_attention_decode_fused(const float* qkv, int ld, int qkv_
     ROCML_REQUIRE(!row_ssq || (row_parts > 0 && row_eps > 0.f && row_width > 0),
                   "fused decode attention: a row scale needs parts, eps and the norm's width");
     DecodeProj pj{qkv, ld, qkv_splits, qkv_split_stride, q_gain, k_gain, eps, cos_t, sin_t, write_kv,
-                  row_ssq, row_parts, row_eps, row_ssq ? 1.0f / (float)row_width : 0.f, bias};
+                  row_ssq, row_parts, row_eps, row_ssq ? 1.0f / (float)row_width : 0.f, bias, rot, v_is_k};
     AttnArgs a{nullptr, (bf16_t*)out, (const bf16_t*)kcache, (const bf16_t*)vcache, block_table, bt_width,
                token_seq, token_pos, nullptr, 0, n_tokens, 0, max_len, hq, hkv, scale, window, workspace,
                workspace_bytes, n_splits, &pj};
-    a.extra = MaskExtra{chunk, slopes, sink};
-    a.has_extra = chunk > 0 || slopes || sink || bias;        // (the bias rides in the same instantiation)
+    a.extra = MaskExtra{chunk, slopes, sink, sinks, 0.f, keep_first};
+    // (the bias, a rotation of a part of the head and values taken from the keys ride in the same instantiation)
+    a.has_extra = chunk > 0 || slopes || sink || bias || keep_first > 0 || rot != d || v_is_k;
     int rc = d == 64 ? launch_decode_fused<64>(a, stream)
              : d == 128 ? launch_decode_fused<128>(a, stream)
              : d == 192 ? launch_decode_fused<192>(a, stream) : launch_decode_fused<256>(a, stream);

@@ -18,7 +18,8 @@
 //  * sink: one more term exp(0) in the denominator, with no value: the running maximum starts at 0
 //    and the running sum at 1;
 //  * sinks[h]: with sink, the term is exp(sinks[h]) instead: the running maximum starts there;
-//  * softcap: the scaled score s becomes softcap * tanh(s / softcap), before the mask and the slope.
+//  * softcap: the scaled score s becomes softcap * tanh(s / softcap), before the mask and the slope;
+//  * keep_first: with a window, the first keep_first positions are seen whatever their distance.
 #pragma once
 #include "common.h"
 
@@ -55,6 +56,7 @@ struct AttnExtra {
     int sink;
     const float* sinks;     // [Hq] or null
     float softcap;          // 0: none
+    int keep_first;         // 0: none
 };
 
 __device__ __forceinline__ int attn_first_key(int pos, int window, int chunk) {
@@ -77,6 +79,9 @@ attn_generic_kernel(const T* __restrict__ q, T* __restrict__ out, const T* __res
     const int* pages = block_table + (size_t)token_seq[t] * bt_width;
     int kvh = h / (hq / hkv);
     int lo = attn_first_key(pos, window, ex.chunk);
+    // the keys to visit, numbered 0 .. n_seen - 1: kept first positions before the window, then the window
+    int n_kept = min(ex.keep_first, lo), n_seen = n_kept + pos - lo + 1;
+    auto key_of = [&](int i) { return i < n_kept ? i : lo + i - n_kept; };
     int dv = ex.dv;
     float slope = ex.slopes ? ex.slopes[h] : 0.f;
     const T* qrow = q + ((size_t)t * hq + h) * d;
@@ -84,10 +89,11 @@ attn_generic_kernel(const T* __restrict__ q, T* __restrict__ out, const T* __res
     __syncthreads();
     float m = ex.sink ? (ex.sinks ? ex.sinks[h] : 0.f) : -INFINITY, l = ex.sink ? 1.f : 0.f;
     float acc[AG_MAX_D_PER_THREAD] = {};
-    for (int c0 = lo; c0 <= pos; c0 += AG_BLOCK) {
-        int j = c0 + tid;
+    for (int c0 = 0; c0 < n_seen; c0 += AG_BLOCK) {
+        int j = key_of(c0 + tid);
+        bool seen = c0 + tid < n_seen;
         float s = -INFINITY;
-        if (j <= pos) {
+        if (seen) {
             int page = pages[j / page_size];
             const T* krow = kcache + (((size_t)page * hkv + kvh) * page_size + j % page_size) * d;
             float dot = 0.f;
@@ -98,10 +104,10 @@ attn_generic_kernel(const T* __restrict__ q, T* __restrict__ out, const T* __res
         }
         float m_new = fmaxf(m, ag_block_max(s, red));
         float corr = expf(m - m_new);            // first chunk: exp(-inf) = 0
-        float p = j <= pos ? expf(s - m_new) : 0.f;
+        float p = seen ? expf(s - m_new) : 0.f;
         ps[tid] = p;
         l = l * corr + ag_block_sum(p, red);     // barrier inside also publishes ps
-        int n_keys = min(AG_BLOCK, pos - c0 + 1);
+        int n_keys = min(AG_BLOCK, n_seen - c0);
 #pragma unroll
         for (int r = 0; r < AG_MAX_D_PER_THREAD; ++r) {
             int e = tid + r * AG_BLOCK;
@@ -109,14 +115,14 @@ attn_generic_kernel(const T* __restrict__ q, T* __restrict__ out, const T* __res
             float a = acc[r] * corr;
             if (ex.v_in_k) {
                 for (int jj = 0; jj < n_keys; ++jj) {
-                    int key = c0 + jj;
+                    int key = key_of(c0 + jj);
                     int page = pages[key / page_size];
                     const T* krow = kcache + (((size_t)page * hkv + kvh) * page_size + key % page_size) * d;
                     a = fmaf(ps[jj], Elem<T>::load(krow + e), a);
                 }
             } else {
                 for (int jj = 0; jj < n_keys; ++jj) {
-                    int key = c0 + jj;
+                    int key = key_of(c0 + jj);
                     int page = pages[key / page_size];
                     const T* vcol = vcache + ((size_t)page * hkv + kvh) * dv * page_size + key % page_size;
                     a = fmaf(ps[jj], Elem<T>::load(vcol + (size_t)e * page_size), a);

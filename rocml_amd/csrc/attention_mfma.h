@@ -54,6 +54,8 @@ struct DecodeProj {
     const float* row_ssq; int row_parts; float row_eps; float row_inv_width;
     const float* bias;      // null: none; else one number per column of a projection row, added to the sums
                             // (behind the row scale: the bias is no part of the normed input's product)
+    int rot;                // leading values of a head that are rotated (all of them without EXTRA)
+    int v_is_k;             // the new value is the projected key (before norm and rotation): the rows hold no value columns
 };
 
 // grid (n_splits, Hkv, tokens), 4 or 8 waves; the block's pages are cut into 32-key pieces that the
@@ -75,6 +77,7 @@ struct MaskExtra {
     int sink;               // one more term exp(0) in the softmax's denominator, with no value
     const float* sinks;     // [Hq] or null: with `sink`, the term is exp(sinks[head]) instead
     float softcap;          // > 0: the scaled score s becomes softcap * tanh(s / softcap) before the mask
+    int keep_first;         // > 0 (with a window): the first keep_first positions are seen whatever their distance
 };
 constexpr float AM_LOG2E = 1.4426950408889634f;
 // tanh by one exponential and one reciprocal (both hardware approximations; the kernels here round to bfloat16 anyway)
@@ -126,6 +129,14 @@ attn_decode_mfma_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
     }
     int first_page = lo / AM_PAGE;
     int n_pages = (len + AM_PAGE - 1) / AM_PAGE - first_page;
+    // the pages of kept first positions that lie before the window's come first in the list of pages to visit
+    int keep = 0, kept_pages = 0;
+    if constexpr (EXTRA) {
+        keep = mx.keep_first;
+        kept_pages = min(first_page, (keep + AM_PAGE - 1) / AM_PAGE);
+        n_pages += kept_pages;
+    }
+    auto logical_page = [&](int i) { return EXTRA && i < kept_pages ? i : first_page + i - kept_pages; };
     // split s takes pages s, s + n_splits, ...: the splits of a sequence, which run side by side,
     // then read neighbouring pages at any one time instead of n_splits distant ranges
     int my_pages = split < n_pages ? (n_pages - split + n_splits - 1) / n_splits : 0;
@@ -147,7 +158,7 @@ attn_decode_mfma_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
         if (from_start && round < 4)
             phys = round == 0 ? early[0] : round == 1 ? early[1] : round == 2 ? early[2] : early[3];
         else
-            phys = pages[first_page + split + round * n_splits];
+            phys = pages[logical_page(split + round * n_splits)];
         const bf16_t* kbase = kcache + (((size_t)phys * hkv + kvh) * AM_PAGE + half * 32) * D;
         const bf16_t* vbase = vcache + ((size_t)phys * hkv + kvh) * D * AM_PAGE + half * 32;
 #pragma unroll
@@ -188,7 +199,7 @@ attn_decode_mfma_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
         __shared__ __attribute__((aligned(16))) bf16_t sm_knew[D];
         __shared__ __attribute__((aligned(16))) bf16_t sm_vnew[D];
         int last_lpage = new_pos / AM_PAGE;
-        owner = pj.write_kv && (last_lpage - first_page) % n_splits == split;
+        owner = pj.write_kv && (last_lpage - first_page + kept_pages) % n_splits == split;
         int n_rows = group + (owner ? 2 : 0);       // q heads, then key, then value
         const float* tok = pj.qkv + (size_t)t * pj.ld;
         float row_scale = 1.0f;
@@ -212,7 +223,7 @@ attn_decode_mfma_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
 #pragma unroll
             for (int i = 0; i < 2; ++i) {
                 r[i] = base + i * WAVES + wave;
-                prow[i] = r[i] < group ? kvh * group + r[i] : (r[i] == group ? hq + kvh : hq + hkv + kvh);
+                prow[i] = r[i] < group ? kvh * group + r[i] : (r[i] == group || (EXTRA && pj.v_is_k) ? hq + kvh : hq + hkv + kvh);
                 src[i] = tok + (size_t)(r[i] < n_rows ? prow[i] : 0) * D + lane;
 #pragma unroll
                 for (int j = 0; j < J; ++j)
@@ -253,17 +264,18 @@ attn_decode_mfma_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
             for (int i = 0; i < 2; ++i) {
                 if (r[i] >= n_rows) continue;
                 bool rotate = pj.cos_t != nullptr && r[i] <= group;
-                const float* c = pj.cos_t + (size_t)t * (D / 2);
-                const float* sn = pj.sin_t + (size_t)t * (D / 2);
+                const int rot = EXTRA ? pj.rot : D, half = rot / 2;
+                const float* c = pj.cos_t + (size_t)t * half;
+                const float* sn = pj.sin_t + (size_t)t * half;
                 bf16_t* dst = r[i] < group ? sm_q + r[i] * D : (r[i] == group ? sm_knew : sm_vnew);
                 int phys = pages[last_lpage], in_page = new_pos % AM_PAGE;
 #pragma unroll
                 for (int j = 0; j < J; ++j) {
                     int e = lane + j * 64;
                     float x = val[i][j];
-                    if (rotate) {
-                        if (e < D / 2) x = x * c[e] - sm_f[wave][i][e + D / 2] * sn[e];
-                        else x = sm_f[wave][i][e - D / 2] * sn[e - D / 2] + x * c[e - D / 2];
+                    if (rotate && e < rot) {
+                        if (e < half) x = x * c[e] - sm_f[wave][i][e + half] * sn[e];
+                        else x = sm_f[wave][i][e - half] * sn[e - half] + x * c[e - half];
                     }
                     bf16_t xb = f32_to_bf16(x);
                     dst[e] = xb;
@@ -324,7 +336,7 @@ attn_decode_mfma_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
                 if constexpr (EXTRA) {
                     if (cap_out != 0.f) v = am_tanh(v * cap_in) * cap_out;
                 }
-                v = (key >= from && key < to) ? v : -INFINITY;
+                v = ((key >= from || (EXTRA && key < keep)) && key < to) ? v : -INFINITY;
                 if constexpr (EXTRA) v -= slope_l2 * (float)(len - 1 - key);
                 s[u][i] = v;
                 mx = fmaxf(mx, v);
@@ -358,7 +370,7 @@ attn_decode_mfma_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
     };
     // (FUSED: the new key is not yet in the cache where a block reads it; it comes last, from LDS)
     int cached = (FUSED && owner) ? new_pos : len;
-    auto first_key = [&](int piece) { return (first_page + split + (piece >> 1) * n_splits) * AM_PAGE + (piece & 1) * 32; };
+    auto first_key = [&](int piece) { return logical_page(split + (piece >> 1) * n_splits) * AM_PAGE + (piece & 1) * 32; };
     for (int piece = wave; piece < n_pieces; piece += WAVES * AHEAD) {
         multiply_piece(first_key(piece), lo, cached, kbuf[0], vbuf[0]);
         if (piece + WAVES * AHEAD < n_pieces) request_piece(piece + WAVES * AHEAD, kbuf[0], vbuf[0]);
@@ -638,6 +650,11 @@ attn_prefill_mfma_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
     constexpr int K_PIECES = AM_PAGE * D / 8 / AM_THREADS, V_PIECES = D * AM_PAGE / 8 / AM_THREADS;
     u32x4 kreg[K_PIECES], vreg[V_PIECES];
     int first_page = blk_first_key / AM_PAGE, last_page = blk_last_key / AM_PAGE;
+    // kept first positions: their pages before the window's come first, then the window's
+    const int keep = EXTRA ? mx.keep_first : 0;
+    const int kept_pages = EXTRA ? min(first_page, (keep + AM_PAGE - 1) / AM_PAGE) : 0;
+    auto logical_page = [&](int i) { return EXTRA && i < kept_pages ? i : first_page + i - kept_pages; };
+    const int n_visits = last_page - first_page + 1 + kept_pages;
 #define AM_LOAD_PAGE(lp_)                                                                         \
     {                                                                                             \
         int phys_ = pages[lp_];                                                                   \
@@ -651,8 +668,9 @@ attn_prefill_mfma_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
     int wave_min_pos = pos0 + w_lo;
     int wave_max_lo = am_first_key(pos0 + w_hi, window, chunk);
     bool wave_full = w_hi - w_lo == 31;
-    AM_LOAD_PAGE(first_page)
-    for (int lpage = first_page; lpage <= last_page; ++lpage) {
+    AM_LOAD_PAGE(logical_page(0))
+    for (int visit = 0; visit < n_visits; ++visit) {
+        const int lpage = logical_page(visit);
         __syncthreads();                                // the previous page has been consumed
 #pragma unroll
         for (int i = 0; i < K_PIECES; ++i) {
@@ -672,7 +690,7 @@ attn_prefill_mfma_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
             dst[2] = make_uint2(vreg[i][2], vreg[i][3]);
         }
         __syncthreads();
-        if (lpage < last_page) AM_LOAD_PAGE(lpage + 1)
+        if (visit + 1 < n_visits) AM_LOAD_PAGE(logical_page(visit + 1))
         if (!wave_active) continue;
         // The scores of both 32-key halves are started before either is finished: the softmax of
         // the first half (vector ALU) then runs while the matrix core still multiplies the second,
@@ -684,7 +702,7 @@ attn_prefill_mfma_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
 #pragma unroll
         for (int half = 0; half < 2; ++half) {
             int key0 = page_key0 + half * 32;
-            live[half] = !(key0 > wave_last_key || key0 + 31 < wave_first_key);   // wave-uniform
+            live[half] = !(key0 > wave_last_key || (key0 + 31 < wave_first_key && !(EXTRA && key0 < keep)));   // wave-uniform
             if (!live[half]) continue;
 #pragma unroll
             for (int e = 0; e < 16; ++e) sc[half][e] = 0.f;
@@ -712,7 +730,7 @@ attn_prefill_mfma_kernel(const bf16_t* __restrict__ q, bf16_t* __restrict__ out,
 #pragma unroll
                 for (int e = 0; e < 16; ++e) {
                     int key = key0 + 8 * (e >> 2) + 4 * h2 + (e & 3);
-                    s[e] = (row_ok && key <= my_pos && key >= my_lo) ? s[e] : -INFINITY;
+                    s[e] = (row_ok && key <= my_pos && (key >= my_lo || (EXTRA && key < keep))) ? s[e] : -INFINITY;
                 }
             }
             if constexpr (EXTRA) {

@@ -113,6 +113,23 @@ __device__ __forceinline__ void store4(bf16_t* p, float a, float b, float c, flo
     v.y = (uint32_t)f32_to_bf16(c) | ((uint32_t)f32_to_bf16(d) << 16);
     *(uint2*)p = v;
 }
+template <typename T>
+__device__ __forceinline__ void store4(T* p, float4 v) { store4(p, v.x, v.y, v.z, v.w); }
+__device__ __forceinline__ float4 load4(const float* p) { return *(const float4*)p; }
+__device__ __forceinline__ float4 load4(const bf16_t* p) {
+    uint2 v = *(const uint2*)p;
+    return make_float4(__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16),
+                       __uint_as_float(v.y & 0xffff0000u));
+}
+// the numbers as a value of type T holds them
+template <typename T> __device__ __forceinline__ float rounded(float v);
+template <> __device__ __forceinline__ float rounded<float>(float v) { return v; }
+template <> __device__ __forceinline__ float rounded<bf16_t>(float v) { return bf16_to_f32(f32_to_bf16(v)); }
+template <typename T>
+__device__ __forceinline__ float4 rounded4(float4 v) { return make_float4(rounded<T>(v.x), rounded<T>(v.y), rounded<T>(v.z), rounded<T>(v.w)); }
+__device__ __forceinline__ float4 fma4(float4 a, float4 b, float4 c) {
+    return make_float4(fmaf(a.x, b.x, c.x), fmaf(a.y, b.y, c.y), fmaf(a.z, b.z, c.z), fmaf(a.w, b.w, c.w));
+}
 
 template <typename TO, int RN_VEC>
 __global__ void __launch_bounds__(EW_BLOCK)
@@ -226,6 +243,32 @@ __device__ __forceinline__ float gate_activation(float g, int act) {
     return g / (1.0f + expf(-g));
 }
 
+// out[i] = act(x[i]) without a gate: the activations above, or 4: max(x, 0)^2.
+template <typename TO>
+__global__ void activate_kernel(const float* __restrict__ x, TO* __restrict__ out, long long total, int act) {
+    long long idx = (long long)blockIdx.x * EW_BLOCK + threadIdx.x;
+    if (idx >= total) return;
+    float v = x[idx];
+    if (act == 4) {
+        v = fmaxf(v, 0.f);
+        v *= v;
+    } else {
+        v = gate_activation(v, act);
+    }
+    Elem<TO>::store(out + idx, v);
+}
+
+ROCML_EXPORT int rocml_activate(const float* x, void* out, int out_dtype, long long total, int act, hipStream_t stream) {
+    ROCML_REQUIRE(total >= 0 && x && out && act >= 0 && act <= 4, "activate: bad arguments (activation %d)", act);
+    if (total == 0) return 0;
+    int grid = ceil_div(total, EW_BLOCK);
+    if (out_dtype == ROCML_F32) activate_kernel<float><<<grid, EW_BLOCK, 0, stream>>>(x, (float*)out, total, act);
+    else if (out_dtype == ROCML_BF16) activate_kernel<bf16_t><<<grid, EW_BLOCK, 0, stream>>>(x, (bf16_t*)out, total, act);
+    else return rocml_fail("activate: unknown dtype code %d", out_dtype);
+    ROCML_CHECK_LAUNCH("activate");
+    return 0;
+}
+
 // limit > 0: g is cut off above at limit and u is held inside [-limit, limit] first; up_offset is
 // added to u (after the limit).
 template <typename TI, typename TO>
@@ -320,13 +363,14 @@ __global__ void qk_norm_rope_append_kernel(
     const int* __restrict__ block_table, int bt_width, const int* __restrict__ token_seq,
     const int* __restrict__ token_pos, int page_size, int write_kv, int n_splits, long long split_stride,
     int rows_per_token, int pairing, int first_row, const float* __restrict__ bias, int dv,
-    float qt_coef, int qt_every, const float* __restrict__ span_inv, int span_self) {
+    float qt_coef, int qt_every, const float* __restrict__ span_inv, int span_self, int v_col0) {
+    // v_col0: first value column (behind the q and k rows, or at the first k row: values that are the projected keys).
     // span_inv (may be null): [T, 2], the norm's factor of a token's whole q row and whole k row; the gains then
     // have one number per column of the q (k) projection, and a head takes its own part of them.  span_self: the
     // same norm, but every wave forms its row's factor itself (few tokens: one launch less).
     // qt_coef, qt_every: the queries' stretch with their position (after the norm); every = 0: none.
     // bias (may be null): one number per column of the packed row, added to the projection's sums.
-    // dv: the size of a value head; the value rows start behind the Hq + Hkv rows of d numbers.
+    // dv: the size of a value head.
     extern __shared__ float stage[];   // [QK_WAVES][d]
     int wave = threadIdx.x / WAVE;
     int lane = threadIdx.x & (WAVE - 1);
@@ -337,7 +381,7 @@ __global__ void qk_norm_rope_append_kernel(
     int kind = r < hq ? 0 : (r < hq + hkv ? 1 : 2);   // q, k, v
     if (!write_kv && kind != 0) active = false;
     int width = kind == 2 ? dv : d;
-    size_t col0 = kind == 2 ? (size_t)(hq + hkv) * d + (size_t)(r - hq - hkv) * dv : (size_t)r * d;
+    size_t col0 = kind == 2 ? (size_t)v_col0 + (size_t)(r - hq - hkv) * dv : (size_t)r * d;
     const TI* src = qkv + (size_t)t * ld + col0;
     float v[QK_PER_LANE];
     float ss = 0.f;
@@ -611,7 +655,8 @@ ROCML_EXPORT int rocml_qk_norm_rope_append(
     void* kcache, void* vcache, int out_dtype, const int* block_table, int bt_width,
     const int* token_seq, const int* token_pos, int page_size, int write_kv, int n_splits,
     long long split_stride, const float* bias, int dv, float qt_coef, int qt_every, const float* span_inv, int span_self,
-    hipStream_t stream) {
+    int v_is_k, hipStream_t stream) {
+    // v_is_k: the rows hold no value columns, a value is the projected key before norm and rotation (dv = d)
     // span_self: the norm spans a token's whole q row and whole k row as with span_inv, and the kernel forms the
     // factors itself (a step of few tokens)
     // span_inv (may be null): [T, 2] factors of a norm over a token's whole q row and whole k row (qk_span_stats);
@@ -628,7 +673,9 @@ ROCML_EXPORT int rocml_qk_norm_rope_append(
                   "qk_norm_rope_append: partial sums must be 32-bit with a positive stride");
     ROCML_REQUIRE(d <= QK_MAX_PER_LANE * WAVE, "qk_norm_rope_append: head_dim %d exceeds %d", d,
                   QK_MAX_PER_LANE * WAVE);
-    ROCML_REQUIRE(ld >= (hq + hkv) * d + hkv * dv || (!write_kv && ld >= hq * d),
+    ROCML_REQUIRE(!v_is_k || dv == d, "qk_norm_rope_append: values that are the keys have the keys' size");
+    const int v_col0 = (v_is_k ? hq : hq + hkv) * d;
+    ROCML_REQUIRE(ld >= v_col0 + hkv * dv || (!write_kv && ld >= hq * d),
                   "qk_norm_rope_append: row stride %d too small", ld);
     ROCML_REQUIRE(rot >= 0 && rot <= d && rot % 2 == 0, "qk_norm_rope_append: rot_dim %d must be even and <= %d", rot, d);
     ROCML_REQUIRE(pairing == 0 || pairing == 1, "qk_norm_rope_append: pairing %d (0: halves, 1: neighbours)", pairing);
@@ -663,7 +710,7 @@ ROCML_EXPORT int rocml_qk_norm_rope_append(
     qk_norm_rope_append_kernel<TI, TO, N, LP><<<grid, EW_BLOCK, lds, stream>>>(                 \
         (const TI*)qkv, ld, n_tokens, hq, hkv, d, q_gain, k_gain, eps, cos_t, sin_t, rot,       \
         (TO*)q_out, (TO*)kcache, (TO*)vcache, block_table, bt_width, token_seq, token_pos,      \
-        page_size, write_kv, n_splits, split_stride, rows_per_token, pairing, first_row, bias, dv, qt_coef, qt_every, span_inv, span_self)
+        page_size, write_kv, n_splits, split_stride, rows_per_token, pairing, first_row, bias, dv, qt_coef, qt_every, span_inv, span_self, v_col0)
 #define LAUNCH_ROWS(TI, TO, N)                                                                  \
     qk_norm_rope_rows_kernel<TI, TO, N, MANY><<<grid, EW_BLOCK, 0, stream>>>(                   \
         (const TI*)qkv, ld, n_tokens, hq, hkv, d, q_gain, k_gain, eps, rot ? cos_t : nullptr,   \
@@ -679,7 +726,7 @@ ROCML_EXPORT int rocml_qk_norm_rope_append(
         if (v_tiled) {                                                                          \
             dim3 vgrid(ceil_div(n_tokens, VT_TOKENS), hkv, ceil_div(dv, VT_VALUES));            \
             v_append_tile_kernel<TI, TO><<<vgrid, EW_BLOCK, 0, stream>>>(                       \
-                (const TI*)qkv, ld, n_tokens, (hq + hkv) * d, hkv, dv, (TO*)vcache, block_table,\
+                (const TI*)qkv, ld, n_tokens, v_col0, hkv, dv, (TO*)vcache, block_table,\
                 bt_width, token_seq, token_pos, page_size, bias);                               \
         }                                                                                       \
     }
@@ -830,6 +877,19 @@ __device__ __forceinline__ float block_sum_256(float v, float* scratch) {
     return r;
 }
 
+// Number e of a part whose first `dims` numbers turn: pairs (e, e + dims/2), or with pairing 1 (2i, 2i + 1), by the
+// angle whose cosine and sine stand in c and s.
+__device__ __forceinline__ float turned(const float* __restrict__ v, int e, int dims, int pairing, const float* __restrict__ c,
+                                        const float* __restrict__ s) {
+    if (e >= dims) return v[e];
+    if (pairing == 1) {
+        int i = e >> 1;
+        return (e & 1) ? v[e] * c[i] + v[e - 1] * s[i] : v[e] * c[i] - v[e + 1] * s[i];
+    }
+    int half = dims / 2;
+    return e < half ? v[e] * c[e] - v[e + half] * s[e] : v[e] * c[e - half] + v[e - half] * s[e - half];
+}
+
 template <typename TO>
 __global__ void __launch_bounds__(EW_BLOCK)
 latent_prepare_kernel(const float* __restrict__ proj, int ld, int q_rank, int kv_rank, int rot_part, int dims,
@@ -837,18 +897,19 @@ latent_prepare_kernel(const float* __restrict__ proj, int ld, int q_rank, int kv
                       const float* __restrict__ cos_t, const float* __restrict__ sin_t,
                       TO* __restrict__ cq_out, TO* __restrict__ cache, const int* __restrict__ block_table,
                       int bt_width, const int* __restrict__ token_seq, const int* __restrict__ token_pos,
-                      int page_size, int write_cache) {
+                      int page_size, int write_cache, int pairing) {
     __shared__ float red[EW_BLOCK / WAVE];
     int t = blockIdx.x, tid = threadIdx.x;
     const float* row = proj + (size_t)t * ld;
     float sq = 0.f, sk = 0.f;
     for (int e = tid; e < q_rank; e += EW_BLOCK) sq = fmaf(row[e], row[e], sq);
-    for (int e = tid; e < kv_rank; e += EW_BLOCK) sk = fmaf(row[q_rank + e], row[q_rank + e], sk);
+    if (write_cache)          // (a row may hold the query latent alone: a layer that reads another's rows)
+        for (int e = tid; e < kv_rank; e += EW_BLOCK) sk = fmaf(row[q_rank + e], row[q_rank + e], sk);
     float inv_q = 1.0f / sqrtf(block_sum_256(sq, red) / (float)q_rank + eps);
-    float inv_k = 1.0f / sqrtf(block_sum_256(sk, red) / (float)kv_rank + eps);
     for (int e = tid; e < q_rank; e += EW_BLOCK)
         Elem<TO>::store(cq_out + (size_t)t * q_rank + e, row[e] * inv_q * q_gain[e]);
     if (!write_cache) return;
+    float inv_k = 1.0f / sqrtf(block_sum_256(sk, red) / (float)kv_rank + eps);
     int pos = token_pos[t];
     int page = block_table[(size_t)token_seq[t] * bt_width + pos / page_size];
     if (page < 0) return;
@@ -857,37 +918,30 @@ latent_prepare_kernel(const float* __restrict__ proj, int ld, int q_rank, int kv
         Elem<TO>::store(dst + e, row[q_rank + e] * inv_k * kv_gain[e]);
     const float* kr = row + q_rank + kv_rank;
     int half = dims / 2;
-    for (int e = tid; e < rot_part; e += EW_BLOCK) {
-        float v = kr[e];
-        if (e < half) {
-            float c = cos_t[(size_t)t * half + e], s = sin_t[(size_t)t * half + e];
-            v = kr[e] * c - kr[e + half] * s;
-        } else if (e < dims) {
-            float c = cos_t[(size_t)t * half + e - half], s = sin_t[(size_t)t * half + e - half];
-            v = kr[e] * c + kr[e - half] * s;
-        }
-        Elem<TO>::store(dst + kv_rank + e, v);
-    }
+    for (int e = tid; e < rot_part; e += EW_BLOCK)
+        Elem<TO>::store(dst + kv_rank + e, turned(kr, e, dims, pairing, cos_t + (size_t)t * half, sin_t + (size_t)t * half));
 }
 
 ROCML_EXPORT int rocml_latent_prepare(const float* proj, int ld, int n_tokens, int q_rank, int kv_rank, int rot_part,
                                       int dims, const float* q_gain, const float* kv_gain, float eps,
                                       const float* cos_t, const float* sin_t, void* cq_out, void* cache,
                                       int out_dtype, const int* block_table, int bt_width, const int* token_seq,
-                                      const int* token_pos, int page_size, int write_cache, hipStream_t stream) {
+                                      const int* token_pos, int page_size, int write_cache, int pairing, hipStream_t stream) {
+    // without write_cache only the query latent is read (the rows may hold nothing else)
+    ROCML_REQUIRE(pairing == 0 || pairing == 1, "latent_prepare: pairing %d (0: halves, 1: neighbours)", pairing);
     ROCML_REQUIRE(n_tokens >= 0 && q_rank > 0 && kv_rank > 0 && rot_part >= 0 && dims >= 0 && dims % 2 == 0 && dims <= rot_part,
                   "latent_prepare: bad sizes T=%d q_rank=%d kv_rank=%d rotated part=%d of which %d turn", n_tokens,
                   q_rank, kv_rank, rot_part, dims);
-    ROCML_REQUIRE(ld >= q_rank + kv_rank + rot_part, "latent_prepare: rows of %d numbers, %d are needed", ld,
+    ROCML_REQUIRE(ld >= q_rank + (write_cache ? kv_rank + rot_part : 0), "latent_prepare: rows of %d numbers, %d are needed", ld,
                   q_rank + kv_rank + rot_part);
-    ROCML_REQUIRE(q_gain && kv_gain && cq_out && (dims == 0 || (cos_t && sin_t)), "latent_prepare: gains, tables or output missing");
+    ROCML_REQUIRE(q_gain && (kv_gain || !write_cache) && cq_out && (dims == 0 || (cos_t && sin_t)), "latent_prepare: gains, tables or output missing");
     ROCML_REQUIRE(!write_cache || (cache && block_table && bt_width > 0 && page_size > 0 && token_seq && token_pos),
                   "latent_prepare: cache arguments missing");
     if (n_tokens == 0) return 0;
 #define LAUNCH(TO)                                                                                              \
     latent_prepare_kernel<TO><<<n_tokens, EW_BLOCK, 0, stream>>>(proj, ld, q_rank, kv_rank, rot_part, dims,    \
         q_gain, kv_gain, eps, cos_t, sin_t, (TO*)cq_out, (TO*)cache, block_table, bt_width, token_seq,         \
-        token_pos, page_size, write_cache)
+        token_pos, page_size, write_cache, pairing)
     if (out_dtype == ROCML_F32) LAUNCH(float);
     else if (out_dtype == ROCML_BF16) LAUNCH(bf16_t);
     else return rocml_fail("latent_prepare: unknown dtype code %d", out_dtype);
@@ -904,7 +958,7 @@ template <typename TO>
 __global__ void rope_heads_kernel(const float* __restrict__ q, int ldq, int head_stride, int offset, int rot_part,
                                   int dims, const float* __restrict__ cos_t, const float* __restrict__ sin_t,
                                   TO* __restrict__ out, int ldo, int out_stride, int out_offset, int n_heads,
-                                  int lead, long long total) {
+                                  int lead, long long total, int pairing) {
     long long idx = (long long)blockIdx.x * EW_BLOCK + threadIdx.x;
     if (idx >= total) return;
     int width = lead + rot_part;
@@ -918,19 +972,15 @@ __global__ void rope_heads_kernel(const float* __restrict__ q, int ldq, int head
         return;
     }
     int half = dims / 2;
-    float v = src[e];
-    if (e < half) {
-        v = src[e] * cos_t[t * half + e] - src[e + half] * sin_t[t * half + e];
-    } else if (e < dims) {
-        v = src[e] * cos_t[t * half + e - half] + src[e - half] * sin_t[t * half + e - half];
-    }
+    float v = turned(src, e, dims, pairing, cos_t + t * half, sin_t + t * half);
     Elem<TO>::store(out + (size_t)t * ldo + (size_t)h * out_stride + out_offset + lead + e, v);
 }
 
 ROCML_EXPORT int rocml_rope_heads(const float* q, int ldq, int head_stride, int offset, int rot_part, int dims,
                                   const float* cos_t, const float* sin_t, void* out, int out_dtype, int ldo,
-                                  int out_stride, int out_offset, int n_tokens, int n_heads, int lead,
+                                  int out_stride, int out_offset, int n_tokens, int n_heads, int lead, int pairing,
                                   hipStream_t stream) {
+    ROCML_REQUIRE(pairing == 0 || pairing == 1, "rope_heads: pairing %d (0: halves, 1: neighbours)", pairing);
     ROCML_REQUIRE(n_tokens >= 0 && n_heads > 0 && rot_part >= 0 && dims >= 0 && dims % 2 == 0 && dims <= rot_part,
                   "rope_heads: bad sizes T=%d H=%d part=%d dims=%d", n_tokens, n_heads, rot_part, dims);
     ROCML_REQUIRE(lead >= 0 && offset >= lead && offset + rot_part <= head_stride && ldq >= n_heads * head_stride &&
@@ -942,10 +992,10 @@ ROCML_EXPORT int rocml_rope_heads(const float* q, int ldq, int head_stride, int 
     int grid = ceil_div(total, EW_BLOCK);
     if (out_dtype == ROCML_F32)
         rope_heads_kernel<float><<<grid, EW_BLOCK, 0, stream>>>(q, ldq, head_stride, offset, rot_part, dims, cos_t, sin_t,
-                                                                (float*)out, ldo, out_stride, out_offset, n_heads, lead, total);
+                                                                (float*)out, ldo, out_stride, out_offset, n_heads, lead, total, pairing);
     else if (out_dtype == ROCML_BF16)
         rope_heads_kernel<bf16_t><<<grid, EW_BLOCK, 0, stream>>>(q, ldq, head_stride, offset, rot_part, dims, cos_t, sin_t,
-                                                                 (bf16_t*)out, ldo, out_stride, out_offset, n_heads, lead, total);
+                                                                 (bf16_t*)out, ldo, out_stride, out_offset, n_heads, lead, total, pairing);
     else return rocml_fail("rope_heads: unknown dtype code %d", out_dtype);
     ROCML_CHECK_LAUNCH("rope_heads");
     return 0;
@@ -1074,9 +1124,10 @@ ROCML_EXPORT int rocml_latent_window_gather(const void* cache, int dtype, int ro
 
 // out[t, h * n + i] = x[t, h * x_stride + i] * sigmoid(g[t, h * n + i]) (g null: a plain copy of the heads'
 // leading n numbers): the heads of an attention output that is wider than the values, gated and packed.
+// gate_one: one gate number per head, g[t, h], instead of one per value.
 template <typename T>
 __global__ void gate_heads_kernel(const T* __restrict__ x, int ldx, int x_stride, const float* __restrict__ g, int ldg,
-                                  T* __restrict__ out, int n_heads, int n, long long total) {
+                                  T* __restrict__ out, int n_heads, int n, long long total, int gate_one) {
     long long idx = (long long)blockIdx.x * EW_BLOCK + threadIdx.x;
     if (idx >= total) return;
     int i = (int)(idx % n);
@@ -1084,19 +1135,20 @@ __global__ void gate_heads_kernel(const T* __restrict__ x, int ldx, int x_stride
     int h = (int)(th % n_heads);
     long long t = th / n_heads;
     float v = Elem<T>::load(x + (size_t)t * ldx + (size_t)h * x_stride + i);
-    if (g) v *= 1.0f / (1.0f + expf(-g[(size_t)t * ldg + (size_t)h * n + i]));
+    if (g) v *= 1.0f / (1.0f + expf(-g[(size_t)t * ldg + (gate_one ? (size_t)h : (size_t)h * n + i)]));
     Elem<T>::store(out + idx, v);
 }
 
 ROCML_EXPORT int rocml_gate_heads(const void* x, int dtype, int ldx, int x_stride, const float* g, int ldg, void* out,
-                                  int n_rows, int n_heads, int n, hipStream_t stream) {
-    ROCML_REQUIRE(n_rows >= 0 && n_heads > 0 && n > 0 && n <= x_stride && ldx >= n_heads * x_stride && (!g || ldg >= n_heads * n),
+                                  int n_rows, int n_heads, int n, int gate_one, hipStream_t stream) {
+    ROCML_REQUIRE(n_rows >= 0 && n_heads > 0 && n > 0 && n <= x_stride && ldx >= n_heads * x_stride &&
+                      (!g || ldg >= n_heads * (gate_one ? 1 : n)),
                   "gate_heads: bad sizes rows=%d heads=%d n=%d stride=%d", n_rows, n_heads, n, x_stride);
     long long total = (long long)n_rows * n_heads * n;
     if (total == 0) return 0;
     int grid = ceil_div(total, EW_BLOCK);
-    if (dtype == ROCML_F32) gate_heads_kernel<float><<<grid, EW_BLOCK, 0, stream>>>((const float*)x, ldx, x_stride, g, ldg, (float*)out, n_heads, n, total);
-    else if (dtype == ROCML_BF16) gate_heads_kernel<bf16_t><<<grid, EW_BLOCK, 0, stream>>>((const bf16_t*)x, ldx, x_stride, g, ldg, (bf16_t*)out, n_heads, n, total);
+    if (dtype == ROCML_F32) gate_heads_kernel<float><<<grid, EW_BLOCK, 0, stream>>>((const float*)x, ldx, x_stride, g, ldg, (float*)out, n_heads, n, total, gate_one);
+    else if (dtype == ROCML_BF16) gate_heads_kernel<bf16_t><<<grid, EW_BLOCK, 0, stream>>>((const bf16_t*)x, ldx, x_stride, g, ldg, (bf16_t*)out, n_heads, n, total, gate_one);
     else return rocml_fail("gate_heads: unknown dtype code %d", dtype);
     ROCML_CHECK_LAUNCH("gate_heads");
     return 0;
@@ -1324,17 +1376,43 @@ norm_add_kernel(float* __restrict__ x, float* __restrict__ y, const float* __res
 
 // The same for rows of up to 8192 values that are a multiple of 4: the row stays in registers and all
 // loads are issued at once.
-template <typename TC, bool LAYER, int VEC>
+// TAPS > 0 (steps of one token per sequence, with next_gain): what reads the next norm's output is first replaced by
+// itself plus its causal convolution over the sequence (see added_conv below); row b is sequence b's one token, and the
+// kept rows of its slot move up by one.
+struct NextConv {
+    const float* w;             // [taps, n]
+    void* state;                // [slot, taps - 1, n] in copy's type
+    const int* slots;           // [rows]
+};
+
+template <typename TC, bool LAYER, int VEC, int TAPS = 0>
 __global__ void __launch_bounds__(EW_BLOCK)
 norm_add_vec_kernel(float* __restrict__ x, const float* __restrict__ y, const float* __restrict__ gain,
                     const float* __restrict__ bias, float eps, int n, TC* __restrict__ copy,
                     const float* __restrict__ partials, int n_splits, long long split_stride, int replace,
-                    const float* __restrict__ next_gain, float next_eps) {
+                    const float* __restrict__ next_gain, float next_eps, NextConv cv = NextConv{}) {
     __shared__ float scratch[EW_BLOCK / WAVE];
     size_t row = (size_t)blockIdx.x * n;
     int nv = n / 4;
     const float4 zero4 = make_float4(0.f, 0.f, 0.f, 0.f);
     float4 yv[VEC], xv[VEC], gv[VEC], bv[VEC];
+    constexpr int KEPT = TAPS > 1 ? TAPS - 1 : 1;
+    float4 kept[KEPT][VEC], tap[TAPS > 0 ? TAPS : 1][VEC];
+    TC* state_row = nullptr;
+    if constexpr (TAPS > 0) {
+        // (asked for beside the row's own numbers; they do not depend on it)
+        state_row = (TC*)cv.state + (size_t)cv.slots[blockIdx.x] * (TAPS - 1) * n;
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) {
+            int i = threadIdx.x + j * EW_BLOCK;
+            bool ok = i < nv;
+#pragma unroll
+            for (int k = 0; k < TAPS; ++k) {
+                tap[k][j] = ok ? ((const float4*)(cv.w + (size_t)k * n))[i] : zero4;
+                if (k < TAPS - 1) kept[k][j] = ok ? load4(state_row + (size_t)k * n + 4 * (size_t)i) : zero4;
+            }
+        }
+    }
 #pragma unroll
     for (int j = 0; j < VEC; ++j) {
         int i = threadIdx.x + j * EW_BLOCK;
@@ -1399,7 +1477,18 @@ norm_add_vec_kernel(float* __restrict__ x, const float* __restrict__ y, const fl
             int i = threadIdx.x + j * EW_BLOCK;
             if (i >= nv) continue;
             float4 g2 = ((const float4*)next_gain)[i];
-            store4(copy + row + 4 * (size_t)i, xv[j].x * inv2 * g2.x, xv[j].y * inv2 * g2.y, xv[j].z * inv2 * g2.z, xv[j].w * inv2 * g2.w);
+            float4 h = make_float4(xv[j].x * inv2 * g2.x, xv[j].y * inv2 * g2.y, xv[j].z * inv2 * g2.z, xv[j].w * inv2 * g2.w);
+            if constexpr (TAPS > 0) {
+                h = rounded4<TC>(h);
+#pragma unroll
+                for (int k = 0; k < TAPS - 1; ++k)
+                    store4(state_row + (size_t)k * n + 4 * (size_t)i, k + 1 < TAPS - 1 ? kept[k + 1 < KEPT ? k + 1 : 0][j] : h);
+                float4 a = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+                for (int k = 0; k < TAPS; ++k) a = fma4(tap[k][j], k < TAPS - 1 ? kept[k < KEPT ? k : 0][j] : h, a);
+                h.x += a.x; h.y += a.y; h.z += a.z; h.w += a.w;
+            }
+            store4(copy + row + 4 * (size_t)i, h.x, h.y, h.z, h.w);
         }
     }
 }
@@ -1407,13 +1496,25 @@ norm_add_vec_kernel(float* __restrict__ x, const float* __restrict__ y, const fl
 template <typename TC, bool LAYER>
 static void launch_norm_add(float* x, float* y, const float* gain, const float* bias, float eps, int n_rows, int n,
                             TC* copy, const float* partials, int n_splits, long long split_stride, int replace,
-                            const float* next_gain, float next_eps, hipStream_t stream) {
+                            const float* next_gain, float next_eps, const NextConv& cv, int taps, hipStream_t stream) {
     bool vec = n % 4 == 0 && n <= 4 * EW_BLOCK * RN_MAX_VEC && (uintptr_t)x % 16 == 0 && (uintptr_t)y % 16 == 0 &&
                (uintptr_t)gain % 16 == 0 && (!bias || (uintptr_t)bias % 16 == 0) && (!copy || (uintptr_t)copy % 8 == 0) &&
                (!next_gain || (uintptr_t)next_gain % 16 == 0) &&
                (n_splits == 0 || ((uintptr_t)partials % 16 == 0 && split_stride % 4 == 0));
     int v = ceil_div(n / 4, EW_BLOCK);
 #define NAV(V_) norm_add_vec_kernel<TC, LAYER, V_><<<n_rows, EW_BLOCK, 0, stream>>>(x, y, gain, bias, eps, n, copy, partials, n_splits, split_stride, replace, next_gain, next_eps)
+    if constexpr (!LAYER) {
+        if (taps > 0) {         // (the caller asked norm_add_conv_fits and checked the alignment)
+#define NAC(V_, T_) norm_add_vec_kernel<TC, false, V_, T_><<<n_rows, EW_BLOCK, 0, stream>>>(x, y, gain, bias, eps, n, copy, partials, n_splits, split_stride, replace, next_gain, next_eps, cv)
+#define NAC_BY_TAPS(V_) { if (taps == 2) NAC(V_, 2); else if (taps == 3) NAC(V_, 3); else NAC(V_, 4); }
+            if (v <= 1) NAC_BY_TAPS(1)
+            else if (v <= 2) NAC_BY_TAPS(2)
+            else NAC_BY_TAPS(4)
+#undef NAC_BY_TAPS
+#undef NAC
+            return;
+        }
+    }
     if (!vec) norm_add_kernel<TC, LAYER><<<n_rows, EW_BLOCK, 0, stream>>>(x, y, gain, bias, eps, n, copy, partials, n_splits, split_stride, replace, next_gain, next_eps);
     else if (v <= 1) NAV(1);
     else if (v <= 2) NAV(2);
@@ -1536,9 +1637,21 @@ ROCML_EXPORT int rocml_norm_add_branches(float* x, const float* y0, const float*
     return 0;
 }
 
+// Whether norm_add also forms the convolution of the next norm's output (rows in registers, 2 to 4 taps).
+ROCML_EXPORT int rocml_norm_add_conv_fits(int n, int taps) { return n > 0 && n % 4 == 0 && n <= 4 * EW_BLOCK * 4 && taps >= 2 && taps <= 4; }
+
 ROCML_EXPORT int rocml_norm_add(float* x, float* y, int n_rows, int n, const float* gain, const float* bias,
                                 float eps, int layer, void* copy, int copy_dtype, const float* partials, int n_splits,
-                                long long split_stride, int replace, const float* next_gain, float next_eps, hipStream_t stream) {
+                                long long split_stride, int replace, const float* next_gain, float next_eps,
+                                const float* conv_w, void* conv_state, int conv_slots_n, const int* conv_slots, int taps,
+                                hipStream_t stream) {
+    // conv_w (may be null; needs next_gain): [taps, n]; the next norm's output h is replaced by h + its causal convolution,
+    // every row being the one token of a sequence whose kept rows are conv_state [conv_slots_n, taps - 1, n] (copy's type)
+    // at conv_slots [rows]
+    NextConv cv{conv_w, conv_state, conv_slots};
+    if (!conv_w) taps = 0;
+    ROCML_REQUIRE(taps == 0 || (next_gain && conv_state && conv_slots && conv_slots_n > 0 && !layer && rocml_norm_add_conv_fits(n, taps)),
+                  "norm_add: a convolution of the next norm's output needs that norm, the kept rows and sizes it fits (n=%d taps=%d)", n, taps);
     // next_gain (may be null; needs copy): copy gets the new x normed, x / sqrt(mean(x^2) + next_eps) * next_gain
     ROCML_REQUIRE(!next_gain || copy, "norm_add: the next norm's output needs a place");
     // layer = 1: layer norm (mean taken off, bias added if given); 0: root-mean-square norm (bias is not read)
@@ -1549,13 +1662,19 @@ ROCML_EXPORT int rocml_norm_add(float* x, float* y, int n_rows, int n, const flo
                   "norm_add: %d partial sums with a stride of %lld do not fit", n_splits, split_stride);
     ROCML_REQUIRE(!copy || copy_dtype == ROCML_F32 || copy_dtype == ROCML_BF16, "norm_add: unknown dtype code %d", copy_dtype);
     if (n_rows == 0) return 0;
+    if (taps > 0) {
+        const void* ptrs[] = {x, y, gain, next_gain, conv_w, partials};
+        for (const void* q : ptrs) ROCML_REQUIRE((uintptr_t)q % 16 == 0, "norm_add: operands must start on 16 bytes");
+        ROCML_REQUIRE((uintptr_t)copy % 16 == 0 && (uintptr_t)conv_state % 16 == 0 && (n_splits == 0 || split_stride % 4 == 0),
+                      "norm_add: operands must start on 16 bytes");
+    }
     bool half = copy && copy_dtype == ROCML_BF16;
     if (layer) {
-        if (half) launch_norm_add<bf16_t, true>(x, y, gain, bias, eps, n_rows, n, (bf16_t*)copy, partials, n_splits, split_stride, replace, next_gain, next_eps, stream);
-        else launch_norm_add<float, true>(x, y, gain, bias, eps, n_rows, n, (float*)copy, partials, n_splits, split_stride, replace, next_gain, next_eps, stream);
+        if (half) launch_norm_add<bf16_t, true>(x, y, gain, bias, eps, n_rows, n, (bf16_t*)copy, partials, n_splits, split_stride, replace, next_gain, next_eps, cv, taps, stream);
+        else launch_norm_add<float, true>(x, y, gain, bias, eps, n_rows, n, (float*)copy, partials, n_splits, split_stride, replace, next_gain, next_eps, cv, taps, stream);
     } else {
-        if (half) launch_norm_add<bf16_t, false>(x, y, gain, nullptr, eps, n_rows, n, (bf16_t*)copy, partials, n_splits, split_stride, replace, next_gain, next_eps, stream);
-        else launch_norm_add<float, false>(x, y, gain, nullptr, eps, n_rows, n, (float*)copy, partials, n_splits, split_stride, replace, next_gain, next_eps, stream);
+        if (half) launch_norm_add<bf16_t, false>(x, y, gain, nullptr, eps, n_rows, n, (bf16_t*)copy, partials, n_splits, split_stride, replace, next_gain, next_eps, cv, taps, stream);
+        else launch_norm_add<float, false>(x, y, gain, nullptr, eps, n_rows, n, (float*)copy, partials, n_splits, split_stride, replace, next_gain, next_eps, cv, taps, stream);
     }
     ROCML_CHECK_LAUNCH("norm_add");
     return 0;
@@ -1715,5 +1834,155 @@ ROCML_EXPORT int rocml_row_gate_add(float* x, const float* y, const float* g, in
     if (total == 0) return 0;
     row_gate_add_kernel<<<ceil_div(total, EW_BLOCK), EW_BLOCK, 0, stream>>>(x, y, g, ldg, n, total);
     ROCML_CHECK_LAUNCH("row_gate_add");
+    return 0;
+}
+
+// ---- input plus its causal convolution ---------------------------------------------------------
+// out_t = h_t + sum_j w[j, :] h_(t - taps + 1 + j) per channel, the sums 32-bit: h and out [T, n] in one type, w
+// [taps, n] 32-bit.  Before a sequence's first token of the step stand its kept rows, state [slot, taps - 1, n] in h's
+// type (its last taps - 1 inputs, oldest first; zeros at its start).  A block column takes W neighbouring channels per
+// thread and a run of AC_RUN consecutive tokens of one sequence, and slides over them, so an input is read once (and
+// taps - 1 times more at the run's start).  Only the first run of a sequence reads the kept rows (a run is longer than
+// they are), and the same thread replaces them when it is done with them.
+constexpr int AC_RUN = 16, AC_MAX_TAPS = 8;
+
+template <typename T, int W> struct AcPiece;
+template <> struct AcPiece<float, 4> { typedef float4 type; };
+template <> struct AcPiece<bf16_t, 8> { typedef uint4 type; };
+template <> struct AcPiece<float, 1> { typedef float type; };
+template <> struct AcPiece<bf16_t, 1> { typedef bf16_t type; };
+
+template <typename T, int W>
+__device__ __forceinline__ void ac_load(float (&v)[W], const T* p) {
+    typedef typename AcPiece<T, W>::type piece_t;
+    piece_t raw = *(const piece_t*)p;
+    const T* r = (const T*)&raw;
+#pragma unroll
+    for (int i = 0; i < W; ++i) v[i] = Elem<T>::load(r + i);
+}
+template <typename T, int W>
+__device__ __forceinline__ void ac_store(T* p, const float (&v)[W]) {
+    typedef typename AcPiece<T, W>::type piece_t;
+    piece_t raw;
+    T* r = (T*)&raw;
+#pragma unroll
+    for (int i = 0; i < W; ++i) Elem<T>::store(r + i, v[i]);
+    *(piece_t*)p = raw;
+}
+
+template <typename T, int W, int TAPS>
+__global__ void __launch_bounds__(EW_BLOCK)
+added_conv_kernel(const T* __restrict__ h, T* __restrict__ out, int n, const float* __restrict__ w, T* __restrict__ state,
+                  const int* __restrict__ cu_seqlens, const int* __restrict__ seq_slots, int n_seqs) {
+    int c = (blockIdx.y * EW_BLOCK + threadIdx.x) * W;
+    int run = blockIdx.x, b = 0, first = 0, count = 0;
+    if (gridDim.x == (unsigned)n_seqs) {         // a run per sequence (a step of one token each, or short prompts)
+        b = run;
+        run = 0;
+        first = cu_seqlens[b];
+        count = cu_seqlens[b + 1] - first;
+    } else {
+        for (; b < n_seqs; ++b) {
+            first = cu_seqlens[b];
+            count = cu_seqlens[b + 1] - first;
+            int runs = (count + AC_RUN - 1) / AC_RUN;
+            if (run < runs) break;
+            run -= runs;
+        }
+        if (b >= n_seqs) return;
+    }
+    if (c >= n) return;
+    int t0 = run * AC_RUN, t1 = min(count, t0 + AC_RUN);         // the run, in tokens of the sequence's part of the step
+    constexpr int KEPT = TAPS - 1;
+    float tap[TAPS][W], past[KEPT > 0 ? KEPT : 1][W];
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+        for (int i = 0; i < W; ++i) tap[j][i] = w[(size_t)j * n + c + i];
+    T* kept = state + (size_t)seq_slots[b] * KEPT * n + c;
+#pragma unroll
+    for (int j = 0; j < KEPT; ++j) {
+        if (t0 == 0) ac_load<T, W>(past[j], kept + (size_t)j * n);
+        else ac_load<T, W>(past[j], h + (size_t)(first + t0 - KEPT + j) * n + c);
+    }
+    if (KEPT > 0 && t0 == 0) {
+        // the rows kept for the next step: the last of this step's, behind old ones where it brings fewer
+#pragma unroll
+        for (int j = 0; j < KEPT; ++j) {
+            int src = count - KEPT + j;
+            float v[W];
+            if (src >= 0) {
+                ac_load<T, W>(v, h + (size_t)(first + src) * n + c);
+            } else {
+#pragma unroll
+                for (int k = 0; k < KEPT; ++k)
+                    if (k == KEPT + src) {
+#pragma unroll
+                        for (int i = 0; i < W; ++i) v[i] = past[k][i];
+                    }
+            }
+            ac_store<T, W>(kept + (size_t)j * n, v);
+        }
+    }
+    for (int t = t0; t < t1; ++t) {
+        float cur[W], y[W];
+        size_t at = (size_t)(first + t) * n + c;
+        ac_load<T, W>(cur, h + at);
+#pragma unroll
+        for (int i = 0; i < W; ++i) {
+            float a = 0.f;
+#pragma unroll
+            for (int j = 0; j < KEPT; ++j) a = fmaf(tap[j][i], past[j][i], a);
+            a = fmaf(tap[KEPT][i], cur[i], a);
+            y[i] = cur[i] + a;
+#pragma unroll
+            for (int j = 0; j + 1 < KEPT; ++j) past[j][i] = past[j + 1][i];
+            if (KEPT > 0) past[KEPT > 0 ? KEPT - 1 : 0][i] = cur[i];
+        }
+        ac_store<T, W>(out + at, y);
+    }
+}
+
+template <typename T, int W>
+static int launch_added_conv(const T* h, T* out, int n, const float* w, T* state, const int* cu_seqlens, const int* seq_slots,
+                             int n_seqs, int runs, int taps, hipStream_t stream) {
+    int per_row = n / W;
+    dim3 grid(runs, ceil_div(per_row, EW_BLOCK));
+    int threads = per_row >= EW_BLOCK ? EW_BLOCK : (per_row + WAVE - 1) / WAVE * WAVE;
+    if (threads < EW_BLOCK) grid.y = 1;
+#define AC(T_) case T_: added_conv_kernel<T, W, T_><<<grid, threads, 0, stream>>>(h, out, n, w, state, cu_seqlens, seq_slots, n_seqs); break
+    switch (taps) {
+        AC(1); AC(2); AC(3); AC(4); AC(5); AC(6); AC(7); AC(8);
+        default: return rocml_fail("added_conv: %d taps (1 to %d)", taps, AC_MAX_TAPS);
+    }
+#undef AC
+    return 0;
+}
+
+// q_counts (host): tokens each sequence brings.
+ROCML_EXPORT int rocml_added_conv(const void* h, void* out, int dtype, int n_tokens, int n, const float* w, int taps, void* state,
+                                  int n_slots, const int* cu_seqlens, const int* seq_slots, int n_seqs, const int* q_counts,
+                                  hipStream_t stream) {
+    ROCML_REQUIRE(n_tokens >= 0 && n > 0 && n_seqs >= 0 && taps >= 1 && taps <= AC_MAX_TAPS, "added_conv: bad sizes T=%d n=%d taps=%d",
+                  n_tokens, n, taps);
+    ROCML_REQUIRE(h && out && h != out && w && cu_seqlens && seq_slots && q_counts && (taps == 1 || (state && n_slots > 0)),
+                  "added_conv: missing arguments (the output needs a place of its own)");
+    if (n_tokens == 0 || n_seqs == 0) return 0;
+    long long runs = 0, counted = 0;
+    for (int b = 0; b < n_seqs; ++b) {
+        ROCML_REQUIRE(q_counts[b] >= 1, "added_conv: sequence %d brings %d tokens", b, q_counts[b]);
+        runs += (q_counts[b] + AC_RUN - 1) / AC_RUN;
+        counted += q_counts[b];
+    }
+    ROCML_REQUIRE(counted == n_tokens && runs < (1ll << 31), "added_conv: the sequences bring %lld tokens, the step has %d", counted, n_tokens);
+    bool aligned = (((uintptr_t)h | (uintptr_t)out | (uintptr_t)state) & 15) == 0;
+    int rc;
+#define AC_GO(T, W) rc = launch_added_conv<T, W>((const T*)h, (T*)out, n, w, (T*)state, cu_seqlens, seq_slots, n_seqs, (int)runs, taps, stream)
+    if (dtype == ROCML_F32) { if (aligned && n % 4 == 0) AC_GO(float, 4); else AC_GO(float, 1); }
+    else if (dtype == ROCML_BF16) { if (aligned && n % 8 == 0) AC_GO(bf16_t, 8); else AC_GO(bf16_t, 1); }
+    else return rocml_fail("added_conv: unknown dtype code %d", dtype);
+#undef AC_GO
+    if (rc) return rc;
+    ROCML_CHECK_LAUNCH("added_conv");
     return 0;
 }

@@ -503,7 +503,7 @@ ROCML_EXPORT int rocml_gemm_residual_prescale_pays(int m, int n, int k) {
 // 256x192, 128x192, 256x96 and 64x256 tiles.
 // accumulate: out += product (out must be 32-bit); this is the residual sum's epilogue.
 // epilogue: 0 = none; 1 = gated activation: W's rows are (gate_j, up_j) pairs and out is
-//   [M, N/2] = silu(gate) * up.
+//   [M, N/2] = silu(gate) * up; 2 = the same with max(gate, 0) * up; 3 = max(sum, 0)^2, bfloat16.
 // defer: if the product was split along K, leave the partial sums [splits][M][N] at the start of
 //   the workspace and report their number in *deferred_splits (0 if the product is complete);
 //   the caller's next kernel adds them.  Needs a dense out (ldo == N).
@@ -522,7 +522,10 @@ ROCML_EXPORT int rocml_gemm(const void* x, int x_dtype, int ldx, const void* w, 
     if (deferred_splits) *deferred_splits = 0;
     ROCML_REQUIRE(m >= 0 && n > 0 && k > 0, "gemm: bad sizes M=%d N=%d K=%d", m, n, k);
     bool gated = epilogue == 1 || epilogue == 2;        // 1: silu(gate) * up, 2: max(gate, 0) * up
-    ROCML_REQUIRE(epilogue >= 0 && epilogue <= 2, "gemm: unknown epilogue %d", epilogue);
+    bool relu2 = epilogue == 3;                         // max(sum, 0)^2
+    ROCML_REQUIRE(epilogue >= 0 && epilogue <= 3, "gemm: unknown epilogue %d", epilogue);
+    ROCML_REQUIRE(!relu2 || (!accumulate && !defer && x_dtype == ROCML_BF16 && out_dtype == ROCML_BF16),
+                  "gemm: the squared-rectifier epilogue stores whole sums of bfloat16 operands as bfloat16");
     ROCML_REQUIRE(!gated || (n % 2 == 0 && !accumulate), "gemm: the gated epilogue needs an even N and no accumulation");
     int out_cols = gated ? n / 2 : n;
     ROCML_REQUIRE(ldx >= k && ldw >= k && ldo >= out_cols, "gemm: row strides (%d, %d, %d) below (K, K, N)",
@@ -542,7 +545,7 @@ ROCML_EXPORT int rocml_gemm(const void* x, int x_dtype, int ldx, const void* w, 
     if (algo == ALGO_MFMA_KPAR)
         ROCML_REQUIRE(m <= 16, "gemm: the 16-rows kernel takes at most 16 rows, got %d", m);
     ROCML_REQUIRE(out_dtype == ROCML_F32 || out_dtype == ROCML_BF16, "gemm: unknown output type %d", out_dtype);
-    int epi = gated ? (epilogue == 2 ? EPI_RELUGLU : EPI_SWIGLU) : accumulate ? EPI_ACC : (out_dtype == ROCML_BF16 ? EPI_BF16 : EPI_F32);
+    int epi = relu2 ? EPI_RELU2 : gated ? (epilogue == 2 ? EPI_RELUGLU : EPI_SWIGLU) : accumulate ? EPI_ACC : (out_dtype == ROCML_BF16 ? EPI_BF16 : EPI_F32);
     bool use_mfma = mfma_ok && algo != ALGO_PLAIN;
     if (row_ssq)
         ROCML_REQUIRE(gated && m <= 16 && use_mfma && row_parts > 0 && row_eps > 0.f &&
@@ -565,6 +568,7 @@ ROCML_EXPORT int rocml_gemm(const void* x, int x_dtype, int ldx, const void* w, 
         (epi == EPI_F32 ? fn<EPI_F32>(__VA_ARGS__)                   \
          : epi == EPI_BF16 ? fn<EPI_BF16>(__VA_ARGS__)               \
          : epi == EPI_ACC ? fn<EPI_ACC>(__VA_ARGS__)                 \
+         : epi == EPI_RELU2 ? fn<EPI_RELU2>(__VA_ARGS__)             \
          : epi == EPI_RELUGLU ? fn<EPI_RELUGLU>(__VA_ARGS__) : fn<EPI_SWIGLU>(__VA_ARGS__))
         // One or two rows (but not the gated product, which has its own choice of blocks): the
         // kernel whose waves split K, unless the output is narrow (fewer than
@@ -587,6 +591,7 @@ ROCML_EXPORT int rocml_gemm(const void* x, int x_dtype, int ldx, const void* w, 
         ROCML_CHECK_LAUNCH("gemm");
         return 0;
     }
+    ROCML_REQUIRE(!relu2, "gemm: the squared-rectifier epilogue goes with the matrix-core kernels (K and row strides multiples of 8)");
     // plain kernel; the gated epilogue runs as a second kernel over a 32-bit product in the workspace
     void* dst = out;
     int dst_ld = ldo, dst_dtype = out_dtype;
@@ -624,15 +629,16 @@ ROCML_EXPORT int rocml_gemm(const void* x, int x_dtype, int ldx, const void* w, 
 // are column ranges of wider matrices, w is [batch, N, K]).  32-bit accumulation by fused
 // multiply-add in K order for every type; x may be 32-bit while w is bfloat16.
 // gate (may be null): 32-bit [M, ldg] with the heads side by side, batch_g apart: out = product * sigmoid(gate).
+// gate_one: one gate number per head instead of one per column.
 ROCML_EXPORT int rocml_gemm_batched(const void* x, int x_dtype, int ldx, long long batch_x, const void* w, int w_dtype,
                                     int ldw, long long batch_w, void* out, int out_dtype, int ldo, long long batch_o,
                                     int batch, int m, int n, int k, const float* gate, int ldg, long long batch_g,
-                                    hipStream_t stream) {
+                                    int gate_one, hipStream_t stream) {
     ROCML_REQUIRE(batch > 0 && batch < 65536 && m >= 0 && n > 0 && k > 0, "gemm_batched: bad sizes batch=%d M=%d N=%d K=%d", batch, m, n, k);
     ROCML_REQUIRE(ldx >= k && ldw >= k && ldo >= n && batch_x >= 0 && batch_w >= 0 && batch_o >= 0,
                   "gemm_batched: row strides (%d, %d, %d) below (K, K, N) or a negative batch stride", ldx, ldw, ldo);
     ROCML_REQUIRE(ceil_div(m, GT_BM) < 65536, "gemm_batched: too many rows %d", m);
-    ROCML_REQUIRE(!gate || ldg >= n, "gemm_batched: gate rows of %d numbers for N=%d", ldg, n);
+    ROCML_REQUIRE(!gate || ldg >= (gate_one ? 1 : n), "gemm_batched: gate rows of %d numbers for N=%d", ldg, n);
     if (m == 0) return 0;
     // The matrix cores: bfloat16 weights [batch, N, K] without gaps, operands that 16-byte loads reach.
     int x_align = x_dtype == ROCML_F32 ? 4 : 8;
@@ -643,9 +649,9 @@ ROCML_EXPORT int rocml_gemm_batched(const void* x, int x_dtype, int ldx, long lo
         dim3 grid(few ? ceil_div(n, 32) : ceil_div(n, GH_BN), few ? 1 : ceil_div(m, GH_BM), batch);
 #define GH(TX, G)                                                                                        \
         if (few) gemm_heads_few_rows_kernel<TX, bf16_t, G><<<grid, 256, 0, stream>>>(                    \
-            (const TX*)x, ldx, (int)batch_x, (const bf16_t*)w, (bf16_t*)out, ldo, (int)batch_o, m, n, k, gate, ldg, (int)batch_g); \
+            (const TX*)x, ldx, (int)batch_x, (const bf16_t*)w, (bf16_t*)out, ldo, (int)batch_o, m, n, k, gate, ldg, (int)batch_g, gate_one); \
         else gemm_heads_mfma_kernel<TX, bf16_t, G><<<grid, 256, 0, stream>>>(                            \
-            (const TX*)x, ldx, (int)batch_x, (const bf16_t*)w, (bf16_t*)out, ldo, (int)batch_o, m, n, k, gate, ldg, (int)batch_g)
+            (const TX*)x, ldx, (int)batch_x, (const bf16_t*)w, (bf16_t*)out, ldo, (int)batch_o, m, n, k, gate, ldg, (int)batch_g, gate_one)
         if (x_dtype == ROCML_F32) { if (gate) { GH(float, true); } else { GH(float, false); } }
         else { if (gate) { GH(bf16_t, true); } else { GH(bf16_t, false); } }
 #undef GH

@@ -10,7 +10,7 @@
 // into the MFMA registers, 16 bytes a lane: with K this short every operand byte is used by all
 // tiles of the wave in the same step, and the next block finds the weights in L2.  x may be 32-bit
 // (rounded to bfloat16 on the way in).  GATE: out = product * sigmoid(gate) with gate 32-bit,
-// [M, gate width], the heads side by side at g_stride.
+// [M, gate width], the heads side by side at g_stride; gate_one: one number per head, else one per column.
 #pragma once
 #include "gemm_mfma.h"
 
@@ -33,7 +33,7 @@ template <typename TX, typename TO, bool GATE>
 __global__ void __launch_bounds__(256)
 gemm_heads_mfma_kernel(const TX* __restrict__ x, int ldx, int x_stride, const bf16_t* __restrict__ w,
                        TO* __restrict__ out, int ldo, int o_stride, int m, int n, int k,
-                       const float* __restrict__ gate, int ldg, int g_stride) {
+                       const float* __restrict__ gate, int ldg, int g_stride, int gate_one) {
     int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     int g = lane >> 4, col = lane & 15;
     int h = blockIdx.z;
@@ -90,10 +90,10 @@ gemm_heads_mfma_kernel(const TX* __restrict__ x, int ldx, int x_stride, const bf
             int gn = n0 + j * 16 + 4 * g;
             float v[4] = {acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]};
             if (GATE) {
-                const float* gp = gate + (size_t)gm * ldg + (size_t)h * g_stride + gn;
+                const float* gp = gate + (size_t)gm * ldg + (size_t)h * g_stride + (gate_one ? 0 : gn);
 #pragma unroll
                 for (int e = 0; e < 4; ++e)
-                    if (gn + e < n) v[e] *= 1.0f / (1.0f + expf(-gp[e]));
+                    if (gn + e < n) v[e] *= 1.0f / (1.0f + expf(-gp[gate_one ? 0 : e]));
             }
             TO* op = out + (size_t)gm * ldo + (size_t)h * o_stride + gn;
             if (sizeof(TO) == 2 && gn + 3 < n && ((uintptr_t)op & 7) == 0) {
@@ -114,7 +114,7 @@ template <typename TX, typename TO, bool GATE>
 __global__ void __launch_bounds__(256)
 gemm_heads_few_rows_kernel(const TX* __restrict__ x, int ldx, int x_stride, const bf16_t* __restrict__ w,
                            TO* __restrict__ out, int ldo, int o_stride, int m, int n, int k,
-                           const float* __restrict__ gate, int ldg, int g_stride) {
+                           const float* __restrict__ gate, int ldg, int g_stride, int gate_one) {
     __shared__ float red[3][2][64][4];
     int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     int g = lane >> 4, col = lane & 15;
@@ -160,10 +160,10 @@ gemm_heads_few_rows_kernel(const TX* __restrict__ x, int ldx, int x_stride, cons
 #pragma unroll
         for (int e = 0; e < 4; ++e) v[e] = ((acc[j][e] + red[0][j][lane][e]) + red[1][j][lane][e]) + red[2][j][lane][e];
         if (GATE) {
-            const float* gp = gate + (size_t)col * ldg + (size_t)h * g_stride + gn;
+            const float* gp = gate + (size_t)col * ldg + (size_t)h * g_stride + (gate_one ? 0 : gn);
 #pragma unroll
             for (int e = 0; e < 4; ++e)
-                if (gn + e < n) v[e] *= 1.0f / (1.0f + expf(-gp[e]));
+                if (gn + e < n) v[e] *= 1.0f / (1.0f + expf(-gp[gate_one ? 0 : e]));
         }
         TO* op = out + (size_t)col * ldo + (size_t)h * o_stride + gn;
 #pragma unroll

@@ -44,7 +44,8 @@ __device__ __forceinline__ bf16x8_t as_frag4(u32x4_t v) { return __builtin_bit_c
 // out[m][j] = silu(gate) * up (rocml-kernels/kernels/silu_mul.hip:12-20), formed from the 32-bit
 // accumulators so that gate and up are never rounded or written.
 // EPI_RELUGLU: the same with max(gate, 0) * up.
-enum GemmEpilogue : int { EPI_F32 = 0, EPI_BF16 = 1, EPI_ACC = 2, EPI_SWIGLU = 3, EPI_RELUGLU = 4 };
+// EPI_RELU2: bfloat16 [M, N], every sum v stored as max(v, 0)^2.
+enum GemmEpilogue : int { EPI_F32 = 0, EPI_BF16 = 1, EPI_ACC = 2, EPI_SWIGLU = 3, EPI_RELUGLU = 4, EPI_RELU2 = 5 };
 
 constexpr bool epi_gated(int epi) { return epi == EPI_SWIGLU || epi == EPI_RELUGLU; }
 
@@ -180,6 +181,7 @@ __device__ __forceinline__ void epilogue_store(void* out, size_t idx, float v) {
     if (EPI == EPI_F32) ((float*)out)[idx] = v;
     else if (EPI == EPI_BF16) ((bf16_t*)out)[idx] = f32_to_bf16(v);
     else if (EPI == EPI_ACC) ((float*)out)[idx] += v;
+    else if (EPI == EPI_RELU2) { v = fmaxf(v, 0.f); ((bf16_t*)out)[idx] = f32_to_bf16(v * v); }
 }
 
 // ---- many rows ---------------------------------------------------------------------------

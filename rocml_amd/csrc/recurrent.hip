@@ -905,7 +905,7 @@ head_norm_gate_kernel(const float* __restrict__ o, const float* __restrict__ g, 
     float inv = 1.0f / sqrtf(wave_sum(ss) / (float)dv + eps);
     const float* gr = g + (size_t)t * ldg + g_col0 + (size_t)h * dv;
     for (int j = lane; j < dv; j += WAVE) {
-        float gate = 1.0f / (1.0f + expf(-gr[j]));
+        float gate = g ? 1.0f / (1.0f + expf(-gr[j])) : 1.0f;
         if (silu) gate *= gr[j];
         Elem<TO>::store(out + (size_t)row * dv + j, src[j] * inv * (gain ? gain[(size_t)h * dv + j] : 1.0f) * gate);
     }
@@ -942,7 +942,7 @@ head_norm_gate_vec_kernel(const float* __restrict__ o, const float* __restrict__
         int c = lane + k * WAVE;
         bool ok = c < nv;
         v[k] = ok ? src[c] : zero4;
-        z[k] = ok ? gr[c] : zero4;
+        z[k] = (ok && g) ? gr[c] : zero4;
         w[k] = (ok && wr) ? wr[c] : one4;
     }
     float ss = 0.f;
@@ -961,6 +961,7 @@ head_norm_gate_vec_kernel(const float* __restrict__ o, const float* __restrict__
         float g0 = 1.0f / (1.0f + expf(-z[k].x)), g1 = 1.0f / (1.0f + expf(-z[k].y));
         float g2 = 1.0f / (1.0f + expf(-z[k].z)), g3 = 1.0f / (1.0f + expf(-z[k].w));
         if (silu) { g0 *= z[k].x; g1 *= z[k].y; g2 *= z[k].z; g3 *= z[k].w; }
+        if (!g) g0 = g1 = g2 = g3 = 1.0f;
         float r0 = v[k].x * inv * w[k].x * g0;
         float r1 = v[k].y * inv * w[k].y * g1;
         float r2 = v[k].z * inv * w[k].z * g2;
@@ -983,7 +984,7 @@ head_norm_gate_pack_kernel(const float* __restrict__ o, const float* __restrict_
     const sc_f4 zero4 = {0.f, 0.f, 0.f, 0.f};
     const sc_f4 one4 = {1.f, 1.f, 1.f, 1.f};
     sc_f4 v = ok ? *(const sc_f4*)(o + (size_t)row * dv + 4 * c) : zero4;
-    sc_f4 z = ok ? *(const sc_f4*)(g + (size_t)t * ldg + g_col0 + (size_t)h * dv + 4 * c) : zero4;
+    sc_f4 z = (ok && g) ? *(const sc_f4*)(g + (size_t)t * ldg + g_col0 + (size_t)h * dv + 4 * c) : zero4;
     sc_f4 w = (ok && gain) ? *(const sc_f4*)(gain + (size_t)h * dv + 4 * c) : one4;
     float ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, v.w * v.w)));
 #pragma unroll
@@ -993,6 +994,7 @@ head_norm_gate_pack_kernel(const float* __restrict__ o, const float* __restrict_
     float g0 = 1.0f / (1.0f + expf(-z.x)), g1 = 1.0f / (1.0f + expf(-z.y));
     float g2 = 1.0f / (1.0f + expf(-z.z)), g3 = 1.0f / (1.0f + expf(-z.w));
     if (silu) { g0 *= z.x; g1 *= z.y; g2 *= z.z; g3 *= z.w; }
+    if (!g) g0 = g1 = g2 = g3 = 1.0f;
     rc_store4(out + (size_t)row * dv + 4 * c, v.x * inv * w.x * g0, v.y * inv * w.y * g1, v.z * inv * w.z * g2, v.w * inv * w.w * g3);
 }
 
@@ -1007,11 +1009,12 @@ static void launch_head_norm_gate_pack(const float* o, const float* g, int ldg, 
     else head_norm_gate_pack_kernel<TO, 32><<<grid, RC_BLOCK, 0, stream>>>(o, g, ldg, g_col0, gain, out, rows, n_heads, dv, eps, silu);
 }
 
-// gate_act: 0 the gate is sigmoid(g), 1 it is silu(g) = g sigmoid(g).  gain may be null (ones).
+// gate_act: 0 the gate is sigmoid(g), 1 it is silu(g) = g sigmoid(g), 2 there is none (g is null).  gain may be null (ones).
 ROCML_EXPORT int rocml_head_norm_gate(const float* o, const float* g, int ldg, int g_col0, const float* gain, void* out,
                                       int out_dtype, int n_tokens, int n_heads, int dv, float eps, int gate_act, hipStream_t stream) {
-    ROCML_REQUIRE(gate_act == 0 || gate_act == 1, "head_norm_gate: unknown gate activation %d", gate_act);
-    ROCML_REQUIRE(n_tokens >= 0 && n_heads > 0 && dv > 0 && g_col0 >= 0 && ldg >= g_col0 + n_heads * dv && o && g && out,
+    ROCML_REQUIRE(gate_act >= 0 && gate_act <= 2 && (gate_act == 2) == (g == nullptr), "head_norm_gate: unknown gate activation %d, or a gate missing", gate_act);
+    if (gate_act == 2) gate_act = ldg = g_col0 = 0;          // (what is left: no gate pointer)
+    ROCML_REQUIRE(n_tokens >= 0 && n_heads > 0 && dv > 0 && g_col0 >= 0 && (!g || ldg >= g_col0 + n_heads * dv) && o && out,
                   "head_norm_gate: bad arguments T=%d heads=%d dv=%d ld=%d", n_tokens, n_heads, dv, ldg);
     long long rows = (long long)n_tokens * n_heads;
     if (rows == 0) return 0;
@@ -1154,6 +1157,10 @@ ROCML_EXPORT int rocml_gated_part_norm(const float* y, const float* z, int ldz, 
 // token's key and value: S <- diag(w_t) S + k_t v_t^T.  Two ways to read it:
 //   after the update (a retention):        o_t = S_t^T q_t, with w_t one constant per head;
 //   before it, with a bonus on the token:  o_t = (S_(t-1) + diag(u) k_t v_t^T)^T q_t, with w_t per token and channel.
+// A third form writes what it forgets: there is no key, S_t = diag(1 - g_t) S_(t-1) + g_t v_t^T = S_(t-1) + diag(g_t)
+// (v_t^T - S_(t-1)) and o_t = S_t^T silu(q_t), with g_t = (1 - l) sigmoid(-(x_t + b)) from logits x and, per channel, a bias
+// b and the forget gate's lower bound l (the forget gate 1 - g = l + (1 - l) sigmoid(x + b)); silu and g are formed on the
+// way into LDS.  Writing the update through g and not through 1 - g keeps the small g of a gate that forgets little exact.
 // The columns of S (one per value) do not depend on each other: a block takes (sequence, head, 16 CPL values).  The
 // 16 lanes of a row of lanes hold CPL neighbouring columns, lane l the R entries l R .. l R + R - 1 of each: what a
 // lane reads of q, k and the decays serves CPL columns, which is what keeps the walk off the LDS's bandwidth.  The
@@ -1178,23 +1185,29 @@ struct DecayScanArgs {
     const float* w_offset;                     // [H * dk] or null: w holds logits x, the decay is exp(-exp(x + offset))
     const float* head_decay;                   // [H], or null (then w)
     const float* bonus;                        // [H * dk], or null: the state is read after its update
+    const float* gate_lower;                   // [H * dk] or null: k holds logits of a forget gate with this lower bound and the
+    const float* gate_bias;                    // bias gate_bias; q is raw and passes silu (there is no key and no other decay)
     float* state; const int* cu_seqlens; const int* seq_slots;
     float* out; int n_heads; int dk; int dv;
 };
 
-// R: entries of a column per lane (dk <= 16 R).  CPL: columns per lane.  BONUS: a decay per token and channel and a
-// bonus, the state read before its update; else one decay per head, the state read after it.
+enum DecayMode : int { DECAY_HEAD = 0, DECAY_BONUS = 1, DECAY_GATE = 2 };
+
+// R: entries of a column per lane (dk <= 16 R).  CPL: columns per lane.  DECAY_BONUS: a decay per token and channel and a
+// bonus, the state read before its update; DECAY_HEAD: one decay per head, the state read after it; DECAY_GATE: the
+// forget gate that writes (its g in place of the key), the state read after it.
 // A token's row in LDS has a fixed layout, whatever dk: q, k (and the decays) padded to 16 R numbers each, the block's
-// 16 CPL values, and without BONUS the token's decay (the head's, or one for the rows beyond the sequence's last
-// token, which then leave the state as it is: with BONUS their decays are one and their keys zero).  A lane reads its
+// 16 CPL values, and with DECAY_HEAD the token's decay (the head's, or one for the rows beyond the sequence's last
+// token, which then leave the state as it is: with DECAY_BONUS their decays are one and their keys zero, with DECAY_GATE their g is).  A lane reads its
 // R numbers of each part as whole vectors at fixed offsets, without a bound to check.
-template <int R, int CPL, bool BONUS>
+template <int R, int CPL, int MODE>
 __global__ void __launch_bounds__(DS_THREADS)
 decay_scan_kernel(DecayScanArgs a) {
+    constexpr bool BONUS = MODE == DECAY_BONUS, GATE = MODE == DECAY_GATE, HEAD = MODE == DECAY_HEAD;
     constexpr int ARRAYS = BONUS ? 3 : 2;
     constexpr int DKP = DS_LANES * R;
     constexpr int TILE = DS_GROUPS * CPL;                            // columns of a block
-    constexpr int ROW = ARRAYS * DKP + TILE + (BONUS ? 0 : 4);
+    constexpr int ROW = ARRAYS * DKP + TILE + (HEAD ? 4 : 0);
     constexpr int SLOTS = (ROW + DS_THREADS - 1) / DS_THREADS;
     constexpr int NV = DS_TOKENS * CPL;                              // sums of a lane per group of tokens
     __shared__ __attribute__((aligned(16))) float ds_rows[DS_CHUNK * ROW];
@@ -1204,11 +1217,13 @@ decay_scan_kernel(DecayScanArgs a) {
     int dk = a.dk;
     int col0 = tile * TILE + c * CPL;
     int first = a.cu_seqlens[b], n = a.cu_seqlens[b + 1] - first;
-    float hd = BONUS ? 0.f : a.head_decay[h];
+    float hd = HEAD ? a.head_decay[h] : 0.f;
     // the columns of a chunk's rows that this thread brings in: where they come from, per slot
     const float* src[SLOTS];
     int src_ld[SLOTS];
     float offset[SLOTS], beyond[SLOTS], fixed[SLOTS];
+    float span[SLOTS];            // GATE: one less the forget gate's lower bound
+    int form[SLOTS];              // GATE: 1 a query's column, 2 a gate's, 0 neither
     bool is_logit[SLOTS];
 #pragma unroll
     for (int m = 0; m < SLOTS; ++m) {
@@ -1219,12 +1234,18 @@ decay_scan_kernel(DecayScanArgs a) {
         beyond[m] = 0.f;           // what rows beyond the sequence's last token hold
         fixed[m] = 0.f;            // what a column without a source holds
         is_logit[m] = false;
+        span[m] = 0.f;
+        form[m] = 0;
         int part = x / DKP, ch = x - part * DKP;
         if (part < ARRAYS) {
             if (ch < dk) {
                 size_t e = (size_t)h * dk + ch;
-                if (part == 0) { src[m] = a.q + a.q_col0 + e; src_ld[m] = a.ldq; }
-                else if (part == 1) { src[m] = a.k + a.k_col0 + e; src_ld[m] = a.ldk; }
+                if (part == 0) { src[m] = a.q + a.q_col0 + e; src_ld[m] = a.ldq; form[m] = 1; }
+                else if (part == 1) {
+                    src[m] = a.k + a.k_col0 + e;
+                    src_ld[m] = a.ldk;
+                    if constexpr (GATE) { form[m] = 2; span[m] = 1.f - a.gate_lower[e]; offset[m] = a.gate_bias[e]; }
+                }
                 else {
                     src[m] = a.w + a.w_col0 + e;
                     src_ld[m] = a.ldw;
@@ -1286,6 +1307,17 @@ decay_scan_kernel(DecayScanArgs a) {
                 }
                 sums[p] = sum;
             }
+        } else if constexpr (GATE) {
+#pragma unroll
+            for (int p = 0; p < CPL; ++p) {
+                float sum = 0.f;
+#pragma unroll
+                for (int r = 0; r < R; ++r) {
+                    s[p][r] = fmaf(kk[r], vv[p] - s[p][r], s[p][r]);
+                    sum = fmaf(s[p][r], qq[r], sum);
+                }
+                sums[p] = sum;
+            }
         } else {
 #pragma unroll
             for (int p = 0; p < CPL; ++p) {
@@ -1333,6 +1365,12 @@ decay_scan_kernel(DecayScanArgs a) {
             qq[r] = in ? a.q[t * a.ldq + a.q_col0 + e] : 0.f;
             kk[r] = in ? a.k[t * a.ldk + a.k_col0 + e] : 0.f;
             ww[r] = 0.f;
+            if constexpr (GATE) {
+                if (in) {
+                    qq[r] = rc_silu(qq[r]);
+                    kk[r] = (1.f - a.gate_lower[e]) / (1.0f + expf(kk[r] + a.gate_bias[e]));
+                }
+            }
             if constexpr (BONUS) {
                 if (in) {
                     float x = a.w[t * a.ldw + a.w_col0 + e];
@@ -1370,6 +1408,14 @@ decay_scan_kernel(DecayScanArgs a) {
                 for (int j = 0; j < DS_CHUNK; ++j) {
                     float val = next[m][j];
                     if (BONUS && is_logit[m]) val = expf(-expf(val + offset[m]));
+                    if constexpr (GATE) {
+                        // silu(q) = q / (1 + e^-q), and g = (1 - l) / (1 + e^(x + b))
+                        if (form[m]) {
+                            bool is_q = form[m] == 1;
+                            float e = expf(is_q ? -val : val + offset[m]);
+                            val = (is_q ? val : span[m]) / (1.0f + e);
+                        }
+                    }
                     if (!src[m]) val = fixed[m];
                     if (t0 + j >= n) val = beyond[m];
                     ds_rows[j * ROW + x] = val;
@@ -1415,7 +1461,7 @@ decay_scan_kernel(DecayScanArgs a) {
                     for (int p = 0; p < CPL; ++p) vv[p] = vals[c * CPL + p];
                 }
                 float dec = 0.f;
-                if constexpr (!BONUS) dec = vals[TILE];
+                if constexpr (HEAD) dec = vals[TILE];
                 token(qq, kk, ww, vv, dec, acc + jj * CPL);
             }
 #pragma unroll
@@ -1435,8 +1481,9 @@ decay_scan_kernel(DecayScanArgs a) {
 template <int R, int CPL>
 static void launch_decay_scan_cols(const DecayScanArgs& a, int n_seqs, hipStream_t stream) {
     dim3 grid(n_seqs, a.n_heads, ceil_div(a.dv, DS_GROUPS * CPL));
-    if (a.bonus) decay_scan_kernel<R, CPL, true><<<grid, DS_THREADS, 0, stream>>>(a);
-    else decay_scan_kernel<R, CPL, false><<<grid, DS_THREADS, 0, stream>>>(a);
+    if (a.bonus) decay_scan_kernel<R, CPL, DECAY_BONUS><<<grid, DS_THREADS, 0, stream>>>(a);
+    else if (a.gate_lower) decay_scan_kernel<R, CPL, DECAY_GATE><<<grid, DS_THREADS, 0, stream>>>(a);
+    else decay_scan_kernel<R, CPL, DECAY_HEAD><<<grid, DS_THREADS, 0, stream>>>(a);
 }
 
 template <int R>
@@ -1451,21 +1498,23 @@ static void launch_decay_scan(const DecayScanArgs& a, int n_seqs, hipStream_t st
 
 ROCML_EXPORT int rocml_decay_scan(const float* q, int ldq, int q_col0, const float* k, int ldk, int k_col0, const float* v,
                                   int ldv, int v_col0, const float* w, int ldw, int w_col0, const float* w_offset,
-                                  const float* head_decay, const float* bonus, float* state, int n_slots, const int* cu_seqlens,
+                                  const float* head_decay, const float* bonus, const float* gate_lower, const float* gate_bias,
+                                  float* state, int n_slots, const int* cu_seqlens,
                                   const int* seq_slots, int n_seqs, int n_tokens, float* out, int n_heads, int dk, int dv,
                                   hipStream_t stream) {
     ROCML_REQUIRE(n_tokens >= 0 && n_seqs >= 0 && n_slots > 0 && n_heads > 0 && dk > 0 && dv > 0, "decay_scan: bad sizes T=%d B=%d H=%d",
                   n_tokens, n_seqs, n_heads);
     ROCML_REQUIRE(dk <= 16 * DS_LANES, "decay_scan: a key size of %d exceeds %d", dk, 16 * DS_LANES);
     ROCML_REQUIRE(q && k && v && state && cu_seqlens && seq_slots && out, "decay_scan: missing arguments");
-    ROCML_REQUIRE((w != nullptr) != (head_decay != nullptr) && (w != nullptr) == (bonus != nullptr),
-                  "decay_scan: a decay per token and channel with a bonus, or one decay per head without");
+    ROCML_REQUIRE((w != nullptr) + (head_decay != nullptr) + (gate_lower != nullptr) == 1 && (w != nullptr) == (bonus != nullptr) &&
+                      (gate_lower != nullptr) == (gate_bias != nullptr),
+                  "decay_scan: a decay per token and channel with a bonus, one decay per head without, or a forget gate's lower bound and bias");
     ROCML_REQUIRE(!w_offset || w, "decay_scan: an offset goes with decays given as logits");
     ROCML_REQUIRE(q_col0 >= 0 && k_col0 >= 0 && v_col0 >= 0 && ldq >= q_col0 + n_heads * dk && ldk >= k_col0 + n_heads * dk &&
                       ldv >= v_col0 + n_heads * dv && (!w || (w_col0 >= 0 && ldw >= w_col0 + n_heads * dk)),
                   "decay_scan: a row stride is too small for its columns");
     if (n_tokens == 0 || n_seqs == 0) return 0;
-    DecayScanArgs a{q, ldq, q_col0, k, ldk, k_col0, v, ldv, v_col0, w, ldw, w_col0, w_offset, head_decay, bonus, state, cu_seqlens,
+    DecayScanArgs a{q, ldq, q_col0, k, ldk, k_col0, v, ldv, v_col0, w, ldw, w_col0, w_offset, head_decay, bonus, gate_lower, gate_bias, state, cu_seqlens,
                     seq_slots, out, n_heads, dk, dv};
     int r = ceil_div(dk, DS_LANES);
     if (r <= 1) launch_decay_scan<1>(a, n_seqs, stream);

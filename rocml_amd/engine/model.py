@@ -143,8 +143,27 @@ class DecoderModel:
     # -- cache -------------------------------------------------------------------------
     def cache_requests(self) -> List[Optional[object]]:
         """What each schedule entry needs of the cache (None if it reads another's)."""
-        return [None if e.reads_cache_of is not None else self.blocks[e.layer].cache_request()
+        return [self._reader_request(self.blocks[e.layer]) if e.reads_cache_of is not None else self.blocks[e.layer].cache_request()
                 for e in self.spec.schedule]
+
+    @staticmethod
+    def _reader_request(block) -> Optional[object]:
+        """What a block that reads another entry's line keeps for itself."""
+        return block.reader_request() if hasattr(block, "reader_request") else None
+
+    def entry_view(self, i: int, cache: Cache, step: StepContext):
+        """The cache view of schedule entry ``i``: its own line, or the line of the entry it reads, of which a block with
+        state of its own beside the mixer's shares a part and keeps the rest itself."""
+        entry = self.spec.schedule[i]
+        own = cache.view(i, step) if cache.has_line(i) else None
+        if entry.reads_cache_of is None:
+            return own
+        owner = entry.reads_cache_of
+        shared = cache.view(owner, step) if cache.has_line(owner) else None
+        source, block = self.blocks[self.spec.schedule[owner].layer], self.blocks[entry.layer]
+        if hasattr(source, "shared_view"):
+            shared = source.shared_view(shared)
+        return block.reader_view(shared, own) if hasattr(block, "reader_view") else shared
 
     def activation_bytes(self, n_tokens: int, n_wanted: int) -> int:
         """Bytes of activations and scratch memory a step of ``n_tokens`` tokens with ``n_wanted``
@@ -188,9 +207,10 @@ class DecoderModel:
             # entries that add the embedding's output to the stream later need it kept
             x0 = ws.get("model.x0", (step.n_tokens, s.hidden), torch.float32)
             ops.weighted_sum(x0, [x], [1.0])
+        following_view = None
         for i, entry in enumerate(s.schedule):
-            owner = i if entry.reads_cache_of is None else entry.reads_cache_of
-            view = cache.view(owner, step) if cache.has_line(owner) else None
+            view = following_view if following_view is not None else self.entry_view(i, cache, step)
+            following_view = None
             block = self.blocks[entry.layer]
             if entry.offset_row is not None:
                 # (sums that a product left for the next norm may still be missing from x: additions commute)
@@ -205,11 +225,12 @@ class DecoderModel:
             if following is not None and (s.schedule[i + 1].offset_row is not None or s.schedule[i + 1].add_embedding):
                 following = None      # the stream changes between the two blocks: nothing can be prepared across
             if getattr(block, "takes_next_norm", False) and hasattr(following, "entry_hint"):
-                hint = following.entry_hint(step)
+                following_view = self.entry_view(i + 1, cache, step)
+                hint = following.entry_hint(step, following_view)
             if hint is not None:
-                block.forward(step, x, view, owner == i, next_norm=hint)
+                block.forward(step, x, view, entry.reads_cache_of is None, next_norm=hint)
             else:
-                block.forward(step, x, view, owner == i)
+                block.forward(step, x, view, entry.reads_cache_of is None)
         if n_want == 0:
             ws.drop_pending()
             return None

@@ -32,20 +32,23 @@ _SIGNATURES = {
         "rocml_swiglu": [_P, _I, _P, _I, _I, _I, _I, _I, _F, _F, _P],
         "rocml_rope_table": [_P, _P, _P, _P, _I, _I, _F, _P],
         "rocml_qk_norm_rope_append": [_P, _I, _I, _I, _I, _I, _I, _P, _P, _F, _P, _P, _I, _I, _P, _P, _P,
-                                      _I, _P, _I, _P, _P, _I, _I, _I, _LL, _P, _I, _F, _I, _P, _I, _P],
+                                      _I, _P, _I, _P, _P, _I, _I, _I, _LL, _P, _I, _F, _I, _P, _I, _I, _P],
         "rocml_qk_span_stats": [_P, _I, _I, _I, _I, _I, _P, _F, _P, _P],
-        "rocml_norm_add": [_P, _P, _I, _I, _P, _P, _F, _I, _P, _I, _P, _I, _LL, _I, _P, _F, _P],
+        "rocml_norm_add": [_P, _P, _I, _I, _P, _P, _F, _I, _P, _I, _P, _I, _LL, _I, _P, _F, _P, _P, _I, _P, _I, _P],
+        "rocml_norm_add_conv_fits": [_I, _I],
+        "rocml_added_conv": [_P, _P, _I, _I, _I, _P, _I, _P, _I, _P, _P, _I, _P, _P],
+        "rocml_activate": [_P, _P, _I, _LL, _I, _P],
         "rocml_norm_add_branches": [_P, _P, _P, _P, _P, _F, _F, _I, _I, _P, _P, _F, _I, _P, _I, _P],
         "rocml_norm_add_branches_fits": [_I],
         "rocml_layernorm": [_P, _P, _I, _I, _P, _P, _F, _P, _I, _P],
         "rocml_token_side_gate": [_P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P, _I, _P],
         "rocml_add_into": [_P, _P, _I, _LL, _P],
         "rocml_add_row_vector": [_P, _P, _I, _I, _P],
-        "rocml_latent_prepare": [_P, _I, _I, _I, _I, _I, _I, _P, _P, _F, _P, _P, _P, _P, _I, _P, _I, _P, _P, _I, _I, _P],
-        "rocml_rope_heads": [_P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
+        "rocml_latent_prepare": [_P, _I, _I, _I, _I, _I, _I, _P, _P, _F, _P, _P, _P, _P, _I, _P, _I, _P, _P, _I, _I, _I, _P],
+        "rocml_rope_heads": [_P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P],
         "rocml_latent_window_plan": [_P, _P, _P, _I, _I, _I, _I, _P, _I, _P, _I, _P],
         "rocml_latent_window_gather": [_P, _I, _I, _I, _P, _I, _P, _P],
-        "rocml_gate_heads": [_P, _I, _I, _I, _P, _I, _P, _I, _I, _I, _P],
+        "rocml_gate_heads": [_P, _I, _I, _I, _P, _I, _P, _I, _I, _I, _I, _P],
         "rocml_sigmoid_gate": [_P, _I, _P, _I, _I, _I, _I, _P],
         "rocml_sum_norm": [_P, _I, _I, _F, _F, _I, _P, _P, _P, _F, _P, _I, _P],
         "rocml_convert": [_P, _P, _I, _LL, _P],
@@ -60,7 +63,7 @@ _SIGNATURES = {
         "rocml_mlstm_scan": [_P, _I, _I, _I, _I, _I, _I, _P, _P, _F, _F, _F, _P, _P, _P, _I, _P, _P, _I, _I, _P, _I, _I, _I, _P],
         "rocml_mlstm_tile": [],
         "rocml_head_norm_gate": [_P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _F, _I, _P],
-        "rocml_decay_scan": [_P, _I, _I, _P, _I, _I, _P, _I, _I, _P, _I, _I, _P, _P, _P, _P, _I, _P, _P, _I, _I, _P, _I, _I, _I, _P],
+        "rocml_decay_scan": [_P, _I, _I, _P, _I, _I, _P, _I, _I, _P, _I, _I, _P, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _P, _I, _I, _I, _P],
         "rocml_rotate_rows": [_P, _I, _I, _I, _I, _I, _I, _P, _P, _F, _I, _F, _P],
         "rocml_shift_mix": [_P, _I, _I, _I, _P, _I, _P, _I, _P, _P, _P, _I, _P, _P],
         "rocml_tanh": [_P, _P, _I, _LL, _P],
@@ -75,15 +78,15 @@ _SIGNATURES = {
     "gemm": {
         "rocml_gemm": [_P, _I, _I, _P, _I, _I, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P, _P, _LL, _P, _I, _F, _I, _P],
         "rocml_splitk_reduce": [_P, _P, _I, _I, _I, _I, _I, _I, _P],
-        "rocml_gemm_batched": [_P, _I, _I, _LL, _P, _I, _I, _LL, _P, _I, _I, _LL, _I, _I, _I, _I, _P, _I, _LL, _P],
+        "rocml_gemm_batched": [_P, _I, _I, _LL, _P, _I, _I, _LL, _P, _I, _I, _LL, _I, _I, _I, _I, _P, _I, _LL, _I, _P],
         "rocml_gemm_residual_prescale_pays": [_I, _I, _I],
         "rocml_gemm_residual_prescale": [_P, _I, _P, _I, _P, _I, _P, _P, _I, _P, _I, _I, _I, _I, _P],
     },
     "attention": {
         "rocml_attention": [_P, _P, _P, _P, _I, _P, _I, _P, _P, _I, _I, _I, _I, _I, _F, _I, _I,
-                            _P, _I, _I, _P, _I, _I, _P, _LL, _I, _I, _I, _P, _I, _P, _F, _P],
+                            _P, _I, _I, _P, _I, _I, _P, _LL, _I, _I, _I, _P, _I, _P, _F, _I, _P],
         "rocml_attention_decode_fused": [_P, _I, _I, _LL, _P, _P, _F, _P, _P, _I, _P, _P, _P, _P, _I, _P, _P,
-                                         _I, _I, _I, _I, _I, _F, _I, _I, _I, _P, _LL, _P, _I, _F, _I, _P, _I, _P, _I, _P],
+                                         _I, _I, _I, _I, _I, _F, _I, _I, _I, _P, _LL, _P, _I, _F, _I, _P, _I, _P, _I, _P, _I, _I, _I, _P],
         "rocml_attention_prefill_fused": [_P, _I, _P, _F, _P, _P, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _F, _I,
                                           _P, _I, _P, _P],
     },
@@ -261,6 +264,21 @@ def swiglu(gate_up: torch.Tensor, out: torch.Tensor, interleaved: bool = False, 
         GATE_ACTIVATIONS[activation], 0.0 if limit is None else float(limit), float(up_offset), _stream()))
 
 
+ACTIVATIONS = {**GATE_ACTIVATIONS, "relu2": 4}      # relu2: max(x, 0)^2
+
+
+def activate(x: torch.Tensor, out: torch.Tensor, activation: str) -> None:
+    """``out = act(x)`` in ``out``'s type, for 32-bit ``x`` (``out`` may be ``x`` itself); one of ``ACTIVATIONS``."""
+    _dev(x, out)
+    _want(x, torch.float32, "the values")
+    if activation not in ACTIVATIONS:
+        raise KernelError(f"unknown activation {activation!r}; known: {sorted(ACTIVATIONS)}")
+    if x.numel() != out.numel():
+        raise KernelError("activate: sizes differ")
+    _check("elementwise", library("elementwise").rocml_activate(_ptr(x), _ptr(out), _code(out), x.numel(), ACTIVATIONS[activation],
+                                                                _stream()))
+
+
 def rope_table(positions: torch.Tensor, inv_freq: torch.Tensor, cos: torch.Tensor, sin: torch.Tensor,
                scale: float = 1.0) -> None:
     """``cos[t, i] = scale * cos(positions[t] * inv_freq[i])`` and the sines likewise (angles in 64-bit)."""
@@ -287,7 +305,7 @@ def qk_norm_rope_append(qkv: torch.Tensor, n_heads: int, n_kv_heads: int, head_d
                         token_seq: torch.Tensor, token_pos: torch.Tensor, write_kv: bool = True,
                         n_splits: int = 1, pairing: str = "halves", bias: Optional[torch.Tensor] = None,
                         v_head_dim: Optional[int] = None, q_temp=None, span_inv: Optional[torch.Tensor] = None,
-                        span_self: bool = False) -> None:
+                        span_self: bool = False, values_are_keys: bool = False) -> None:
     """``qkv`` is ``[T, ld]`` with q, k, v side by side (k and v may be absent when
     ``write_kv`` is false).  Keys are ``[pages, Hkv, page_size, D]``, values
     ``[pages, Hkv, D, page_size]``.  ``pairing``: which two values of the rotated width turn
@@ -300,7 +318,8 @@ def qk_norm_rope_append(qkv: torch.Tensor, n_heads: int, n_kv_heads: int, head_d
     ``1 + coef * ln(floor((p + 1) / every) + 1)`` after its norm.  ``span_inv``: ``[T, 2]`` 32-bit, the
     factors of a norm over a token's whole q row and whole k row (``qk_span_stats``); the gains then
     have one number per column of the q and of the k projection.  ``span_self``: the same norm, its
-    factors formed inside the kernel (for steps of few tokens)."""
+    factors formed inside the kernel (for steps of few tokens).  ``values_are_keys``: ``qkv`` holds no value columns, a
+    value is the projected key (with its bias) before norm and rotation."""
     qt_coef, qt_every = (0.0, 0) if q_temp is None else (float(q_temp[0]), int(q_temp[1]))
     if q_temp is not None and qt_every <= 0:
         raise KernelError(f"the period of the query's stretch must be positive, got {qt_every}")
@@ -318,7 +337,7 @@ def qk_norm_rope_append(qkv: torch.Tensor, n_heads: int, n_kv_heads: int, head_d
     if bias is not None:
         _want(bias, torch.float32, "projection bias")
         # (rows may be wider than the projection: a product shared with other mixers, whose columns follow)
-        if bias.numel() > ld or bias.numel() < n_heads * head_dim + (n_kv_heads * (head_dim + dv) if write_kv else 0):
+        if bias.numel() > ld or bias.numel() < n_heads * head_dim + (n_kv_heads * (head_dim + (0 if values_are_keys else dv)) if write_kv else 0):
             raise KernelError(f"the bias has {bias.numel()} values for rows of {ld}")
     whole = span_inv is not None or span_self
     if span_inv is not None:
@@ -356,7 +375,7 @@ def qk_norm_rope_append(qkv: torch.Tensor, n_heads: int, n_kv_heads: int, head_d
         eps, _ptr(cos), _ptr(sin), rot_dim if cos is not None else 0, ROPE_PAIRINGS[pairing], _ptr(q_out), _ptr(k_cache),
         _ptr(v_cache), _code(q_out if q_out is not None else k_cache), _ptr(block_table), bt_width, _ptr(token_seq),
         _ptr(token_pos), page_size, 1 if write_kv else 0, n_splits, split_stride, _ptr(bias), dv, qt_coef, qt_every,
-        _ptr(span_inv), 1 if span_self else 0, _stream()))
+        _ptr(span_inv), 1 if span_self else 0, 1 if values_are_keys else 0, _stream()))
 
 
 def qk_span_stats(qkv: torch.Tensor, q_width: int, k_width: int, bias: Optional[torch.Tensor], eps: float,
@@ -375,13 +394,15 @@ def qk_span_stats(qkv: torch.Tensor, q_width: int, k_width: int, bias: Optional[
 
 def norm_add(x: torch.Tensor, y: torch.Tensor, gain: torch.Tensor, bias: Optional[torch.Tensor], eps: float,
              layer: bool, copy: Optional[torch.Tensor] = None, partials: Optional[torch.Tensor] = None,
-             replace: bool = False, next_gain: Optional[torch.Tensor] = None, next_eps: float = 0.0) -> None:
+             replace: bool = False, next_gain: Optional[torch.Tensor] = None, next_eps: float = 0.0, conv=None) -> None:
     """``x += f(y)`` row by row in 32-bit: ``f`` a layer norm ``(y - mean) / sqrt(var + eps) * gain + bias``
     (``layer``) or ``y / sqrt(mean(y^2) + eps) * gain``.  ``copy`` gets the new ``x`` in its own type.
     ``partials`` (``[splits, rows, n]`` 32-bit): the K pieces of the product that made ``y``, added to ``y`` in
     split order first, or with ``replace`` all of ``y`` (what ``y`` holds is not read).  ``next_gain`` (with ``copy``):
     ``copy`` gets the root-mean-square norm of the new ``x`` instead, ``x / sqrt(mean(x^2) + next_eps) * next_gain``: the
-    norm that reads the stream next."""
+    norm that reads the stream next.  ``conv``: ``(weights [taps, n], state [slots, taps - 1, n], slots [rows])``, for a step
+    of one token per sequence (row ``b`` is sequence ``b``'s token): that norm's output ``h`` is replaced by ``h`` plus its
+    causal convolution and the kept rows move up by one, as ``added_conv`` does; only where ``norm_add_conv_fits``."""
     _dev(x, y, gain, bias, copy, partials, next_gain)
     if next_gain is not None and (copy is None or next_gain.dtype != torch.float32 or next_gain.numel() != x.shape[1]):
         raise KernelError("norm_add: the next norm needs a 32-bit gain of the row's size and a place for its output")
@@ -398,10 +419,53 @@ def norm_add(x: torch.Tensor, y: torch.Tensor, gain: torch.Tensor, bias: Optiona
     if x.dim() != 2 or y.shape != x.shape or gain.numel() != x.shape[1] or (copy is not None and copy.shape != x.shape) \
             or (bias is not None and (bias.dtype != torch.float32 or bias.numel() != x.shape[1])):
         raise KernelError("norm_add: shapes do not fit")
+    conv_w = conv_state = conv_slots = None
+    taps = 0
+    if conv is not None:
+        conv_w, conv_state, conv_slots = conv
+        _dev(conv_w, conv_state, conv_slots)
+        _want(conv_w, torch.float32, "convolution weights")
+        _want(conv_slots, torch.int32, "sequence slots")
+        taps = conv_w.shape[0]
+        if next_gain is None or layer or not norm_add_conv_fits(x.shape[1], taps) or conv_w.shape[1] != x.shape[1] \
+                or conv_state.dtype != copy.dtype or conv_state.dim() != 3 or conv_state.shape[1:] != (taps - 1, x.shape[1]) \
+                or conv_slots.numel() != x.shape[0]:
+            raise KernelError("norm_add: the convolution's weights, kept rows or slots do not fit the step")
     _check("elementwise", library("elementwise").rocml_norm_add(
         _ptr(x), _ptr(y), x.shape[0], x.shape[1], _ptr(gain), _ptr(bias), float(eps), 1 if layer else 0, _ptr(copy),
         _code(copy) if copy is not None else 0, _ptr(partials), n_splits, split_stride, 1 if replace else 0, _ptr(next_gain),
-        float(next_eps), _stream()))
+        float(next_eps), _ptr(conv_w), _ptr(conv_state), 0 if conv_state is None else conv_state.shape[0], _ptr(conv_slots), taps,
+        _stream()))
+
+
+def norm_add_conv_fits(n: int, taps: int) -> bool:
+    """Whether ``norm_add`` takes a convolution of so many taps over rows of ``n`` values."""
+    return bool(library("elementwise").rocml_norm_add_conv_fits(int(n), int(taps)))
+
+
+ADDED_CONV_MAX_TAPS = 8
+
+
+def added_conv(h: torch.Tensor, w: torch.Tensor, state: Optional[torch.Tensor], cu_seqlens: torch.Tensor, seq_slots: torch.Tensor,
+               q_counts: Sequence[int], out: torch.Tensor) -> None:
+    """``out_t = h_t + sum_j w[j] * h_(t - (taps - 1) + j)`` per channel, 32-bit sums, for ``h``, ``out [T, n]`` of one type and
+    the 32-bit ``w [taps, n]``.  ``state [slots, taps - 1, n]`` in ``h``'s type holds every sequence's last ``taps - 1`` inputs
+    (zeros at its start; None with one tap), is read for the inputs before the step's first token and brought up to date.
+    ``q_counts`` (host): tokens of each sequence in the step."""
+    _dev(h, w, state, cu_seqlens, seq_slots, out)
+    _want(w, torch.float32, "convolution weights")
+    _want(cu_seqlens, torch.int32, "sequence offsets")
+    _want(seq_slots, torch.int32, "sequence slots")
+    n_tokens, n = h.shape
+    taps, n_seqs = w.shape[0], seq_slots.numel()
+    if w.shape != (taps, n) or out.shape != h.shape or out.dtype != h.dtype or cu_seqlens.numel() != n_seqs + 1 or len(q_counts) != n_seqs:
+        raise KernelError(f"added_conv: weights {tuple(w.shape)}, output {tuple(out.shape)} or tables do not fit {tuple(h.shape)}")
+    if taps > 1 and (state is None or state.dtype != h.dtype or state.dim() != 3 or state.shape[1:] != (taps - 1, n)):
+        raise KernelError(f"added_conv: the kept rows do not fit {taps} taps of {n} channels in {h.dtype}")
+    counts = (ctypes.c_int * n_seqs)(*[int(c) for c in q_counts])
+    _check("elementwise", library("elementwise").rocml_added_conv(
+        _ptr(h), _ptr(out), _code(h), n_tokens, n, _ptr(w), taps, _ptr(state), 0 if state is None else state.shape[0],
+        _ptr(cu_seqlens), _ptr(seq_slots), n_seqs, counts, _stream()))
 
 
 def norm_add_branches_fits(n: int, n_branches: int) -> bool:
@@ -481,21 +545,28 @@ def add_row_vector(x: torch.Tensor, b: torch.Tensor) -> None:
 
 
 def latent_prepare(proj: torch.Tensor, q_rank: int, kv_rank: int, rot_part: int, rot_dims: int,
-                   q_gain: torch.Tensor, kv_gain: torch.Tensor, eps: float, cos: Optional[torch.Tensor],
+                   q_gain: torch.Tensor, kv_gain: Optional[torch.Tensor], eps: float, cos: Optional[torch.Tensor],
                    sin: Optional[torch.Tensor], cq_out: torch.Tensor, cache: Optional[torch.Tensor],
                    block_table: Optional[torch.Tensor], token_seq: torch.Tensor, token_pos: torch.Tensor,
-                   write_cache: bool = True) -> None:
+                   write_cache: bool = True, pairing: str = "halves") -> None:
     """What follows a latent attention's first projection.  A row of ``proj`` (32-bit) holds the
     query latent (``q_rank``), the key/value latent (``kv_rank``) and the shared rotated key part
     (``rot_part``, of which the first ``rot_dims`` turn in pairs ``(i, i + rot_dims/2)``).  Both
     latents get their root-mean-square norm; the query latent goes to ``cq_out [T, q_rank]``, the
-    other two into the token's row of ``cache [pages, page_size, kv_rank + rot_part]``."""
+    other two into the token's row of ``cache [pages, page_size, kv_rank + rot_part]``.  ``pairing``: as in
+    ``qk_norm_rope_append``.  Without ``write_cache`` only the query latent is read (a row may hold nothing else of these,
+    and ``kv_gain`` may be None)."""
+    if pairing not in ROPE_PAIRINGS:
+        raise KernelError(f"unknown rotation pairing {pairing!r}; known: {sorted(ROPE_PAIRINGS)}")
     _dev(proj, q_gain, kv_gain, cos, sin, cq_out, cache, block_table, token_seq, token_pos)
     _want(proj, torch.float32, "projection output")
     _want(q_gain, torch.float32, "latent norm gain")
-    _want(kv_gain, torch.float32, "latent norm gain")
     n_tokens, ld = proj.shape
-    if q_gain.numel() != q_rank or kv_gain.numel() != kv_rank or cq_out.shape != (n_tokens, q_rank):
+    if write_cache:
+        if kv_gain is None:
+            raise KernelError("appending to the cache needs the key/value latent's gain")
+        _want(kv_gain, torch.float32, "latent norm gain")
+    if q_gain.numel() != q_rank or (write_cache and kv_gain.numel() != kv_rank) or cq_out.shape != (n_tokens, q_rank):
         raise KernelError("latent gains or the query latent's output do not fit the ranks")
     if rot_dims:
         if cos is None or sin is None or cos.shape != (n_tokens, rot_dims // 2) or sin.shape != cos.shape \
@@ -516,16 +587,19 @@ def latent_prepare(proj: torch.Tensor, q_rank: int, kv_rank: int, rot_part: int,
     _check("elementwise", library("elementwise").rocml_latent_prepare(
         _ptr(proj), ld, n_tokens, q_rank, kv_rank, rot_part, rot_dims, _ptr(q_gain), _ptr(kv_gain), eps, _ptr(cos),
         _ptr(sin), _ptr(cq_out), _ptr(cache), _code(cq_out), _ptr(block_table), bt_width, _ptr(token_seq),
-        _ptr(token_pos), page_size, 1 if write_cache else 0, _stream()))
+        _ptr(token_pos), page_size, 1 if write_cache else 0, ROPE_PAIRINGS[pairing], _stream()))
 
 
 def rope_heads(q: torch.Tensor, n_heads: int, head_stride: int, offset: int, rot_part: int, rot_dims: int,
                cos: Optional[torch.Tensor], sin: Optional[torch.Tensor], out: torch.Tensor, out_stride: int,
-               out_offset: int, lead: int = 0) -> None:
+               out_offset: int, lead: int = 0, pairing: str = "halves") -> None:
     """The part of every head of ``q [T, n_heads * head_stride]`` (32-bit) that starts at ``offset``
     and is ``rot_part`` wide, rotated (its first ``rot_dims`` numbers, pairs ``(i, i + rot_dims/2)``),
     written to ``out [T, n_heads * out_stride]`` at ``out_offset`` of every head.  ``lead``: so many
-    numbers before the part are copied unchanged in front of it (``out_offset`` is where they start)."""
+    numbers before the part are copied unchanged in front of it (``out_offset`` is where they start).  ``pairing``: as in
+    ``qk_norm_rope_append``."""
+    if pairing not in ROPE_PAIRINGS:
+        raise KernelError(f"unknown rotation pairing {pairing!r}; known: {sorted(ROPE_PAIRINGS)}")
     _dev(q, cos, sin, out)
     _want(q, torch.float32, "queries")
     n_tokens = q.shape[0]
@@ -536,7 +610,7 @@ def rope_heads(q: torch.Tensor, n_heads: int, head_stride: int, offset: int, rot
         raise KernelError(f"rotation tables must be float32 {(n_tokens, rot_dims // 2)}")
     _check("elementwise", library("elementwise").rocml_rope_heads(
         _ptr(q), q.shape[1], head_stride, offset, rot_part, rot_dims, _ptr(cos), _ptr(sin), _ptr(out), _code(out),
-        out.shape[1], out_stride, out_offset, n_tokens, n_heads, int(lead), _stream()))
+        out.shape[1], out_stride, out_offset, n_tokens, n_heads, int(lead), ROPE_PAIRINGS[pairing], _stream()))
 
 
 def latent_window_plan(cu_seqlens: torch.Tensor, token_pos: torch.Tensor, block_table: torch.Tensor, window: Optional[int],
@@ -573,15 +647,19 @@ def latent_window_gather(cache: torch.Tensor, plan: torch.Tensor, out: torch.Ten
 
 def gate_heads(x: torch.Tensor, x_stride: int, gate: Optional[torch.Tensor], out: torch.Tensor, n_heads: int, n: int) -> None:
     """``out[t, h * n + i] = x[t, h * x_stride + i] * sigmoid(gate[t, h * n + i])`` (``gate`` None: the
-    plain copy): the leading ``n`` numbers of every head of ``x``, gated and packed."""
+    plain copy): the leading ``n`` numbers of every head of ``x``, gated and packed.  A gate of ``n_heads`` columns holds
+    one number per head."""
+    gate_one = gate is not None and n > 1 and gate.shape[1] == n_heads
     _dev(x, out)
-    if gate is not None and (not gate.is_cuda or gate.dtype != torch.float32 or gate.stride(1) != 1 or gate.shape != out.shape):
-        raise KernelError("the gate must be 32-bit and of the output's shape")
+    if gate is not None and (not gate.is_cuda or gate.dtype != torch.float32 or gate.stride(1) != 1
+                             or gate.shape != (out.shape[0], n_heads if gate_one else out.shape[1])):
+        raise KernelError("the gate must be 32-bit and of the output's shape, or hold one number per head")
     if x.dtype != out.dtype or out.shape != (x.shape[0], n_heads * n) or x.shape[1] < n_heads * x_stride:
         raise KernelError("gate_heads: shapes do not fit")
     ldg = 0 if gate is None else (gate.stride(0) if x.shape[0] > 1 else max(gate.stride(0), gate.shape[1]))
     _check("elementwise", library("elementwise").rocml_gate_heads(
-        _ptr(x), _code(x), x.shape[1], x_stride, _ptr(gate), ldg, _ptr(out), x.shape[0], n_heads, n, _stream()))
+        _ptr(x), _code(x), x.shape[1], x_stride, _ptr(gate), ldg, _ptr(out), x.shape[0], n_heads, n, 1 if gate_one else 0,
+        _stream()))
 
 
 def sigmoid_gate(y: torch.Tensor, gate: torch.Tensor, group: int = 1) -> None:
@@ -683,7 +761,7 @@ def add_into(x: torch.Tensor, y: torch.Tensor) -> None:
 # ---- matrix product ------------------------------------------------------------------
 GEMM_AUTO, GEMM_PLAIN = 0, 1
 # epilogues of a product whose weight rows are (gate, up) pairs: act(gate) * up
-GEMM_EPILOGUES = {None: 0, "swiglu": 1, "relu_glu": 2}
+GEMM_EPILOGUES = {None: 0, "swiglu": 1, "relu_glu": 2, "relu2": 3}      # relu2: max(sum, 0)^2, no pairs
 ROW_SCALE_MAX_ROWS = 16     # most rows of a product whose consumer applies a row scale
 
 
@@ -706,7 +784,8 @@ def gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, accumulate: bool =
          defer: bool = False, row_scale: Optional["RowScale"] = None, max_splits: int = 0) -> int:
     """``out (+)= x @ w.T`` for ``x [M, K]``, ``w [N, K]``, ``out [M, N]`` (rows may be
     strided views with unit inner stride).  ``epilogue="swiglu"``: ``w``'s rows are (gate, up)
-    pairs and ``out`` is ``[M, N/2] = silu(gate) * up``.  With ``defer`` a product that was
+    pairs and ``out`` is ``[M, N/2] = silu(gate) * up`` (``"relu_glu"``: ``max(gate, 0) * up``); ``"relu2"``: ``out`` is
+    ``max(x @ w.T, 0)^2``, bfloat16 operands and output on the matrix-core kernels only.  With ``defer`` a product that was
     split along K leaves its partial sums ``[splits, M, N]`` at the start of ``workspace`` and
     returns their number for the caller's next kernel to add; it returns 0 when ``out`` is
     complete.  ``row_scale``: ``x`` lacks its norm's scale (see ``RowScale``), which the gated
@@ -721,7 +800,7 @@ def gemm(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, accumulate: bool =
         raise KernelError(f"unknown epilogue {epilogue!r}")
     m, k = x.shape
     n = w.shape[0]
-    cols = n // 2 if epilogue else n
+    cols = n // 2 if epilogue in ("swiglu", "relu_glu") else n
     if w.shape[1] != k or out.shape != (m, cols):
         raise KernelError(f"matrix product shapes do not fit: x {tuple(x.shape)}, w {tuple(w.shape)}, out {tuple(out.shape)}")
     ws_ptr, ws_bytes = (None, 0) if workspace is None else (workspace.data_ptr(), workspace.numel() * workspace.element_size())
@@ -750,14 +829,17 @@ def gemm_batched(x: torch.Tensor, x_head_stride: int, w: torch.Tensor, out: torc
     ... + K] @ w[h].T`` for ``w [heads, N, K]``; ``x`` and ``out`` are ``[tokens, width]`` matrices
     that hold the heads side by side.  32-bit accumulation; ``x`` may be 32-bit with bfloat16 weights.
     ``gate`` (32-bit ``[tokens, heads * N]``, rows may be a column range of a wider matrix): the
-    product is multiplied by ``sigmoid(gate)``; only where ``gemm_batched_gate_fusable``."""
+    product is multiplied by ``sigmoid(gate)``; only where ``gemm_batched_gate_fusable``.  A gate of ``heads`` columns
+    holds one number per head."""
+    gate_one = gate is not None and w.shape[1] > 1 and gate.shape[1] == w.shape[0]
     _dev(x, w, out)
     ldg = g_stride = 0
     if gate is not None:
-        if not gate.is_cuda or gate.dtype != torch.float32 or gate.stride(1) != 1 or gate.shape != (x.shape[0], w.shape[0] * w.shape[1]) \
+        if not gate.is_cuda or gate.dtype != torch.float32 or gate.stride(1) != 1 \
+                or gate.shape != (x.shape[0], w.shape[0] * (1 if gate_one else w.shape[1])) \
                 or out_head_stride != w.shape[1] or not gemm_batched_gate_fusable(w, x) or x_head_stride % 4:
-            raise KernelError("the gate must be 32-bit [tokens, heads * N] for an output without gaps, on the matrix-core kernel")
-        ldg, g_stride = (gate.stride(0) if x.shape[0] > 1 else max(gate.stride(0), gate.shape[1])), w.shape[1]
+            raise KernelError("the gate must be 32-bit [tokens, heads * N] or [tokens, heads] for an output without gaps, on the matrix-core kernel")
+        ldg, g_stride = (gate.stride(0) if x.shape[0] > 1 else max(gate.stride(0), gate.shape[1])), (1 if gate_one else w.shape[1])
     if x.dim() != 2 or out.dim() != 2 or w.dim() != 3 or x.shape[0] != out.shape[0]:
         raise KernelError("gemm_batched takes x [T, width], w [heads, N, K], out [T, width]")
     heads, n, k = w.shape
@@ -765,7 +847,7 @@ def gemm_batched(x: torch.Tensor, x_head_stride: int, w: torch.Tensor, out: torc
         raise KernelError(f"{heads} heads of K={k} / N={n} do not fit rows of {x.shape[1]} / {out.shape[1]}")
     _check("gemm", library("gemm").rocml_gemm_batched(
         _ptr(x), _code(x), x.shape[1], x_head_stride, _ptr(w), _code(w), k, n * k, _ptr(out), _code(out),
-        out.shape[1], out_head_stride, heads, x.shape[0], n, k, _ptr(gate), ldg, g_stride, _stream()))
+        out.shape[1], out_head_stride, heads, x.shape[0], n, k, _ptr(gate), ldg, g_stride, 1 if gate_one else 0, _stream()))
 
 
 PRESCALE_MAX_ROWS = 16      # most rows gemm_residual_prescale takes
@@ -836,7 +918,7 @@ def attention(q: torch.Tensor, out: torch.Tensor, k_cache: torch.Tensor, v_cache
               q_counts: Optional[Sequence[int]] = None, max_len: int = 0, n_splits: int = 0,
               v_head_dim: Optional[int] = None, values_in_keys: bool = False, chunk: Optional[int] = None,
               slopes: Optional[torch.Tensor] = None, sink: bool = False, sinks: Optional[torch.Tensor] = None,
-              softcap: Optional[float] = None) -> None:
+              softcap: Optional[float] = None, keep_first: int = 0) -> None:
     """Attention of the step's query tokens over the cache.  Keys are ``[pages, Hkv, page, D]``,
     values ``[pages, Hkv, D, page]``.  ``cu_seqlens`` (device), ``q_counts`` (the same knowledge on
     the host: query tokens of each sequence), ``max_new`` (the most of them) and ``max_len``
@@ -848,7 +930,8 @@ def attention(q: torch.Tensor, out: torch.Tensor, k_cache: torch.Tensor, v_cache
     its own block up to itself.  ``slopes`` (32-bit, one per query head): ``slope * (i - j)`` is
     taken off the score of query ``i`` and key ``j``.  ``sink``: the denominator of the softmax has
     one more term ``exp(0)``, or with ``sinks`` (32-bit, one per query head) ``exp(sinks[h])``.
-    ``softcap``: the scaled score ``s`` becomes ``softcap * tanh(s / softcap)`` before the mask."""
+    ``softcap``: the scaled score ``s`` becomes ``softcap * tanh(s / softcap)`` before the mask.
+    ``keep_first``: with a window, the first so many positions are seen whatever their distance."""
     _dev(q, out, k_cache, v_cache, block_table, token_seq, token_pos, cu_seqlens, slopes, sinks)
     if sinks is not None:
         _want(sinks, torch.float32, "sinks")
@@ -895,7 +978,7 @@ def attention(q: torch.Tensor, out: torch.Tensor, k_cache: torch.Tensor, v_cache
         page, scale, 0 if window is None else int(window), algo, _ptr(cu_seqlens), n_seqs, max_new,
         counts, max_len, n_splits, ws_ptr, ws_bytes, dv, 1 if values_in_keys else 0,
         0 if chunk is None else int(chunk), _ptr(slopes), 1 if sink else 0, _ptr(sinks),
-        0.0 if softcap is None else float(softcap), _stream()))
+        0.0 if softcap is None else float(softcap), int(keep_first), _stream()))
 
 
 FUSED_DECODE_HEAD_DIMS = (64, 128, 192, 256)
@@ -936,12 +1019,13 @@ def decode_splits(pairs: int, n_cus: int, most: int) -> int:
 
 
 def attention_decode_fusable(dtype: torch.dtype, n_heads: int, n_kv_heads: int, head_dim: int, page: int,
-                             rot_dim: Optional[int], pairing: str = "halves") -> bool:
+                             rot_dim: Optional[int], pairing: str = "halves", partial: bool = False) -> bool:
     """Whether ``attention_decode_fused`` takes this layer: bfloat16 cache in pages of 64, a head
     size it has a kernel for, at most 16 query heads per kv head, and a rotation (if any) of the
-    whole head in pairs ``(i, i + head_dim / 2)``."""
+    whole head in pairs ``(i, i + head_dim / 2)`` (``partial``: or of the leading ``rot_dim`` values of it)."""
     return (dtype == torch.bfloat16 and page == 64 and head_dim in FUSED_DECODE_HEAD_DIMS
-            and n_heads // n_kv_heads <= 16 and (rot_dim is None or (rot_dim == head_dim and pairing == "halves")))
+            and n_heads // n_kv_heads <= 16
+            and (rot_dim is None or ((rot_dim == head_dim or partial) and pairing == "halves")))
 
 
 PREFILL_FUSED_PAGE = 64
@@ -1009,7 +1093,8 @@ def attention_decode_fused(qkv: torch.Tensor, out: torch.Tensor, k_cache: torch.
                            window: Optional[int] = None, workspace: Optional[torch.Tensor] = None,
                            max_len: int = 0, n_splits: int = 0, row_scale: Optional[RowScale] = None,
                            bias: Optional[torch.Tensor] = None, chunk: Optional[int] = None,
-                           slopes: Optional[torch.Tensor] = None, sink: bool = False) -> None:
+                           slopes: Optional[torch.Tensor] = None, sink: bool = False, sinks: Optional[torch.Tensor] = None,
+                           keep_first: int = 0, values_are_keys: bool = False) -> None:
     """A decode step's attention straight from the q/k/v projection ``qkv`` (float32
     ``[tokens, ld]``, or its split-K partial sums ``[splits, tokens, ld]``): per-head norm,
     rotation, append of the new key and value to the cache and attention over the cache in one
@@ -1017,11 +1102,17 @@ def attention_decode_fused(qkv: torch.Tensor, out: torch.Tensor, k_cache: torch.
     ``t`` of the block table).  ``workspace`` must not overlap ``qkv``.  ``row_scale``: the
     projection's operand lacked its norm's scale, which is applied to the projection's sums here.
     ``bias`` (32-bit, one number per column of a projection row) is added behind that scale;
-    ``chunk``, ``slopes`` and ``sink`` as in ``attention``."""
-    _dev(qkv, out, k_cache, v_cache, block_table, token_seq, token_pos, q_gain, k_gain, cos, sin, bias, slopes)
+    ``chunk``, ``slopes``, ``sink``, ``sinks`` and ``keep_first`` as in ``attention``.  The tables may be narrower than half a
+    head: its leading values turn.  ``values_are_keys``: the rows hold no value columns, the new value is the projected key
+    (with its bias) before norm and rotation."""
+    _dev(qkv, out, k_cache, v_cache, block_table, token_seq, token_pos, q_gain, k_gain, cos, sin, bias, slopes, sinks)
+    if sinks is not None:
+        _want(sinks, torch.float32, "sinks")
+        if sinks.numel() != n_heads or not sink:
+            raise KernelError("one sink per query head is needed, and the sink switched on")
     if bias is not None:
         _want(bias, torch.float32, "projection bias")
-        if bias.numel() < (n_heads + 2 * n_kv_heads) * head_dim and (write_kv or bias.numel() < n_heads * head_dim):
+        if bias.numel() < (n_heads + (1 if values_are_keys else 2) * n_kv_heads) * head_dim and (write_kv or bias.numel() < n_heads * head_dim):
             raise KernelError("the bias is shorter than a projection row")
     if slopes is not None:
         _want(slopes, torch.float32, "distance slopes")
@@ -1035,7 +1126,7 @@ def attention_decode_fused(qkv: torch.Tensor, out: torch.Tensor, k_cache: torch.
     n_tokens, ld = qkv.shape
     page = k_cache.shape[2]
     if not attention_decode_fusable(k_cache.dtype, n_heads, n_kv_heads, head_dim, page,
-                                    None if cos is None else 2 * cos.shape[-1]):
+                                    None if cos is None else 2 * cos.shape[-1], partial=True):
         raise KernelError(f"fused decode attention does not take this layer (cache {k_cache.dtype}, pages of {page}, "
                           f"head size {head_dim}, {n_heads} heads over {n_kv_heads})")
     if out.shape != (n_tokens, n_heads * head_dim) or out.dtype != k_cache.dtype:
@@ -1050,8 +1141,9 @@ def attention_decode_fused(qkv: torch.Tensor, out: torch.Tensor, k_cache: torch.
                 raise KernelError(f"head norm gain has {g.numel()} values for head size {head_dim}")
     if cos is not None:
         _want(cos, torch.float32, "rotation table")
-        if cos.shape != (n_tokens, head_dim // 2) or sin is None or sin.shape != cos.shape or sin.dtype != cos.dtype:
-            raise KernelError(f"rotation tables must be float32 {(n_tokens, head_dim // 2)}")
+        if cos.dim() != 2 or cos.shape[0] != n_tokens or not 0 < cos.shape[1] <= head_dim // 2 or sin is None \
+                or sin.shape != cos.shape or sin.dtype != cos.dtype:
+            raise KernelError(f"rotation tables must be float32 {(n_tokens, head_dim // 2)} or narrower")
     _want(block_table, torch.int32, "block table")
     _want(token_pos, torch.int32, "token position table")
     if token_seq is not None:
@@ -1071,7 +1163,8 @@ def attention_decode_fused(qkv: torch.Tensor, out: torch.Tensor, k_cache: torch.
         1 if write_kv else 0, _ptr(out), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), block_table.shape[1],
         _ptr(token_seq), _ptr(token_pos), n_tokens, n_heads, n_kv_heads, head_dim, page, scale,
         0 if window is None else int(window), max_len, n_splits, ws_ptr, ws_bytes, ssq_ptr, parts, row_eps, width,
-        _ptr(bias), 0 if chunk is None else int(chunk), _ptr(slopes), 1 if sink else 0, _stream()))
+        _ptr(bias), 0 if chunk is None else int(chunk), _ptr(slopes), 1 if sink else 0, _ptr(sinks), int(keep_first),
+        0 if cos is None else 2 * cos.shape[-1], 1 if values_are_keys else 0, _stream()))
 
 
 # ---- sampling ------------------------------------------------------------------------
@@ -1227,25 +1320,25 @@ def mlstm_scan(proj: torch.Tensor, q_col0: int, k_col0: int, v_col0: int, i_col0
         n_seqs, n_tokens, _ptr(out), n_heads, head_dim, v_head_dim, _stream()))
 
 
-HEAD_GATES = {"sigmoid": 0, "silu": 1}
+HEAD_GATES = {"sigmoid": 0, "silu": 1, None: 2}
 
 
-def head_norm_gate(o: torch.Tensor, g: torch.Tensor, g_col0: int, gain: Optional[torch.Tensor], out: torch.Tensor, n_heads: int,
-                   eps: float, gate: str = "sigmoid") -> None:
+def head_norm_gate(o: torch.Tensor, g: Optional[torch.Tensor], g_col0: int, gain: Optional[torch.Tensor], out: torch.Tensor, n_heads: int,
+                   eps: float, gate: Optional[str] = "sigmoid") -> None:
     """``out = rms_heads(o) * gain * act(g)``: every one of the ``n_heads`` equal parts of a row of the 32-bit
     ``o [T, n]`` divided by its own root mean square; ``g`` is columns ``g_col0 ..`` of a 32-bit matrix; ``act`` is
-    ``sigmoid`` or ``silu``; without ``gain`` the normed values are only gated."""
+    ``sigmoid`` or ``silu``; without ``gain`` the normed values are only gated; ``gate`` None (and ``g`` None): no gate."""
     _dev(o, g, gain, out)
-    for t, what in ((o, "norm input"), (g, "gate")) + (((gain, "norm gain"),) if gain is not None else ()):
+    for t, what in ((o, "norm input"),) + (((g, "gate"),) if g is not None else ()) + (((gain, "norm gain"),) if gain is not None else ()):
         _want(t, torch.float32, what)
-    if gate not in HEAD_GATES:
-        raise KernelError(f"unknown gate {gate!r}; known: {sorted(HEAD_GATES)}")
+    if gate not in HEAD_GATES or (gate is None) != (g is None):
+        raise KernelError(f"unknown gate {gate!r}, or its values are missing; known: {list(HEAD_GATES)}")
     rows, n = o.shape
-    if n % n_heads != 0 or (gain is not None and gain.numel() != n) or out.shape != o.shape or g.shape[0] != rows \
-            or g.shape[1] < g_col0 + n:
+    if n % n_heads != 0 or (gain is not None and gain.numel() != n) or out.shape != o.shape \
+            or (g is not None and (g.shape[0] != rows or g.shape[1] < g_col0 + n)):
         raise KernelError("head_norm_gate: sizes differ")
     _check("recurrent", library("recurrent").rocml_head_norm_gate(
-        _ptr(o), _ptr(g), g.shape[1], g_col0, _ptr(gain), _ptr(out), _code(out), rows, n_heads, n // n_heads, float(eps),
+        _ptr(o), _ptr(g), 0 if g is None else g.shape[1], g_col0, _ptr(gain), _ptr(out), _code(out), rows, n_heads, n // n_heads, float(eps),
         HEAD_GATES[gate], _stream()))
 
 
@@ -1253,15 +1346,18 @@ def decay_scan(q: torch.Tensor, q_col0: int, k: torch.Tensor, k_col0: int, v: to
                state: torch.Tensor, cu_seqlens: torch.Tensor, seq_slots: torch.Tensor, out: torch.Tensor,
                n_heads: int, head_dim: int, v_head_dim: int, head_decay: Optional[torch.Tensor] = None,
                decay: Optional[torch.Tensor] = None, decay_col0: int = 0, bonus: Optional[torch.Tensor] = None,
-               decay_offset: Optional[torch.Tensor] = None) -> None:
+               decay_offset: Optional[torch.Tensor] = None, gate_lower: Optional[torch.Tensor] = None,
+               gate_bias: Optional[torch.Tensor] = None) -> None:
     """A recurrence whose state per head, ``S [dk, dv]``, decays row by row, over the step's tokens, per sequence in
     order: ``S <- diag(w_t) S + k_t v_t^T``.  With ``head_decay`` (one number per head) ``w_t`` is that constant and
     the output reads the new state, ``o_t = S_t^T q_t``; with ``decay`` (per token and key channel, columns
     ``decay_col0 ..`` of a 32-bit matrix) and ``bonus`` ``u [H * dk]`` the output reads the state before the update,
     ``o_t = (S_(t-1) + diag(u) k_t v_t^T)^T q_t``.  With ``decay_offset`` (``[H * dk]``) ``decay`` holds logits ``x`` and the
-    decay is ``exp(-exp(x + decay_offset))``.  q, k, v are column ranges of 32-bit matrices ``[T, ld]``;
+    decay is ``exp(-exp(x + decay_offset))``.  With ``gate_lower`` ``l`` and ``gate_bias`` ``b`` (``[H * dk]`` each) ``k`` holds the
+    logits of a forget gate ``f = l + (1 - l) sigmoid(k + b)`` that decides what is written too, ``S <- diag(f) S + (1 - f) v^T``,
+    ``o = S^T silu(q)`` with the new state.  q, k, v are column ranges of 32-bit matrices ``[T, ld]``;
     ``state [slots, H, dv, dk]``; ``out [T, H * dv]``; all 32-bit."""
-    _dev(q, k, v, state, cu_seqlens, seq_slots, out, head_decay, decay, bonus, decay_offset)
+    _dev(q, k, v, state, cu_seqlens, seq_slots, out, head_decay, decay, bonus, decay_offset, gate_lower, gate_bias)
     for t, what in ((q, "queries"), (k, "keys"), (v, "values"), (state, "recurrent state"), (out, "recurrence output")):
         _want(t, torch.float32, what)
     n_tokens, n_seqs = out.shape[0], seq_slots.numel()
@@ -1270,19 +1366,23 @@ def decay_scan(q: torch.Tensor, q_col0: int, k: torch.Tensor, k_col0: int, v: to
     if out.shape != (n_tokens, n_heads * v_head_dim) or cu_seqlens.numel() != n_seqs + 1 \
             or any(t.dim() != 2 or t.shape[0] != n_tokens for t in (q, k, v)):
         raise KernelError("recurrence inputs, output or tables do not fit the step")
-    if (head_decay is None) == (decay is None) or (decay is None) != (bonus is None):
-        raise KernelError("the recurrence takes one decay per head, or a decay per token and channel together with a bonus")
+    if sum(t is not None for t in (head_decay, decay, gate_lower)) != 1 or (decay is None) != (bonus is None) \
+            or (gate_lower is None) != (gate_bias is None):
+        raise KernelError("the recurrence takes one decay per head, a decay per token and channel together with a bonus, or a "
+                          "forget gate's lower bound and bias")
     if decay_offset is not None and decay is None:
         raise KernelError("an offset of the decays' logits goes with decays per token")
     for t, n, what in ((head_decay, n_heads, "the heads' decays"), (bonus, n_heads * head_dim, "the bonus"),
-                       (decay_offset, n_heads * head_dim, "the offset of the decays' logits")):
+                       (decay_offset, n_heads * head_dim, "the offset of the decays' logits"),
+                       (gate_lower, n_heads * head_dim, "the gate's lower bound"), (gate_bias, n_heads * head_dim, "the gate's bias")):
         if t is not None and (t.dtype != torch.float32 or t.numel() != n):
             raise KernelError(f"{what} must be 32-bit with {n} numbers")
     if decay is not None and (decay.dtype != torch.float32 or decay.dim() != 2 or decay.shape[0] != n_tokens):
         raise KernelError("the decays per token must be a 32-bit matrix with a row per token")
     _check("recurrent", library("recurrent").rocml_decay_scan(
         _ptr(q), q.shape[1], q_col0, _ptr(k), k.shape[1], k_col0, _ptr(v), v.shape[1], v_col0, _ptr(decay),
-        0 if decay is None else decay.shape[1], decay_col0, _ptr(decay_offset), _ptr(head_decay), _ptr(bonus), _ptr(state),
+        0 if decay is None else decay.shape[1], decay_col0, _ptr(decay_offset), _ptr(head_decay), _ptr(bonus), _ptr(gate_lower),
+        _ptr(gate_bias), _ptr(state),
         state.shape[0],
         _ptr(cu_seqlens), _ptr(seq_slots), n_seqs, n_tokens, _ptr(out), n_heads, head_dim, v_head_dim, _stream()))
 

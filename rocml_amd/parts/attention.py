@@ -18,7 +18,9 @@ Further options: a learned sink per head (``exp(sink_h)`` in the denominator), a
 scores, and a short causal convolution per channel on q, k and v right behind their projection (32-bit, with
 the last ``taps - 1`` projected rows of a sequence kept as a state beside its keys and values).  The
 matrix-core kernels take the first two; the convolution is a kernel of its own in front of the
-norm-and-rotation kernel.
+norm-and-rotation kernel.  With a window, the first positions may stay visible (``keep_first``; the cache keeps
+their pages, and the kernels visit them before the window's), and the values may be the projected keys
+(``values_are_keys``: no value columns in the projection).  Every kernel here takes both.
 """
 from __future__ import annotations
 
@@ -59,9 +61,18 @@ class Attention(Mixer):
         if spec.distance_slopes is not None and len(spec.distance_slopes) != spec.n_heads:
             raise ConfigError(f"{len(spec.distance_slopes)} distance slopes for {spec.n_heads} heads")
         self.v_head_dim = spec.head_dim if spec.v_head_dim is None else spec.v_head_dim
+        self.keep_first = int(getattr(spec, "keep_first", 0)) if spec.window is not None else 0
+        if self.keep_first < 0:
+            raise ConfigError(f"kept first positions must not be negative, got {self.keep_first}")
+        self.values_are_keys = bool(getattr(spec, "values_are_keys", False))
+        if self.values_are_keys and (self.v_head_dim != spec.head_dim or getattr(spec, "conv", None) is not None
+                                     or getattr(spec, "qk_norm_span", "head") != "head"):
+            raise ConfigError("values that are the projected keys have the keys' size, and go without a convolution on q, k and v "
+                              "and without a norm over the whole projection")
         # what the matrix-core kernels do not know: such a layer runs the plain attention kernel
         self.extras = (self.v_head_dim != spec.head_dim or spec.chunk is not None
-                       or spec.distance_slopes is not None or spec.sink or getattr(spec, "softcap", None) is not None)
+                       or spec.distance_slopes is not None or spec.sink or getattr(spec, "softcap", None) is not None
+                       or self.keep_first > 0 or self.values_are_keys)
         self.sink_learned = bool(getattr(spec, "sink_learned", False))
         if self.sink_learned and not spec.sink:
             raise ConfigError("learned sinks need the sink switched on")
@@ -79,7 +90,7 @@ class Attention(Mixer):
         # themselves do not): a stretch of the query with its position, an output gate
         # (and a norm over a token's whole q and k rows, whose factors a kernel of their own forms first)
         self.separate_q = spec.q_temp is not None or spec.gate or self.span == "projection" or self.conv is not None \
-            or self.sink_learned or self.softcap is not None
+            or self.softcap is not None
         self.gate_per_head = bool(getattr(spec, "gate_per_head", False))
         if self.gate_per_head and not spec.gate:
             raise ConfigError("a gate per head needs the output gate switched on")
@@ -93,7 +104,7 @@ class Attention(Mixer):
         self.n_cus = ops.cu_count(ctx.device)
         self.q_dim = spec.n_heads * spec.head_dim
         self.kv_dim = spec.n_kv_heads * spec.head_dim
-        self.v_dim = spec.n_kv_heads * self.v_head_dim
+        self.v_dim = 0 if self.values_are_keys else spec.n_kv_heads * self.v_head_dim       # value columns of the projection
         self.o_dim = spec.n_heads * self.v_head_dim
         self.g_dim = 0 if not spec.gate else (spec.n_heads if self.gate_per_head else self.o_dim)
         self.position = build_position(spec.position, ctx) if spec.position is not None else None
@@ -119,12 +130,14 @@ class Attention(Mixer):
         s = self.spec
         specs = {"q_proj.weight": ParamSpec((self.q_dim, s.hidden)),
                  "k_proj.weight": ParamSpec((self.kv_dim, s.hidden)),
-                 "v_proj.weight": ParamSpec((self.v_dim, s.hidden)),
                  "o_proj.weight": ParamSpec((s.hidden, self.o_dim))}
+        if not self.values_are_keys:
+            specs["v_proj.weight"] = ParamSpec((self.v_dim, s.hidden))
         if s.bias:       # added in 32-bit to the products' sums
             specs.update({"q_proj.bias": ParamSpec((self.q_dim,), role="gain", init="normal"),
-                          "k_proj.bias": ParamSpec((self.kv_dim,), role="gain", init="normal"),
-                          "v_proj.bias": ParamSpec((self.v_dim,), role="gain", init="normal")})
+                          "k_proj.bias": ParamSpec((self.kv_dim,), role="gain", init="normal")})
+            if not self.values_are_keys:
+                specs["v_proj.bias"] = ParamSpec((self.v_dim,), role="gain", init="normal")
         if self.o_bias:
             specs["o_proj.bias"] = ParamSpec((s.hidden,), role="gain", init="normal")
         if s.qk_norm is not None and self.norm_learned:
@@ -145,12 +158,13 @@ class Attention(Mixer):
         # One [Q + 2 KV, hidden] matrix: q rows first, so a layer that only reads another
         # layer's cache multiplies by the leading Q rows.
         # (an output gate's rows come last: its projection rides in the same product)
-        self.w_qkv = torch.cat([tensors["q_proj.weight"], tensors["k_proj.weight"], tensors["v_proj.weight"]]
+        projected = ("q_proj", "k_proj") if self.values_are_keys else ("q_proj", "k_proj", "v_proj")
+        self.w_qkv = torch.cat([tensors[p + ".weight"] for p in projected]
                                + ([tensors["g_proj.weight"]] if self.spec.gate else []), dim=0).contiguous()
         self.w_o = tensors["o_proj.weight"]
         if self.spec.bias:
             # (an output gate's columns, which come last in the product, have no bias: zeros stand for it)
-            self.b_qkv = torch.cat([tensors["q_proj.bias"], tensors["k_proj.bias"], tensors["v_proj.bias"]]
+            self.b_qkv = torch.cat([tensors[p + ".bias"] for p in projected]
                                    + ([torch.zeros(self.g_dim, dtype=torch.float32, device=self.w_o.device)] if self.g_dim else [])
                                    ).contiguous()
         if self.o_bias:
@@ -177,7 +191,7 @@ class Attention(Mixer):
             elif w is None:
                 keys += n * s0 + n * (n + 1) // 2
             else:
-                keys += sum(min(s0 + i + 1, w) for i in range(n))
+                keys += sum(min(s0 + i + 1, w + self.keep_first) for i in range(n))
         return 2 * sum(new_counts) * self.matrix_elements() + \
             2 * self.spec.n_heads * (self.spec.head_dim + self.v_head_dim) * keys
 
@@ -190,7 +204,7 @@ class Attention(Mixer):
         rot = None if self.position is None else self.position.rot_dim
         # (blocks, slopes, a sink and biases ride in the fused kernel; a value head of another size does not)
         return not self.separate_q and self.v_head_dim == self.spec.head_dim and step.max_new == 1 and ops.attention_decode_fusable(
-            self.dtype, self.spec.n_heads, self.spec.n_kv_heads, self.spec.head_dim, ops.FUSED_DECODE_PAGE, rot, self.pairing)
+            self.dtype, self.spec.n_heads, self.spec.n_kv_heads, self.spec.head_dim, ops.FUSED_DECODE_PAGE, rot, self.pairing, partial=True)
 
     def _fused_prefill(self, step, cache) -> bool:
         """Whether the prompt kernel prepares its queries itself: it pays from about a thousand
@@ -208,9 +222,9 @@ class Attention(Mixer):
     def cache_request(self):
         s = self.spec
         if s.v_head_dim is None and s.chunk is None:
-            kv = KVCacheRequest(s.n_kv_heads, s.head_dim, s.window)
+            kv = KVCacheRequest(s.n_kv_heads, s.head_dim, s.window, keep_first=self.keep_first)
         else:
-            kv = KVCacheRequest(s.n_kv_heads, s.head_dim, s.window, v_head_dim=self.v_head_dim, chunk=s.chunk)
+            kv = KVCacheRequest(s.n_kv_heads, s.head_dim, s.window, v_head_dim=self.v_head_dim, chunk=s.chunk, keep_first=self.keep_first)
         if self.conv is None or self.conv == 1:
             return kv
         # the convolution's last taps - 1 inputs live beside the keys and values
@@ -289,7 +303,8 @@ class Attention(Mixer):
                                        max_len=step.max_len, n_splits=self._decode_splits(step, cache),
                                        row_scale=stream(step).row_scale,
                                        bias=None if self.b_qkv is None else self.b_qkv[:rows], chunk=s.chunk,
-                                       slopes=self.slopes, sink=s.sink)
+                                       slopes=self.slopes, sink=s.sink, sinks=self.sinks, keep_first=self.keep_first,
+                                       values_are_keys=self.values_are_keys)
         else:
             if stream(step).row_scale is not None:
                 raise ConfigError("the attention was handed an input without its norm's scale in a step it cannot scale")
@@ -318,13 +333,14 @@ class Attention(Mixer):
                 ops.qk_norm_rope_append(qkv, s.n_heads, s.n_kv_heads, s.head_dim, self.q_gain, self.k_gain, eps,
                                         cos, sin, rot, q, cache.k, cache.v, cache.block_table, step.token_seq,
                                         step.token_pos, write_kv=owns_cache, n_splits=max(splits, 1), pairing=self.pairing,
-                                        bias=bias, v_head_dim=self.v_head_dim, q_temp=s.q_temp, span_inv=span_inv, span_self=span_self)
+                                        bias=bias, v_head_dim=self.v_head_dim, q_temp=s.q_temp, span_inv=span_inv, span_self=span_self,
+                                        values_are_keys=self.values_are_keys)
                 ops.attention(q, o, cache.k, cache.v, cache.block_table, step.token_seq, step.token_pos,
                               s.n_heads, s.n_kv_heads, s.head_dim, s.scale, s.window, workspace=ws.scratch(),
                               cu_seqlens=step.cu_seqlens, max_new=step.max_new, q_counts=step.new_counts,
                               max_len=step.max_len, n_splits=self._decode_splits(step, cache),
                               v_head_dim=self.v_head_dim, chunk=s.chunk, slopes=self.slopes, sink=s.sink, sinks=self.sinks,
-                              softcap=self.softcap)
+                              softcap=self.softcap, keep_first=self.keep_first)
         if s.gate:
             ops.sigmoid_gate(o, qkv[:, rows - self.g_dim:rows], group=self.v_head_dim if self.gate_per_head else 1)
         if self.b_o is not None:

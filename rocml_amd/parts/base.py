@@ -57,12 +57,14 @@ class KVCacheRequest:
     """Keys and values per position: ``window`` is None when all positions are kept.
     ``v_head_dim``: size of a value head when it is not ``head_dim``.  ``chunk``: positions are
     cut into blocks of so many, counted from 0, and no query looks back beyond the start of its
-    own block (so earlier blocks' pages can be given back)."""
+    own block (so earlier blocks' pages can be given back).  ``keep_first``: with a window, the first so
+    many positions stay visible whatever their distance (their pages are kept)."""
     n_kv_heads: int
     head_dim: int
     window: Optional[int] = None
     v_head_dim: Optional[int] = None
     chunk: Optional[int] = None
+    keep_first: int = 0
 
 
 @dataclass(frozen=True)
@@ -86,6 +88,12 @@ class CompositeRequest:
     """What a mixer made of several parts asks for: one request per part (None for a part that
     keeps nothing; a part's request may be composite again).  Every part gets storage of its own
     and the mixer sees them as ``view.parts``, in this order."""
+    parts: Tuple[Optional[Any], ...]
+
+
+@dataclass(frozen=True)
+class CompositeView:
+    """Views of several parts put together from different cache lines, in the order of a composite request's parts."""
     parts: Tuple[Optional[Any], ...]
 
 
@@ -141,7 +149,11 @@ class NormHint:
 @dataclass(frozen=True)
 class FullNormHint(NormHint):
     """The same norm, for a consumer that wants the norm's whole output (not an operand that still lacks its rows' scale):
-    a kernel that completes the stream may write ``x / sqrt(mean(x^2) + eps) * gain`` in the compute type beside it."""
+    a kernel that completes the stream may write ``x / sqrt(mean(x^2) + eps) * gain`` in the compute type beside it.
+    ``conv``: what the consumer really reads is that output ``h`` plus its causal convolution over the sequence, and in this
+    step (one token per sequence) the kernel may form that too: ``(weights [taps, width], kept rows [slots, taps - 1, width],
+    slots of the step's sequences)``."""
+    conv: Optional[Tuple[torch.Tensor, torch.Tensor, torch.Tensor]] = None
 
 
 class Norm(Part):

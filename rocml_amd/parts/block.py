@@ -8,7 +8,12 @@
 ``a`` the block's ``residual_scale``; the sublayers read the stream itself.
 
 ``sublayer_norm`` norms a sublayer's output alone: ``x += norm(mixer(x))``, ``x += norm(ffn(x))`` and, if the
-layer has one, ``x += norm(side(x))``; the sublayers read the stream itself."""
+layer has one, ``x += norm(side(x))``; the sublayers read the stream itself.
+
+A block may put a short causal convolution between its first norm and its mixer (``InputConv``).  The rows it keeps
+are state of the block's own, beside what the mixer keeps: the block's cache request is then composite, ``(mixer,
+convolution)``.  A schedule entry that reads another entry's cache line shares the mixer's part and keeps its own
+convolution rows (``reader_request``, ``shared_view``, ``reader_view``)."""
 from __future__ import annotations
 
 from typing import Dict
@@ -19,12 +24,54 @@ import torch
 
 from ..config.spec import BlockSpec
 from ..errors import ConfigError
-from .base import BuildContext, FullNormHint, ParamSpec, Part
+from .base import BuildContext, CompositeRequest, CompositeView, FullNormHint, ParamSpec, Part
+from .input_conv import InputConv
 from .registry import build_feed_forward, build_mixer, build_norm, register_block
 from .residual import stream
 
 
-class PreNormBlock(Part):
+def _no_input_conv(spec: BlockSpec) -> None:
+    if getattr(spec, "input_conv", None) is not None:
+        raise ConfigError(f"a convolution on the mixer's input goes with a norm before the mixer, not with {spec.arrangement!r}")
+
+
+class ConvInput:
+    """The part of a block that holds the convolution on the mixer's input, if the layer has one."""
+    input_conv = None
+
+    def _build_input_conv(self, spec: BlockSpec, ctx: BuildContext) -> None:
+        if getattr(spec, "input_conv", None) is not None:
+            self.input_conv = self.children["input_conv"] = InputConv(spec.mixer_norm.size, spec.input_conv, ctx)
+
+    def cache_request(self):
+        if self.input_conv is None:
+            return self.mixer.cache_request()
+        return CompositeRequest((self.mixer.cache_request(), self.input_conv.cache_request()))
+
+    def reader_request(self):
+        """What an execution that reads another entry's cache line still keeps for itself (None: nothing)."""
+        if self.input_conv is None or self.input_conv.cache_request() is None:
+            return None
+        return CompositeRequest((None, self.input_conv.cache_request()))
+
+    def shared_view(self, view):
+        """The part of this block's line that another entry's mixer may read."""
+        return view if self.input_conv is None or view is None else view.parts[0]
+
+    def reader_view(self, shared, own):
+        """The view for an execution that reads another entry's line: that line's shared part and what it keeps itself."""
+        if self.input_conv is None:
+            return shared
+        return CompositeView((shared, None if own is None else own.parts[1]))
+
+    def _views(self, cache):
+        """``(the mixer's view, the convolution's)``."""
+        if self.input_conv is None:
+            return cache, None
+        return (None, None) if cache is None else (cache.parts[0], cache.parts[1])
+
+
+class PreNormBlock(ConvInput, Part):
     def __init__(self, spec: BlockSpec, ctx: BuildContext):
         self.dtype = ctx.dtype
         self.hidden = spec.mixer_norm.size
@@ -33,6 +80,7 @@ class PreNormBlock(Part):
         if spec.ffn is not None:          # a layer may be its mixer alone
             self.children["ffn_norm"] = build_norm(spec.ffn_norm, ctx)
             self.children["ffn"] = build_feed_forward(spec.ffn, ctx)
+        self._build_input_conv(spec, ctx)
         self.mixer_norm = self.children["mixer_norm"]
         self.mixer = self.children["mixer"]
         self.ffn_norm = self.children.get("ffn_norm")
@@ -49,23 +97,24 @@ class PreNormBlock(Part):
             prefix = name + "."
             child.bind({k[len(prefix):]: v for k, v in tensors.items() if k.startswith(prefix)})
 
-    def cache_request(self):
-        return self.mixer.cache_request()
-
     def flops(self, new_counts, starts) -> int:
         return self.mixer.flops(new_counts, starts) + (self.ffn.flops(new_counts, starts) if self.ffn is not None else 0)
 
     def activation_bytes(self, n_tokens: int) -> int:
         size = 2 if self.dtype == torch.bfloat16 else 4
         return n_tokens * self.hidden * size + self.mixer.activation_bytes(n_tokens) + \
-            (self.ffn.activation_bytes(n_tokens) if self.ffn is not None else 0)
+            (self.ffn.activation_bytes(n_tokens) if self.ffn is not None else 0) + \
+            (self.input_conv.activation_bytes(n_tokens) if self.input_conv is not None else 0)
 
     takes_pending = True      # forward() may be handed a stream that still lacks deferred sums
     takes_next_norm = True    # forward() accepts the hint of the norm that reads the stream after it
 
-    def entry_hint(self, step):
+    def entry_hint(self, step, cache=None):
         """The norm this block reads the residual stream with first, for the product that completes
-        the stream before it, if the block's mixer can apply the norm's scale itself in this step."""
+        the stream before it, if the block's mixer can apply the norm's scale itself in this step.
+        ``cache``: the block's view in this step."""
+        if self.input_conv is not None:
+            return None               # the convolution needs the normed rows themselves
         return self._hint(step, self.mixer_norm, self.mixer)
 
     def forward(self, step, x: torch.Tensor, cache, owns_cache: bool, next_norm=None) -> None:
@@ -77,7 +126,10 @@ class PreNormBlock(Part):
         if not getattr(self.mixer, "adds_only", False):
             ws.flush_pending()
         rs.next_norm = self._hint(step, self.ffn_norm, self.ffn) if self.ffn is not None else next_norm
-        self.mixer.forward(step, xn, x, cache, owns_cache)
+        mixer_view, conv_view = self._views(cache)
+        if self.input_conv is not None:
+            xn = self.input_conv.forward(step, xn, conv_view)
+        self.mixer.forward(step, xn, x, mixer_view, owns_cache)
         rs.next_norm = None
         if self.ffn is None:
             rs.row_scale = None
@@ -133,6 +185,7 @@ class PostNormBlock(Part):
     takes_next_norm = False
 
     def __init__(self, spec: BlockSpec, ctx: BuildContext):
+        _no_input_conv(spec)
         self.dtype = ctx.dtype
         self.hidden = spec.mixer_norm.size
         self.alpha = float(spec.residual_scale)
@@ -155,6 +208,7 @@ class PostNormBlock(Part):
     param_specs = PreNormBlock.param_specs
     bind = PreNormBlock.bind
     cache_request = PreNormBlock.cache_request
+    input_conv = None
     flops = PreNormBlock.flops
 
     def activation_bytes(self, n_tokens: int) -> int:
@@ -223,6 +277,7 @@ class SublayerNormBlock(Part):
     takes_next_norm = False
 
     def __init__(self, spec: BlockSpec, ctx: BuildContext):
+        _no_input_conv(spec)
         self.dtype = ctx.dtype
         self.hidden = spec.mixer_norm.size
         self.children = {"mixer_norm": build_norm(spec.mixer_norm, ctx),
@@ -247,6 +302,7 @@ class SublayerNormBlock(Part):
     param_specs = PreNormBlock.param_specs
     bind = PreNormBlock.bind
     cache_request = PreNormBlock.cache_request
+    input_conv = None
 
     def flops(self, new_counts, starts) -> int:
         return sum(part.flops(new_counts, starts) for part in (self.mixer, self.ffn, self.side) if part is not None)
@@ -316,17 +372,18 @@ class SublayerNormBlock(Part):
 register_block("sublayer_norm", SublayerNormBlock)
 
 
-class SandwichNormBlock(Part):
+class SandwichNormBlock(ConvInput, Part):
     """``x += out_norm1(mixer(norm1(x)))``, ``x += out_norm2(ffn(norm2(x)))``: a norm before and one after every
     sublayer (the feed-forward may be absent).  The first norm of a sublayer writes the products' operand in the
     compute type; the sublayer writes its result to a buffer of the block; one kernel then norms that buffer and
     adds it to the 32-bit stream (it takes a product's K pieces in place of the buffer) and, in the same pass over
     the row, forms the norm that reads the stream next: the feed-forward's first norm behind the mixer, the next
-    layer's first norm behind the feed-forward when that layer is of this kind (``entry_hint``).  The norms are
-    root-mean-square norms with a gain."""
+    layer's first norm behind the feed-forward when that layer is of this kind (``entry_hint``), in a step of one token
+    per sequence together with the convolution on that layer's input.  The norms are root-mean-square norms with a gain."""
     takes_pending = False
     takes_next_norm = True
-    _READY = "sandwich_norm.operand"      # in step.memo: (stream, gain, operand) of a norm that the kernel before formed
+    # in step.memo: (stream, gain, operand, whether the convolution on it is in it) of a norm that the kernel before formed
+    _READY = "sandwich_norm.operand"
 
     def __init__(self, spec: BlockSpec, ctx: BuildContext):
         if spec.mixer_out_norm is None or (spec.ffn is not None and (spec.ffn_norm is None or spec.ffn_out_norm is None)):
@@ -340,6 +397,7 @@ class SandwichNormBlock(Part):
             self.children["ffn_norm"] = build_norm(spec.ffn_norm, ctx)
             self.children["ffn"] = build_feed_forward(spec.ffn, ctx)
             self.children["ffn_out_norm"] = build_norm(spec.ffn_out_norm, ctx)
+        self._build_input_conv(spec, ctx)
         self.mixer = self.children["mixer"]
         self.ffn = self.children.get("ffn")
         for name in ("mixer_out_norm", "ffn_out_norm"):
@@ -352,33 +410,40 @@ class SandwichNormBlock(Part):
 
     param_specs = PreNormBlock.param_specs
     bind = PreNormBlock.bind
-    cache_request = PreNormBlock.cache_request
     flops = PreNormBlock.flops
 
     def activation_bytes(self, n_tokens: int) -> int:
         size = 2 if self.dtype == torch.bfloat16 else 4
         return n_tokens * self.hidden * (size + 4) + self.mixer.activation_bytes(n_tokens) + \
-            (self.ffn.activation_bytes(n_tokens) if self.ffn is not None else 0)
+            (self.ffn.activation_bytes(n_tokens) if self.ffn is not None else 0) + \
+            (self.input_conv.activation_bytes(n_tokens) if self.input_conv is not None else 0)
 
-    def entry_hint(self, step):
-        """The norm this block reads the stream with first, for the kernel that completes the stream before it."""
+    def entry_hint(self, step, cache=None):
+        """The norm this block reads the stream with first, for the kernel that completes the stream before it (and
+        the convolution on its output, where that kernel can form it).  ``cache``: the block's view in this step."""
         norm = self.children["mixer_norm"]
         gain = getattr(norm, "gain", None)
         if gain is None or not hasattr(norm, "eps") or getattr(norm, "centred", False):
             return None
-        return FullNormHint(gain, float(norm.eps), self.hidden)
+        conv = None if self.input_conv is None else self.input_conv.in_norm(step, self._views(cache)[1])
+        return FullNormHint(gain, float(norm.eps), self.hidden, conv=conv)
 
-    def _sublayer(self, step, x, norm, run, out_norm, following) -> None:
-        """``following``: a ``FullNormHint`` of the norm that reads the stream after this sublayer, or None."""
+    def _sublayer(self, step, x, norm, run, out_norm, following, conv_view=None) -> None:
+        """``following``: a ``FullNormHint`` of the norm that reads the stream after this sublayer, or None.
+        ``conv_view``: given for the sublayer whose input passes the block's convolution: ``(the rows' view,)``."""
         ws = step.workspace
         rs = stream(step)
         ready = step.memo.pop(self._READY, None)
         gain = getattr(norm, "gain", None)
         if ready is not None and gain is not None and ready[0] == x.data_ptr() and ready[1] == gain.data_ptr():
             xn = ready[2]           # the kernel that completed the stream formed this norm on its way
+            convolved = ready[3]
         else:
             xn = ws.get("block.xn", tuple(x.shape), self.dtype)
             norm.forward(x, xn)
+            convolved = False
+        if conv_view is not None and not convolved:
+            xn = self.input_conv.forward(step, xn, conv_view[0])
         y = ws.get("block.sublayer", tuple(x.shape), torch.float32)
         rs.overwrite = rs.defer_overwrite = True
         run(xn, y)
@@ -389,8 +454,8 @@ class SandwichNormBlock(Part):
             # (the sublayer is done with its operand: the buffer takes the next one)
             nxt = ws.get("block.xn", tuple(x.shape), self.dtype)
             ops.norm_add(x, y, out_norm.gain, None, out_norm.eps, layer=False, partials=partials, replace=replace, copy=nxt,
-                         next_gain=following.gain, next_eps=following.eps)
-            step.memo[self._READY] = (x.data_ptr(), following.gain.data_ptr(), nxt)
+                         next_gain=following.gain, next_eps=following.eps, conv=following.conv)
+            step.memo[self._READY] = (x.data_ptr(), following.gain.data_ptr(), nxt, following.conv is not None)
         else:
             ops.norm_add(x, y, out_norm.gain, None, out_norm.eps, layer=False, partials=partials, replace=replace)
 
@@ -404,8 +469,10 @@ class SandwichNormBlock(Part):
                 n2 = self.children["ffn_norm"]
                 if getattr(n2, "gain", None) is not None and hasattr(n2, "eps") and not getattr(n2, "centred", False):
                     inner = FullNormHint(n2.gain, float(n2.eps), self.hidden)
-            self._sublayer(step, x, self.children["mixer_norm"], lambda xn, y: self.mixer.forward(step, xn, y, cache, owns_cache),
-                           self.children["mixer_out_norm"], inner if self.ffn is not None else next_norm)
+            mixer_view, conv_rows = self._views(cache)
+            self._sublayer(step, x, self.children["mixer_norm"], lambda xn, y: self.mixer.forward(step, xn, y, mixer_view, owns_cache),
+                           self.children["mixer_out_norm"], inner if self.ffn is not None else next_norm,
+                           conv_view=None if self.input_conv is None else (conv_rows,))
             if self.ffn is not None:
                 self._sublayer(step, x, self.children["ffn_norm"], lambda xn, y: self.ffn.forward(step, xn, y),
                                self.children["ffn_out_norm"], next_norm)

@@ -22,6 +22,11 @@ latent with its rotated part, output gate), one kernel that norms both latents, 
 appends to the cache, the product ``W_uq``, the rotation of the queries' rotated parts, the
 per-head products with ``W_uk^T``, the attention, the per-head products with ``W_uv`` (the gate is
 their epilogue in bfloat16), and the output product whose epilogue is the residual sum.
+
+The gate is one number per value or one per head.  A layer without rows of its own (``own_rows`` false) has no
+key/value latent in its first product and reads the rows that another layer appended earlier in the same step; its
+expansions, queries and gate are its own.  The rotated parts turn in pairs of halves or of neighbours, as the position
+encoding says.
 """
 from __future__ import annotations
 
@@ -58,15 +63,22 @@ class LatentAttention(Mixer):
         self.spec = spec
         self.dtype = ctx.dtype
         self.position = build_position(spec.position, ctx)
-        if getattr(self.position, "pairing", "halves") != "halves" or self.position.rot_dim > spec.rot_dim:
-            raise ConfigError("the rotated part turns in pairs (i, i + n/2) of its first n numbers, n at most its size")
+        self.pairing = getattr(self.position, "pairing", "halves")
+        if self.pairing not in ops.ROPE_PAIRINGS or self.position.rot_dim > spec.rot_dim:
+            raise ConfigError("the rotated part turns in pairs of its first n numbers, n at most its size")
+        self.own_rows = bool(getattr(spec, "own_rows", True))
+        self.gate_per_head = bool(getattr(spec, "gate_per_head", False))
+        if self.gate_per_head and not spec.gate:
+            raise ConfigError("a gate per head needs the output gate switched on")
         self.graph_safe = getattr(self.position, "graph_safe", True)
         self.prompt_graph_safe = self.graph_safe and getattr(self.position, "prompt_graph_safe", False)
         self.qk_dim = spec.head_dim + spec.rot_dim             # a head's query as the projection gives it
         self.row = spec.kv_rank + spec.rot_dim                 # a cache row, and a head's query as the attention takes it
         self.o_dim = spec.n_heads * spec.v_head_dim
-        # columns of the first projection: query latent, key/value latent, rotated key part, gate
-        self.first_cols = spec.q_rank + self.row + (self.o_dim if spec.gate else 0)
+        # columns of the first projection: query latent, key/value latent and rotated key part (if the rows are its own), gate
+        self.g_dim = 0 if not spec.gate else (spec.n_heads if self.gate_per_head else self.o_dim)
+        self.g_col = spec.q_rank + (self.row if self.own_rows else 0)
+        self.first_cols = self.g_col + self.g_dim
         self.w_first: Optional[torch.Tensor] = None
         self.w_uq: Optional[torch.Tensor] = None
         self.w_uk_t: Optional[torch.Tensor] = None
@@ -82,18 +94,19 @@ class LatentAttention(Mixer):
         specs = {"dq.weight": ParamSpec((s.q_rank, s.hidden)),
                  "dq_norm.weight": ParamSpec((s.q_rank,), role="gain", init="gain"),
                  "uq.weight": ParamSpec((s.n_heads * self.qk_dim, s.q_rank)),
-                 "dkv.weight": ParamSpec((self.row, s.hidden)),
-                 "dkv_norm.weight": ParamSpec((s.kv_rank,), role="gain", init="gain"),
                  "uk.weight": ParamSpec((s.n_heads * s.head_dim, s.kv_rank)),
                  "uv.weight": ParamSpec((self.o_dim, s.kv_rank)),
                  "o_proj.weight": ParamSpec((s.hidden, self.o_dim))}
+        if self.own_rows:
+            specs["dkv.weight"] = ParamSpec((self.row, s.hidden))
+            specs["dkv_norm.weight"] = ParamSpec((s.kv_rank,), role="gain", init="gain")
         if s.gate:
-            specs["g.weight"] = ParamSpec((self.o_dim, s.hidden))
+            specs["g.weight"] = ParamSpec((self.g_dim, s.hidden))
         return specs
 
     def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
         s = self.spec
-        first = [tensors["dq.weight"], tensors["dkv.weight"]] + ([tensors["g.weight"]] if s.gate else [])
+        first = [tensors["dq.weight"]] + ([tensors["dkv.weight"]] if self.own_rows else []) + ([tensors["g.weight"]] if s.gate else [])
         self.w_first = torch.cat(first, dim=0).contiguous()
         self.w_uq = tensors["uq.weight"]
         # per head [kv_rank, head_dim]: the transposed key expansion, applied to the queries
@@ -101,7 +114,7 @@ class LatentAttention(Mixer):
         self.w_uv = tensors["uv.weight"].view(s.n_heads, s.v_head_dim, s.kv_rank).contiguous()
         self.w_o = tensors["o_proj.weight"]
         self.q_gain = tensors["dq_norm.weight"]
-        self.kv_gain = tensors["dkv_norm.weight"]
+        self.kv_gain = tensors["dkv_norm.weight"] if self.own_rows else None
         if self._expandable():
             # One matrix that turns a cache row [c, k_r] into every head's key [W_uk,a c, k_r] and value
             # [W_uv,a c, zeros up to the key's size]: rows of W_uk and W_uv against c, an identity against k_r.
@@ -146,12 +159,18 @@ class LatentAttention(Mixer):
         return total
 
     def cache_request(self) -> LatentCacheRequest:
+        if not self.own_rows:
+            raise ConfigError("a latent attention without rows of its own runs on another layer's cache")
         return LatentCacheRequest(self.row, self.spec.window)
 
     def forward(self, step, xn, x_accum, cache, owns_cache: bool) -> None:
         s = self.spec
         n = step.n_tokens
         ws = step.workspace
+        if owns_cache and not self.own_rows:
+            raise ConfigError("a latent attention without rows of its own runs on another layer's cache")
+        if cache.k.shape[2] != self.row:
+            raise ConfigError(f"the cache's rows hold {cache.k.shape[2]} numbers, the layer reads {self.row}")
         if stream(step).row_scale is not None:
             raise ConfigError("the latent attention was handed an input without its norm's scale")
         first = ws.get("latent.first", (n, self.first_cols), torch.float32)
@@ -161,7 +180,7 @@ class LatentAttention(Mixer):
         cq = ws.get("latent.cq", (n, s.q_rank), self.dtype)
         ops.latent_prepare(first, s.q_rank, s.kv_rank, s.rot_dim, dims, self.q_gain, self.kv_gain, s.q_norm.eps,
                            cos, sin, cq, cache.k, cache.block_table, step.token_seq, step.token_pos,
-                           write_cache=owns_cache)
+                           write_cache=owns_cache, pairing=self.pairing)
         q = ws.get("latent.q", (n, s.n_heads * self.qk_dim), torch.float32)
         ops.gemm(cq, self.w_uq, q, workspace=ws.scratch())
         # the queries as the attention takes them: per head [W_uk^T q^n, rotated q^r]
@@ -172,20 +191,21 @@ class LatentAttention(Mixer):
             self._expanded_prompt(step, q, first, cos, sin, dims, cache, x_accum)
             return
         ops.gemm_batched(q, self.qk_dim, self.w_uk_t, qa, self.row)
-        ops.rope_heads(q, s.n_heads, self.qk_dim, s.head_dim, s.rot_dim, dims, cos, sin, qa, self.row, s.kv_rank)
+        ops.rope_heads(q, s.n_heads, self.qk_dim, s.head_dim, s.rot_dim, dims, cos, sin, qa, self.row, s.kv_rank,
+                       pairing=self.pairing)
         ol = ws.get("latent.ol", (n, s.n_heads * s.kv_rank), self.dtype)
         ops.attention(qa, ol, cache.k.unsqueeze(1), None, cache.block_table, step.token_seq, step.token_pos,
                       s.n_heads, 1, self.row, s.scale, s.window, workspace=ws.scratch(),
                       cu_seqlens=step.cu_seqlens, max_new=step.max_new, q_counts=step.new_counts,
                       max_len=step.max_len, v_head_dim=s.kv_rank, values_in_keys=True)
         o = ws.get("latent.o", (n, self.o_dim), self.dtype)
-        gate = first[:, s.q_rank + self.row:] if s.gate else None
+        gate = first[:, self.g_col:] if s.gate else None
         if gate is not None and ops.gemm_batched_gate_fusable(self.w_uv, ol) and s.kv_rank % 8 == 0:
             ops.gemm_batched(ol, s.kv_rank, self.w_uv, o, s.v_head_dim, gate=gate)      # the gate is the product's epilogue
         else:
             ops.gemm_batched(ol, s.kv_rank, self.w_uv, o, s.v_head_dim)
             if gate is not None:
-                ops.sigmoid_gate(o, gate)
+                ops.sigmoid_gate(o, gate, group=s.v_head_dim if self.gate_per_head else 1)
         stream(step).add_product(o, self.w_o, x_accum)
 
 
@@ -220,13 +240,14 @@ class LatentAttention(Mixer):
         ops.qk_norm_rope_append(kv, 0, H, D, None, None, 1.0, None, None, 0, None, ks, vs, table_id[:, :pages].contiguous(),
                                 seq_id[:pages * page], pos_id[:pages * page], write_kv=True)
         qf = ws.get("latent.x.q", (n, H * D), self.dtype)
-        ops.rope_heads(q, H, D, s.head_dim, s.rot_dim, dims, cos, sin, qf, D, 0, lead=s.head_dim)
+        ops.rope_heads(q, H, D, s.head_dim, s.rot_dim, dims, cos, sin, qf, D, 0, lead=s.head_dim,
+                       pairing=self.pairing)
         of = ws.get("latent.x.o", (n, H * D), self.dtype)
         ops.attention(qf, of, ks, vs, table, step.token_seq, step.token_pos, H, H, D, s.scale, s.window,
                       workspace=ws.scratch(), cu_seqlens=step.cu_seqlens, max_new=step.max_new, q_counts=step.new_counts,
                       max_len=step.max_len)
         o = ws.get("latent.o", (n, self.o_dim), self.dtype)
-        ops.gate_heads(of, D, first[:, s.q_rank + self.row:] if s.gate else None, o, H, s.v_head_dim)
+        ops.gate_heads(of, D, first[:, self.g_col:] if s.gate else None, o, H, s.v_head_dim)
         stream(step).add_product(o, self.w_o, x_accum)
 
 

@@ -3,7 +3,10 @@
 are one product over the concatenated weight; the residual sum is the down product's
 epilogue.  ``act`` is the spec's: ``silu`` and ``relu`` are epilogues of the gate/up product,
 ``gelu_tanh`` and ``sigmoid_1702`` (``g sigmoid(1.702 g)``) run as a kernel of their own behind it, and so
-does any layer with a ``limit`` on gate and up values or an offset added to the up values."""
+does any layer with a ``limit`` on gate and up values or an offset added to the up values.
+
+``Mlp`` is the feed-forward without a gate, ``down(act(up(x)))``; the squared rectifier is the epilogue of the up
+product in bfloat16, other activations and the 32-bit path run a kernel behind it."""
 from __future__ import annotations
 
 from typing import Dict, Optional
@@ -11,7 +14,7 @@ from typing import Dict, Optional
 import torch
 
 from .. import ops
-from ..config.spec import GatedMlpSpec
+from ..config.spec import GatedMlpSpec, MlpSpec
 from ..errors import ConfigError
 from .base import BuildContext, FeedForward, ParamSpec
 from .registry import register_feed_forward
@@ -79,3 +82,46 @@ class GatedMlp(FeedForward):
 
 
 register_feed_forward("gated_mlp", GatedMlp)
+
+
+class Mlp(FeedForward):
+    adds_only = True
+    prompt_graph_safe = True
+
+    def __init__(self, spec: MlpSpec, ctx: BuildContext):
+        if spec.activation not in ops.ACTIVATIONS:
+            raise ConfigError(f"activation {spec.activation!r} is not supported; known: {sorted(ops.ACTIVATIONS)}")
+        self.spec = spec
+        self.dtype = ctx.dtype
+        self.fused = spec.activation in ops.GEMM_EPILOGUES and ctx.dtype == torch.bfloat16 and spec.hidden % 8 == 0
+        self.w_up: Optional[torch.Tensor] = None
+        self.w_down: Optional[torch.Tensor] = None
+
+    def param_specs(self) -> Dict[str, ParamSpec]:
+        s = self.spec
+        return {"up_proj.weight": ParamSpec((s.intermediate, s.hidden)), "down_proj.weight": ParamSpec((s.hidden, s.intermediate))}
+
+    def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
+        self.w_up, self.w_down = tensors["up_proj.weight"], tensors["down_proj.weight"]
+
+    def activation_bytes(self, n_tokens: int) -> int:
+        size = 2 if self.dtype == torch.bfloat16 else 4
+        return n_tokens * self.spec.intermediate * (size + (0 if self.fused else 4))
+
+    def forward(self, step, xn, x_accum) -> None:
+        s = self.spec
+        n = step.n_tokens
+        ws = step.workspace
+        if stream(step).row_scale is not None:
+            raise ConfigError("the feed-forward was handed an input without its norm's scale")
+        h = ws.get("mlp.h", (n, s.intermediate), self.dtype)
+        if self.fused:
+            ops.gemm(xn, self.w_up, h, workspace=ws.scratch(), epilogue=s.activation)
+        else:
+            z = ws.get("mlp.up", (n, s.intermediate), torch.float32)
+            ops.gemm(xn, self.w_up, z, workspace=ws.scratch())
+            ops.activate(z, h, s.activation)
+        stream(step).add_product(h, self.w_down, x_accum)
+
+
+register_feed_forward("mlp", Mlp)

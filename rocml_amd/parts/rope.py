@@ -7,7 +7,9 @@ With a ``stretch`` (factor ``s``, original length ``L``, ``fast``, ``slow``) the
 down for contexts beyond ``L`` positions: ``d(t) = rot_dim ln(L / (2 pi t)) / (2 ln theta)``,
 ``lo = max(floor(d(fast)), 0)``, ``hi = min(ceil(d(slow)), rot_dim - 1)``,
 ``r_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1)``, ``f_i <- f_i / s * r_i + f_i (1 - r_i)``, and every
-cosine and sine is multiplied by ``0.1 ln(s) + 1``."""
+cosine and sine is multiplied by ``0.1 ln(s) + 1``.
+
+The spec's ``pairing`` says which values turn together; the tables are the same either way."""
 from __future__ import annotations
 
 import math
@@ -29,6 +31,9 @@ class RopeNeox(PositionEncoding):
             raise ConfigError(f"rotary width {spec.rot_dim} must be even and at most the head size {spec.head_dim}")
         self.spec = spec
         self.rot_dim = spec.rot_dim
+        self.pairing = getattr(spec, "pairing", "halves")
+        if self.pairing not in ops.ROPE_PAIRINGS:
+            raise ConfigError(f"unknown rotation pairing {self.pairing!r}; known: {sorted(ops.ROPE_PAIRINGS)}")
         half = spec.rot_dim // 2
         inv = [float(spec.theta) ** (-2.0 * i / spec.rot_dim) for i in range(half)]
         self.magnitude = 1.0
