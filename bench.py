@@ -2,7 +2,7 @@
 """Decode and prefill speed of the Qwen3 shapes with random bfloat16 weights on one MI355X.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--model qwen3-8b|qwen3-14b|qwen3-32b]
-    python bench.py --design dokulix|felovik|sogavik|roravik [--design-size 2b|8b|14b] [--layers N]
+    python bench.py --design dokulix|felovik|sogavik|roravik|kakalorn [--design-size 2b|8b|14b] [--layers N]
 
 The default run is the Qwen3-8B shape.  A step is one decode step of a batch of 8 sequences,
 each with a 2,048-token random prompt in the cache (context length 4,096): the engine's step
@@ -38,6 +38,11 @@ head beside a recurrence with a decay per token and channel in the even layers, 
 feed-forwards and routed experts with a shared expert in turn; a norm before and after every sublayer) beside the
 Felovik model of the same sizes, the library's closest design (a pair of mixers with a recurrence in every layer,
 dense feed-forwards and routed experts in turn).
+``--design kakalorn`` measures a Kakalorn model (latent attention with a gate per head, of which every second layer runs on
+another's rows, windowed attention whose values are its keys, with kept first positions and sinks, and a recurrence whose
+forget gate writes, in turn; a convolution on every mixer's input, a norm before and after every sublayer, squared-rectifier
+feed-forwards) beside the two closest designs at equal size: Dokulix (latent attention, biased attention with a sink, dense
+feed-forwards) and Roravik (a recurrence with a decay, norms before and after every sublayer).
 
 The workloads follow the reference's bench (rocml-cli/src/cmd_bench.rs:79-243): synthetic
 prompts, greedy, no stop token, warm-up first; times are taken around synchronised steps.
@@ -83,12 +88,19 @@ def felovik_config(z: dict, n_layers: int):
             "layers": [{"type": "parallel", "mixer": mixer, "mlp": dense if i % 2 == 0 else moe} for i in range(n_layers)]}
 
 
-COMPANION = {"dokulix": "qwen3", "felovik": "qwen3", "sogavik": "felovik", "roravik": "felovik"}     # the closest model each design is measured beside
+# the closest models each design is measured beside
+COMPANIONS = {"dokulix": ("qwen3",), "felovik": ("qwen3",), "sogavik": ("felovik",), "roravik": ("felovik",), "kakalorn": ("dokulix", "roravik")}
 
 
 def design_configs(size: dict, n_layers: int, design: str = "dokulix"):
-    """config.json of the design's model and of its companion of equal size."""
+    """config.json of the design's model and of its companions of equal size."""
     z = size
+    if design == "kakalorn":
+        from rocml_amd.config.catalog import kakalorn_config
+        # the companions' latent sizes, window and heads; recurrence heads of 128 with an inner width equal to the model's
+        mine = kakalorn_config(z["vocab"], z["width"], z["heads"], z["kv_heads"], z["dim"], z["window"], 4, z["heads"], z["dim"],
+                               z["rot_dim"], z["q_rank"], z["kv_rank"], z["width"] // 128, 128, z["ff"], n_layers)
+        return mine, design_configs(z, n_layers, "dokulix")[0], design_configs(z, n_layers, "roravik")[0]
     if design == "sogavik":
         from rocml_amd.config.catalog import sogavik_config
         return (sogavik_config(z["vocab"], z["width"], z["heads"], z["kv_heads"], z["dim"], z["window"], z["width"] // 128, 128,
@@ -136,8 +148,8 @@ def run_design(args) -> int:
     rng = np.random.default_rng(0)
     dtype = torch.bfloat16 if args.dtype == "bfloat16" else torch.float32
     results = {}
-    other_name = COMPANION[args.design]
-    for name, raw in zip((args.design, other_name), design_configs(DESIGN_SIZES[args.design_size], n_layers, args.design)):
+    others = COMPANIONS[args.design]
+    for name, raw in zip((args.design,) + others, design_configs(DESIGN_SIZES[args.design_size], n_layers, args.design)):
         model = random_model(raw, seed=0, dtype=args.dtype, device="cuda:0")
         vocab = model.spec.vocab
         engine = Engine(model, max_tokens=batch * CONTEXT, max_seqs=batch, max_step_tokens=8192)
@@ -180,17 +192,18 @@ def run_design(args) -> int:
                          "params_m": round(model.n_params() / 1e6, 1), "launches": rows}
         del engine, model, gen
         torch.cuda.empty_cache()
-    mine, other = results[args.design], results[other_name]
-    out = {"metric": f"{args.design} beside the {other_name} shape of equal size ({args.design_size}, {n_layers} layers, "
+    mine = results[args.design]
+    out = {"metric": f"{args.design} beside the {' and '.join(others)} shape of equal size ({args.design_size}, {n_layers} layers, "
                      f"{args.dtype}): decode tok/s at batch {batch} over {PROMPT_LEN}-token prompts",
            "value": mine["decode_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": steps, "warmup": warmup,
            "ms_per_step": mine["decode_ms_per_step"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
            "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
            "data": "synthetic: uniform random token ids, random N(0, 0.02) weights",
-           "config": dict(DESIGN_SIZES[args.design_size], layers=n_layers, global_batch=batch, prompt_len=PROMPT_LEN),
-           f"decode_vs_{other_name}": round(mine["decode_tok_s"] / other["decode_tok_s"], 3),
-           f"prefill_vs_{other_name}": round(mine["prefill_tok_s"] / other["prefill_tok_s"], 3),
-           args.design: mine, other_name: other}
+           "config": dict(DESIGN_SIZES[args.design_size], layers=n_layers, global_batch=batch, prompt_len=PROMPT_LEN)}
+    for o in others:
+        out[f"decode_vs_{o}"] = round(mine["decode_tok_s"] / results[o]["decode_tok_s"], 3)
+        out[f"prefill_vs_{o}"] = round(mine["prefill_tok_s"] / results[o]["prefill_tok_s"], 3)
+    out.update(results)
     print(json.dumps(out))
     return 0
 
@@ -206,7 +219,7 @@ def main() -> int:
     ap.add_argument("--dtype", default="bfloat16", choices=["bfloat16", "float32"])
     ap.add_argument("--no-points", action="store_true", help="skip the further points")
     ap.add_argument("--prefill-runs", type=int, default=3)
-    ap.add_argument("--design", default=None, choices=["dokulix", "felovik", "sogavik", "roravik"],
+    ap.add_argument("--design", default=None, choices=sorted(COMPANIONS),
                     help="measure this architecture at real layer sizes beside the closest Qwen3 shape, instead of the default workload")
     ap.add_argument("--design-size", default="2b", choices=sorted(DESIGN_SIZES), help="layer sizes for --design")
     ap.add_argument("--skip-prompts", action="store_true",

@@ -187,6 +187,41 @@ CATALOG += [
     ModelEntry("roravik-2b", roravik_config(32768, 2048, 16, 8, 128, 1024, 16, 128, 32, 64, 6144, 32, 1024, 4, 24)),
 ]
 
+
+
+def kakalorn_config(vocab, width, heads, kv_heads, dim, window, keep_first, lat_heads, lat_dim, rot_dim, q_rank, kv_rank, rec_heads,
+                    rec_dim, ff, n_layers, taps=4, factor=4.0, original=4096, max_positions=None):
+    """A Kakalorn configuration: latent attention, windowed attention and the gated recurrence in turn; of the latent
+    layers every second one runs on the rows that the one before it keeps."""
+    rot = {"base": 10000.0, "dims": rot_dim, "scaling": {"factor": factor, "original": original, "fast": 32.0, "slow": 1.0}}
+    latent = {"heads": lat_heads, "dim": lat_dim, "rot_dim": rot_dim, "vdim": lat_dim, "q_rank": q_rank, "kv_rank": kv_rank,
+              "scale": (lat_dim + rot_dim) ** -0.5, "rot": rot}
+    attention = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5,
+                 "mask": {"size": window, "keep_first": keep_first}, "rot": {"base": 10000.0, "dims": dim}}
+    recurrence = {"heads": rec_heads, "dim": rec_dim, "vdim": rec_dim}
+    mlp = {"kind": "dense", "ff": ff}
+    layers = []
+    for i in range(n_layers):
+        if i % 3 == 0:
+            layers.append({"type": "latent_attention", "mixer": latent if i % 6 == 0 else dict(latent, kv_from=i - 3), "mlp": mlp})
+        elif i % 3 == 1:
+            layers.append({"type": "attention", "mixer": attention, "mlp": mlp})
+        else:
+            layers.append({"type": "hgrn2", "mixer": recurrence, "mlp": mlp})
+    cfg = {"architecture": "Kakalorn", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "canon": {"taps": taps}, "layers": layers}
+    if max_positions is not None:
+        cfg["max_positions"] = max_positions
+    return cfg
+
+
+# The sixth architecture: a test-sized model and the layer sizes of a 2B-class model (random weights; no
+# checkpoint of this design exists).
+CATALOG += [
+    ModelEntry("kakalorn-tiny", kakalorn_config(352, 96, 4, 2, 24, 40, 3, 2, 32, 16, 48, 64, 3, 32, 192, 6, taps=3),
+               default_ctx=512, init_norm_jitter=True),
+    ModelEntry("kakalorn-2b", kakalorn_config(32768, 2048, 16, 8, 128, 1024, 4, 16, 128, 64, 768, 512, 16, 128, 6144, 24)),
+]
+
 _BY_NAME = {e.name: e for e in CATALOG}
 
 

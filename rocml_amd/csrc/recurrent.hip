@@ -1191,6 +1191,12 @@ struct DecayScanArgs {
     float* out; int n_heads; int dk; int dv;
 };
 
+// The sigmoid form a / (1 + e^x) by one hardware exponential and one hardware reciprocal: both are good to an ulp or so, and
+// where |x| is large enough for the exponent's own rounding to count the result is next to 0 or to a.
+__device__ __forceinline__ float ds_over_one_plus_exp(float a, float x) {
+    return a * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(x * 1.4426950408889634f));
+}
+
 enum DecayMode : int { DECAY_HEAD = 0, DECAY_BONUS = 1, DECAY_GATE = 2 };
 
 // R: entries of a column per lane (dk <= 16 R).  CPL: columns per lane.  DECAY_BONUS: a decay per token and channel and a
@@ -1357,25 +1363,45 @@ decay_scan_kernel(DecayScanArgs a) {
         // One token (a decode step): its numbers come straight from memory, beside the state's; the same arithmetic.
         float qq[R], kk[R], ww[R], vv[CPL], sums[CPL];
         size_t t = (size_t)first;
+        // a lane's R numbers of a row of the head's dk (zeros beyond): 16-byte pieces where the row allows
+        auto row_part = [&](float (&out)[R], const float* row) {
+            if constexpr (R % 4 == 0) {
+                if (dk % 4 == 0 && ((uintptr_t)row & 15) == 0) {
 #pragma unroll
-        for (int r = 0; r < R; ++r) {
-            int i = l * R + r;
-            bool in = i < dk;
-            size_t e = (size_t)h * dk + i;
-            qq[r] = in ? a.q[t * a.ldq + a.q_col0 + e] : 0.f;
-            kk[r] = in ? a.k[t * a.ldk + a.k_col0 + e] : 0.f;
-            ww[r] = 0.f;
-            if constexpr (GATE) {
-                if (in) {
-                    qq[r] = rc_silu(qq[r]);
-                    kk[r] = (1.f - a.gate_lower[e]) / (1.0f + expf(kk[r] + a.gate_bias[e]));
+                    for (int r4 = 0; r4 < R / 4; ++r4) {
+                        int i = l * R + 4 * r4;
+                        float4 v4 = i < dk ? *(const float4*)(row + i) : float4{0.f, 0.f, 0.f, 0.f};
+                        out[4 * r4] = v4.x; out[4 * r4 + 1] = v4.y; out[4 * r4 + 2] = v4.z; out[4 * r4 + 3] = v4.w;
+                    }
+                    return;
                 }
             }
-            if constexpr (BONUS) {
-                if (in) {
-                    float x = a.w[t * a.ldw + a.w_col0 + e];
-                    ww[r] = a.w_offset ? expf(-expf(x + a.w_offset[e])) : x;
-                }
+#pragma unroll
+            for (int r = 0; r < R; ++r) out[r] = l * R + r < dk ? row[l * R + r] : 0.f;
+        };
+        size_t head0 = (size_t)h * dk;
+        row_part(qq, a.q + t * a.ldq + a.q_col0 + head0);
+        row_part(kk, a.k + t * a.ldk + a.k_col0 + head0);
+#pragma unroll
+        for (int r = 0; r < R; ++r) ww[r] = 0.f;
+        if constexpr (GATE) {
+            float low[R], shift[R];
+            row_part(low, a.gate_lower + head0);
+            row_part(shift, a.gate_bias + head0);
+#pragma unroll
+            for (int r = 0; r < R; ++r) {
+                bool in = l * R + r < dk;
+                qq[r] = ds_over_one_plus_exp(qq[r], -qq[r]);
+                kk[r] = in ? ds_over_one_plus_exp(1.f - low[r], kk[r] + shift[r]) : 0.f;
+            }
+        }
+        if constexpr (BONUS) {
+            row_part(ww, a.w + t * a.ldw + a.w_col0 + head0);
+            if (a.w_offset) {
+                float shift[R];
+                row_part(shift, a.w_offset + head0);
+#pragma unroll
+                for (int r = 0; r < R; ++r) ww[r] = l * R + r < dk ? expf(-expf(ww[r] + shift[r])) : 0.f;
             }
         }
 #pragma unroll
@@ -1412,8 +1438,7 @@ decay_scan_kernel(DecayScanArgs a) {
                         // silu(q) = q / (1 + e^-q), and g = (1 - l) / (1 + e^(x + b))
                         if (form[m]) {
                             bool is_q = form[m] == 1;
-                            float e = expf(is_q ? -val : val + offset[m]);
-                            val = (is_q ? val : span[m]) / (1.0f + e);
+                            val = ds_over_one_plus_exp(is_q ? val : span[m], is_q ? -val : val + offset[m]);
                         }
                     }
                     if (!src[m]) val = fixed[m];

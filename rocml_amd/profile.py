@@ -59,8 +59,9 @@ def _attention_cost(q, out, k_cache, v_cache, block_table, token_seq, token_pos,
         keys_per_query = min(keys_per_query, max(1, kw["chunk"] // 2))
         read_len = min(max_len, max_new + kw["chunk"])
     elif window:
-        keys_per_query = min(keys_per_query, window)
-        read_len = min(max_len, max_new + window)
+        seen = window + kw.get("keep_first", 0)
+        keys_per_query = min(keys_per_query, seen)
+        read_len = min(max_len, max_new + seen)
     kv = n_seqs * read_len * n_kv_heads * row * k_cache.element_size()
     return _nbytes(q, out) + kv, 2 * n_heads * (head_dim + dv) * n_tokens * keys_per_query
 
@@ -75,6 +76,10 @@ def _gemm_batched_cost(x, x_head_stride, w, out, out_head_stride, **kw) -> Tuple
 def _fused_attention_cost(qkv, out, k_cache, v_cache, block_table, token_seq, token_pos, n_heads, n_kv_heads, head_dim,
                           *a, **kw) -> Tuple[int, int]:
     max_len = kw.get("max_len", 0)
+    if kw.get("window"):
+        max_len = min(max_len, kw["window"] + kw.get("keep_first", 0))
+    elif kw.get("chunk"):                    # half a block on average
+        max_len = min(max_len, max(1, kw["chunk"] // 2))
     n_seqs = out.shape[0]
     kv = 2 * n_seqs * max_len * n_kv_heads * head_dim * k_cache.element_size()
     return _nbytes(qkv, out) + kv, 4 * n_heads * head_dim * n_seqs * max_len
@@ -104,7 +109,7 @@ _COSTS: Dict[str, Tuple[str, Callable]] = {
         _nbytes(x, w, resid, resid, gain, xg, ssq), 2 * x.shape[0] * w.shape[0] * x.shape[1])),
     "attention": (lambda *a, **kw: "attention over latent rows" if kw.get("values_in_keys") else
                   "attention (blocks, slopes, sink, soft cap)" if kw.get("chunk") or kw.get("sink") or kw.get("slopes") is not None
-                  or kw.get("softcap") is not None
+                  or kw.get("softcap") is not None or kw.get("keep_first")
                   else "attention", _attention_cost),
     "attention_decode_fused": ("attention (norm, rotation, append)", _fused_attention_cost),
     "attention_prefill_fused": ("attention (query norm, rotation)", _prefill_fused_cost),
@@ -126,9 +131,15 @@ _COSTS: Dict[str, Tuple[str, Callable]] = {
     "sigmoid_gate": ("output gate", lambda y, gate, **kw: (2 * _nbytes(y) + gate.numel() * 4, 4 * y.numel())),
     "qk_span_stats": ("q/k norm factors", lambda qkv, q_width, k_width, bias, eps, out: (
         qkv.shape[0] * (q_width + k_width) * qkv.element_size() + _nbytes(out), 2 * qkv.shape[0] * (q_width + k_width))),
-    "norm_add": (lambda *a, **kw: "sublayer norm, residual sum and the next norm" if kw.get("next_gain") is not None
+    "norm_add": (lambda *a, **kw: "sublayer norm, residual sum, the next norm and its convolution" if kw.get("conv") is not None
+                 else "sublayer norm, residual sum and the next norm" if kw.get("next_gain") is not None
                  else "sublayer norm and residual sum", lambda x, y, gain, bias, eps, **kw: (
-        2 * _nbytes(x) + _nbytes(kw.get("copy"), kw.get("partials")) + (0 if kw.get("replace") else _nbytes(y)), 8 * x.numel())),
+        2 * _nbytes(x) + _nbytes(kw.get("copy"), kw.get("partials")) + (0 if kw.get("replace") else _nbytes(y))
+        + (0 if kw.get("conv") is None else _nbytes(kw["conv"][0]) + 2 * (kw["conv"][0].shape[0] - 1) * _nbytes(kw["copy"])), 8 * x.numel())),
+    "added_conv": ("convolution on the mixer's input", lambda h, w, state, cu, slots, counts, out: (
+        _nbytes(h, out, w) + (0 if state is None else 2 * slots.numel() * state.shape[1] * state.shape[2] * state.element_size()),
+        2 * w.shape[0] * h.numel())),
+    "activate": ("activation", lambda x, out, activation: (_nbytes(x, out), 4 * x.numel())),
     "norm_add_branches": ("branch norms, sublayer norm and residual sum", lambda x, branches, gains, weight, beps, gain, bias, eps, layer, **kw: (
         2 * _nbytes(x) + _nbytes(*branches) + _nbytes(kw.get("copy")), 8 * x.numel() * (1 + len(branches)))),
     "layernorm": ("layer norm", lambda x, gain, bias, eps, out, rows=None: (out.numel() * 4 + _nbytes(out), 8 * out.numel())),
@@ -139,8 +150,8 @@ _COSTS: Dict[str, Tuple[str, Callable]] = {
                        proj.shape[0] * n_heads * (2 * head_dim + v_head_dim + 2) * 4 + _nbytes(out)
                        + 2 * slots.numel() * n_heads * head_dim * (v_head_dim + 1) * 4,
                        4 * proj.shape[0] * n_heads * head_dim * (v_head_dim + 1), PEAK_FLOPS[torch.float32])),
-    "head_norm_gate": ("head norm and gate", lambda o, g, g_col0, gain, out, n_heads, eps, **kw: (
-        2 * _nbytes(o) + _nbytes(out), 8 * o.numel())),
+    "head_norm_gate": (lambda o, g, *a, **kw: "head norm" if g is None else "head norm and gate", lambda o, g, g_col0, gain, out, n_heads, eps, **kw: (
+        (1 if g is None else 2) * _nbytes(o) + _nbytes(out), 8 * o.numel())),
     "splitk_reduce": ("sum of K pieces", _tensor_args_cost()),
     "sum_norm": ("residual sum and norm", lambda x, branches, gains, gain, eps, **kw: (
         2 * _nbytes(x) + _nbytes(*branches) + _nbytes(kw.get("copy")), 4 * x.numel() * (1 + len(branches)))),
