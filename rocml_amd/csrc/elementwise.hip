@@ -127,6 +127,15 @@ template <> __device__ __forceinline__ float rounded<float>(float v) { return v;
 template <> __device__ __forceinline__ float rounded<bf16_t>(float v) { return bf16_to_f32(f32_to_bf16(v)); }
 template <typename T>
 __device__ __forceinline__ float4 rounded4(float4 v) { return make_float4(rounded<T>(v.x), rounded<T>(v.y), rounded<T>(v.z), rounded<T>(v.w)); }
+// (products and sums of their own: the norm's output is rounded before the convolution adds to it, whichever kernel does)
+__device__ __forceinline__ float4 scaled4(float4 v, float s, float4 g) {
+#pragma clang fp contract(off)
+    return make_float4(v.x * s * g.x, v.y * s * g.y, v.z * s * g.z, v.w * s * g.w);
+}
+__device__ __forceinline__ float4 sum4(float4 a, float4 b) {
+#pragma clang fp contract(off)
+    return make_float4(a.x + b.x, a.y + b.y, a.z + b.z, a.w + b.w);
+}
 __device__ __forceinline__ float4 fma4(float4 a, float4 b, float4 c) {
     return make_float4(fmaf(a.x, b.x, c.x), fmaf(a.y, b.y, c.y), fmaf(a.z, b.z, c.z), fmaf(a.w, b.w, c.w));
 }
@@ -1477,7 +1486,7 @@ norm_add_vec_kernel(float* __restrict__ x, const float* __restrict__ y, const fl
             int i = threadIdx.x + j * EW_BLOCK;
             if (i >= nv) continue;
             float4 g2 = ((const float4*)next_gain)[i];
-            float4 h = make_float4(xv[j].x * inv2 * g2.x, xv[j].y * inv2 * g2.y, xv[j].z * inv2 * g2.z, xv[j].w * inv2 * g2.w);
+            float4 h = scaled4(xv[j], inv2, g2);
             if constexpr (TAPS > 0) {
                 h = rounded4<TC>(h);
 #pragma unroll
@@ -1486,7 +1495,7 @@ norm_add_vec_kernel(float* __restrict__ x, const float* __restrict__ y, const fl
                 float4 a = make_float4(0.f, 0.f, 0.f, 0.f);
 #pragma unroll
                 for (int k = 0; k < TAPS; ++k) a = fma4(tap[k][j], k < TAPS - 1 ? kept[k < KEPT ? k : 0][j] : h, a);
-                h.x += a.x; h.y += a.y; h.z += a.z; h.w += a.w;
+                h = sum4(h, a);
             }
             store4(copy + row + 4 * (size_t)i, h.x, h.y, h.z, h.w);
         }
@@ -1844,7 +1853,7 @@ ROCML_EXPORT int rocml_row_gate_add(float* x, const float* y, const float* g, in
 // thread and a run of AC_RUN consecutive tokens of one sequence, and slides over them, so an input is read once (and
 // taps - 1 times more at the run's start).  Only the first run of a sequence reads the kept rows (a run is longer than
 // they are), and the same thread replaces them when it is done with them.
-constexpr int AC_RUN = 16, AC_MAX_TAPS = 8;
+constexpr int AC_RUN = 16, AC_MAX_TAPS = 16;
 
 template <typename T, int W> struct AcPiece;
 template <> struct AcPiece<float, 4> { typedef float4 type; };
@@ -1953,6 +1962,7 @@ static int launch_added_conv(const T* h, T* out, int n, const float* w, T* state
 #define AC(T_) case T_: added_conv_kernel<T, W, T_><<<grid, threads, 0, stream>>>(h, out, n, w, state, cu_seqlens, seq_slots, n_seqs); break
     switch (taps) {
         AC(1); AC(2); AC(3); AC(4); AC(5); AC(6); AC(7); AC(8);
+        AC(9); AC(10); AC(11); AC(12); AC(13); AC(14); AC(15); AC(16);
         default: return rocml_fail("added_conv: %d taps (1 to %d)", taps, AC_MAX_TAPS);
     }
 #undef AC

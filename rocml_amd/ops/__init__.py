@@ -443,7 +443,7 @@ def norm_add_conv_fits(n: int, taps: int) -> bool:
     return bool(library("elementwise").rocml_norm_add_conv_fits(int(n), int(taps)))
 
 
-ADDED_CONV_MAX_TAPS = 8
+ADDED_CONV_MAX_TAPS = 16
 
 
 def added_conv(h: torch.Tensor, w: torch.Tensor, state: Optional[torch.Tensor], cu_seqlens: torch.Tensor, seq_slots: torch.Tensor,
