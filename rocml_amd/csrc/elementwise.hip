@@ -113,32 +113,6 @@ __device__ __forceinline__ void store4(bf16_t* p, float a, float b, float c, flo
     v.y = (uint32_t)f32_to_bf16(c) | ((uint32_t)f32_to_bf16(d) << 16);
     *(uint2*)p = v;
 }
-template <typename T>
-__device__ __forceinline__ void store4(T* p, float4 v) { store4(p, v.x, v.y, v.z, v.w); }
-__device__ __forceinline__ float4 load4(const float* p) { return *(const float4*)p; }
-__device__ __forceinline__ float4 load4(const bf16_t* p) {
-    uint2 v = *(const uint2*)p;
-    return make_float4(__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16),
-                       __uint_as_float(v.y & 0xffff0000u));
-}
-// the numbers as a value of type T holds them
-template <typename T> __device__ __forceinline__ float rounded(float v);
-template <> __device__ __forceinline__ float rounded<float>(float v) { return v; }
-template <> __device__ __forceinline__ float rounded<bf16_t>(float v) { return bf16_to_f32(f32_to_bf16(v)); }
-template <typename T>
-__device__ __forceinline__ float4 rounded4(float4 v) { return make_float4(rounded<T>(v.x), rounded<T>(v.y), rounded<T>(v.z), rounded<T>(v.w)); }
-// (products and sums of their own: the norm's output is rounded before the convolution adds to it, whichever kernel does)
-__device__ __forceinline__ float4 scaled4(float4 v, float s, float4 g) {
-#pragma clang fp contract(off)
-    return make_float4(v.x * s * g.x, v.y * s * g.y, v.z * s * g.z, v.w * s * g.w);
-}
-__device__ __forceinline__ float4 sum4(float4 a, float4 b) {
-#pragma clang fp contract(off)
-    return make_float4(a.x + b.x, a.y + b.y, a.z + b.z, a.w + b.w);
-}
-__device__ __forceinline__ float4 fma4(float4 a, float4 b, float4 c) {
-    return make_float4(fmaf(a.x, b.x, c.x), fmaf(a.y, b.y, c.y), fmaf(a.z, b.z, c.z), fmaf(a.w, b.w, c.w));
-}
 
 template <typename TO, int RN_VEC>
 __global__ void __launch_bounds__(EW_BLOCK)
@@ -1385,43 +1359,17 @@ norm_add_kernel(float* __restrict__ x, float* __restrict__ y, const float* __res
 
 // The same for rows of up to 8192 values that are a multiple of 4: the row stays in registers and all
 // loads are issued at once.
-// TAPS > 0 (steps of one token per sequence, with next_gain): what reads the next norm's output is first replaced by
-// itself plus its causal convolution over the sequence (see added_conv below); row b is sequence b's one token, and the
-// kept rows of its slot move up by one.
-struct NextConv {
-    const float* w;             // [taps, n]
-    void* state;                // [slot, taps - 1, n] in copy's type
-    const int* slots;           // [rows]
-};
-
-template <typename TC, bool LAYER, int VEC, int TAPS = 0>
+template <typename TC, bool LAYER, int VEC>
 __global__ void __launch_bounds__(EW_BLOCK)
 norm_add_vec_kernel(float* __restrict__ x, const float* __restrict__ y, const float* __restrict__ gain,
                     const float* __restrict__ bias, float eps, int n, TC* __restrict__ copy,
                     const float* __restrict__ partials, int n_splits, long long split_stride, int replace,
-                    const float* __restrict__ next_gain, float next_eps, NextConv cv = NextConv{}) {
+                    const float* __restrict__ next_gain, float next_eps) {
     __shared__ float scratch[EW_BLOCK / WAVE];
     size_t row = (size_t)blockIdx.x * n;
     int nv = n / 4;
     const float4 zero4 = make_float4(0.f, 0.f, 0.f, 0.f);
     float4 yv[VEC], xv[VEC], gv[VEC], bv[VEC];
-    constexpr int KEPT = TAPS > 1 ? TAPS - 1 : 1;
-    float4 kept[KEPT][VEC], tap[TAPS > 0 ? TAPS : 1][VEC];
-    TC* state_row = nullptr;
-    if constexpr (TAPS > 0) {
-        // (asked for beside the row's own numbers; they do not depend on it)
-        state_row = (TC*)cv.state + (size_t)cv.slots[blockIdx.x] * (TAPS - 1) * n;
-#pragma unroll
-        for (int j = 0; j < VEC; ++j) {
-            int i = threadIdx.x + j * EW_BLOCK;
-            bool ok = i < nv;
-#pragma unroll
-            for (int k = 0; k < TAPS; ++k) {
-                tap[k][j] = ok ? ((const float4*)(cv.w + (size_t)k * n))[i] : zero4;
-                if (k < TAPS - 1) kept[k][j] = ok ? load4(state_row + (size_t)k * n + 4 * (size_t)i) : zero4;
-            }
-        }
-    }
 #pragma unroll
     for (int j = 0; j < VEC; ++j) {
         int i = threadIdx.x + j * EW_BLOCK;
@@ -1486,18 +1434,7 @@ norm_add_vec_kernel(float* __restrict__ x, const float* __restrict__ y, const fl
             int i = threadIdx.x + j * EW_BLOCK;
             if (i >= nv) continue;
             float4 g2 = ((const float4*)next_gain)[i];
-            float4 h = scaled4(xv[j], inv2, g2);
-            if constexpr (TAPS > 0) {
-                h = rounded4<TC>(h);
-#pragma unroll
-                for (int k = 0; k < TAPS - 1; ++k)
-                    store4(state_row + (size_t)k * n + 4 * (size_t)i, k + 1 < TAPS - 1 ? kept[k + 1 < KEPT ? k + 1 : 0][j] : h);
-                float4 a = make_float4(0.f, 0.f, 0.f, 0.f);
-#pragma unroll
-                for (int k = 0; k < TAPS; ++k) a = fma4(tap[k][j], k < TAPS - 1 ? kept[k < KEPT ? k : 0][j] : h, a);
-                h = sum4(h, a);
-            }
-            store4(copy + row + 4 * (size_t)i, h.x, h.y, h.z, h.w);
+            store4(copy + row + 4 * (size_t)i, xv[j].x * inv2 * g2.x, xv[j].y * inv2 * g2.y, xv[j].z * inv2 * g2.z, xv[j].w * inv2 * g2.w);
         }
     }
 }
@@ -1505,25 +1442,13 @@ norm_add_vec_kernel(float* __restrict__ x, const float* __restrict__ y, const fl
 template <typename TC, bool LAYER>
 static void launch_norm_add(float* x, float* y, const float* gain, const float* bias, float eps, int n_rows, int n,
                             TC* copy, const float* partials, int n_splits, long long split_stride, int replace,
-                            const float* next_gain, float next_eps, const NextConv& cv, int taps, hipStream_t stream) {
+                            const float* next_gain, float next_eps, hipStream_t stream) {
     bool vec = n % 4 == 0 && n <= 4 * EW_BLOCK * RN_MAX_VEC && (uintptr_t)x % 16 == 0 && (uintptr_t)y % 16 == 0 &&
                (uintptr_t)gain % 16 == 0 && (!bias || (uintptr_t)bias % 16 == 0) && (!copy || (uintptr_t)copy % 8 == 0) &&
                (!next_gain || (uintptr_t)next_gain % 16 == 0) &&
                (n_splits == 0 || ((uintptr_t)partials % 16 == 0 && split_stride % 4 == 0));
     int v = ceil_div(n / 4, EW_BLOCK);
 #define NAV(V_) norm_add_vec_kernel<TC, LAYER, V_><<<n_rows, EW_BLOCK, 0, stream>>>(x, y, gain, bias, eps, n, copy, partials, n_splits, split_stride, replace, next_gain, next_eps)
-    if constexpr (!LAYER) {
-        if (taps > 0) {         // (the caller asked norm_add_conv_fits and checked the alignment)
-#define NAC(V_, T_) norm_add_vec_kernel<TC, false, V_, T_><<<n_rows, EW_BLOCK, 0, stream>>>(x, y, gain, bias, eps, n, copy, partials, n_splits, split_stride, replace, next_gain, next_eps, cv)
-#define NAC_BY_TAPS(V_) { if (taps == 2) NAC(V_, 2); else if (taps == 3) NAC(V_, 3); else NAC(V_, 4); }
-            if (v <= 1) NAC_BY_TAPS(1)
-            else if (v <= 2) NAC_BY_TAPS(2)
-            else NAC_BY_TAPS(4)
-#undef NAC_BY_TAPS
-#undef NAC
-            return;
-        }
-    }
     if (!vec) norm_add_kernel<TC, LAYER><<<n_rows, EW_BLOCK, 0, stream>>>(x, y, gain, bias, eps, n, copy, partials, n_splits, split_stride, replace, next_gain, next_eps);
     else if (v <= 1) NAV(1);
     else if (v <= 2) NAV(2);
@@ -1646,21 +1571,9 @@ ROCML_EXPORT int rocml_norm_add_branches(float* x, const float* y0, const float*
     return 0;
 }
 
-// Whether norm_add also forms the convolution of the next norm's output (rows in registers, 2 to 4 taps).
-ROCML_EXPORT int rocml_norm_add_conv_fits(int n, int taps) { return n > 0 && n % 4 == 0 && n <= 4 * EW_BLOCK * 4 && taps >= 2 && taps <= 4; }
-
 ROCML_EXPORT int rocml_norm_add(float* x, float* y, int n_rows, int n, const float* gain, const float* bias,
                                 float eps, int layer, void* copy, int copy_dtype, const float* partials, int n_splits,
-                                long long split_stride, int replace, const float* next_gain, float next_eps,
-                                const float* conv_w, void* conv_state, int conv_slots_n, const int* conv_slots, int taps,
-                                hipStream_t stream) {
-    // conv_w (may be null; needs next_gain): [taps, n]; the next norm's output h is replaced by h + its causal convolution,
-    // every row being the one token of a sequence whose kept rows are conv_state [conv_slots_n, taps - 1, n] (copy's type)
-    // at conv_slots [rows]
-    NextConv cv{conv_w, conv_state, conv_slots};
-    if (!conv_w) taps = 0;
-    ROCML_REQUIRE(taps == 0 || (next_gain && conv_state && conv_slots && conv_slots_n > 0 && !layer && rocml_norm_add_conv_fits(n, taps)),
-                  "norm_add: a convolution of the next norm's output needs that norm, the kept rows and sizes it fits (n=%d taps=%d)", n, taps);
+                                long long split_stride, int replace, const float* next_gain, float next_eps, hipStream_t stream) {
     // next_gain (may be null; needs copy): copy gets the new x normed, x / sqrt(mean(x^2) + next_eps) * next_gain
     ROCML_REQUIRE(!next_gain || copy, "norm_add: the next norm's output needs a place");
     // layer = 1: layer norm (mean taken off, bias added if given); 0: root-mean-square norm (bias is not read)
@@ -1671,19 +1584,13 @@ ROCML_EXPORT int rocml_norm_add(float* x, float* y, int n_rows, int n, const flo
                   "norm_add: %d partial sums with a stride of %lld do not fit", n_splits, split_stride);
     ROCML_REQUIRE(!copy || copy_dtype == ROCML_F32 || copy_dtype == ROCML_BF16, "norm_add: unknown dtype code %d", copy_dtype);
     if (n_rows == 0) return 0;
-    if (taps > 0) {
-        const void* ptrs[] = {x, y, gain, next_gain, conv_w, partials};
-        for (const void* q : ptrs) ROCML_REQUIRE((uintptr_t)q % 16 == 0, "norm_add: operands must start on 16 bytes");
-        ROCML_REQUIRE((uintptr_t)copy % 16 == 0 && (uintptr_t)conv_state % 16 == 0 && (n_splits == 0 || split_stride % 4 == 0),
-                      "norm_add: operands must start on 16 bytes");
-    }
     bool half = copy && copy_dtype == ROCML_BF16;
     if (layer) {
-        if (half) launch_norm_add<bf16_t, true>(x, y, gain, bias, eps, n_rows, n, (bf16_t*)copy, partials, n_splits, split_stride, replace, next_gain, next_eps, cv, taps, stream);
-        else launch_norm_add<float, true>(x, y, gain, bias, eps, n_rows, n, (float*)copy, partials, n_splits, split_stride, replace, next_gain, next_eps, cv, taps, stream);
+        if (half) launch_norm_add<bf16_t, true>(x, y, gain, bias, eps, n_rows, n, (bf16_t*)copy, partials, n_splits, split_stride, replace, next_gain, next_eps, stream);
+        else launch_norm_add<float, true>(x, y, gain, bias, eps, n_rows, n, (float*)copy, partials, n_splits, split_stride, replace, next_gain, next_eps, stream);
     } else {
-        if (half) launch_norm_add<bf16_t, false>(x, y, gain, nullptr, eps, n_rows, n, (bf16_t*)copy, partials, n_splits, split_stride, replace, next_gain, next_eps, cv, taps, stream);
-        else launch_norm_add<float, false>(x, y, gain, nullptr, eps, n_rows, n, (float*)copy, partials, n_splits, split_stride, replace, next_gain, next_eps, cv, taps, stream);
+        if (half) launch_norm_add<bf16_t, false>(x, y, gain, nullptr, eps, n_rows, n, (bf16_t*)copy, partials, n_splits, split_stride, replace, next_gain, next_eps, stream);
+        else launch_norm_add<float, false>(x, y, gain, nullptr, eps, n_rows, n, (float*)copy, partials, n_splits, split_stride, replace, next_gain, next_eps, stream);
     }
     ROCML_CHECK_LAUNCH("norm_add");
     return 0;

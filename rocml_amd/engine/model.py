@@ -207,10 +207,8 @@ class DecoderModel:
             # entries that add the embedding's output to the stream later need it kept
             x0 = ws.get("model.x0", (step.n_tokens, s.hidden), torch.float32)
             ops.weighted_sum(x0, [x], [1.0])
-        following_view = None
         for i, entry in enumerate(s.schedule):
-            view = following_view if following_view is not None else self.entry_view(i, cache, step)
-            following_view = None
+            view = self.entry_view(i, cache, step)
             block = self.blocks[entry.layer]
             if entry.offset_row is not None:
                 # (sums that a product left for the next norm may still be missing from x: additions commute)
@@ -225,8 +223,7 @@ class DecoderModel:
             if following is not None and (s.schedule[i + 1].offset_row is not None or s.schedule[i + 1].add_embedding):
                 following = None      # the stream changes between the two blocks: nothing can be prepared across
             if getattr(block, "takes_next_norm", False) and hasattr(following, "entry_hint"):
-                following_view = self.entry_view(i + 1, cache, step)
-                hint = following.entry_hint(step, following_view)
+                hint = following.entry_hint(step)
             if hint is not None:
                 block.forward(step, x, view, entry.reads_cache_of is None, next_norm=hint)
             else:

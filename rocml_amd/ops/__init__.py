@@ -34,8 +34,7 @@ _SIGNATURES = {
         "rocml_qk_norm_rope_append": [_P, _I, _I, _I, _I, _I, _I, _P, _P, _F, _P, _P, _I, _I, _P, _P, _P,
                                       _I, _P, _I, _P, _P, _I, _I, _I, _LL, _P, _I, _F, _I, _P, _I, _I, _P],
         "rocml_qk_span_stats": [_P, _I, _I, _I, _I, _I, _P, _F, _P, _P],
-        "rocml_norm_add": [_P, _P, _I, _I, _P, _P, _F, _I, _P, _I, _P, _I, _LL, _I, _P, _F, _P, _P, _I, _P, _I, _P],
-        "rocml_norm_add_conv_fits": [_I, _I],
+        "rocml_norm_add": [_P, _P, _I, _I, _P, _P, _F, _I, _P, _I, _P, _I, _LL, _I, _P, _F, _P],
         "rocml_added_conv": [_P, _P, _I, _I, _I, _P, _I, _P, _I, _P, _P, _I, _P, _P],
         "rocml_activate": [_P, _P, _I, _LL, _I, _P],
         "rocml_norm_add_branches": [_P, _P, _P, _P, _P, _F, _F, _I, _I, _P, _P, _F, _I, _P, _I, _P],
@@ -394,15 +393,13 @@ def qk_span_stats(qkv: torch.Tensor, q_width: int, k_width: int, bias: Optional[
 
 def norm_add(x: torch.Tensor, y: torch.Tensor, gain: torch.Tensor, bias: Optional[torch.Tensor], eps: float,
              layer: bool, copy: Optional[torch.Tensor] = None, partials: Optional[torch.Tensor] = None,
-             replace: bool = False, next_gain: Optional[torch.Tensor] = None, next_eps: float = 0.0, conv=None) -> None:
+             replace: bool = False, next_gain: Optional[torch.Tensor] = None, next_eps: float = 0.0) -> None:
     """``x += f(y)`` row by row in 32-bit: ``f`` a layer norm ``(y - mean) / sqrt(var + eps) * gain + bias``
     (``layer``) or ``y / sqrt(mean(y^2) + eps) * gain``.  ``copy`` gets the new ``x`` in its own type.
     ``partials`` (``[splits, rows, n]`` 32-bit): the K pieces of the product that made ``y``, added to ``y`` in
     split order first, or with ``replace`` all of ``y`` (what ``y`` holds is not read).  ``next_gain`` (with ``copy``):
     ``copy`` gets the root-mean-square norm of the new ``x`` instead, ``x / sqrt(mean(x^2) + next_eps) * next_gain``: the
-    norm that reads the stream next.  ``conv``: ``(weights [taps, n], state [slots, taps - 1, n], slots [rows])``, for a step
-    of one token per sequence (row ``b`` is sequence ``b``'s token): that norm's output ``h`` is replaced by ``h`` plus its
-    causal convolution and the kept rows move up by one, as ``added_conv`` does; only where ``norm_add_conv_fits``."""
+    norm that reads the stream next."""
     _dev(x, y, gain, bias, copy, partials, next_gain)
     if next_gain is not None and (copy is None or next_gain.dtype != torch.float32 or next_gain.numel() != x.shape[1]):
         raise KernelError("norm_add: the next norm needs a 32-bit gain of the row's size and a place for its output")
@@ -419,28 +416,10 @@ def norm_add(x: torch.Tensor, y: torch.Tensor, gain: torch.Tensor, bias: Optiona
     if x.dim() != 2 or y.shape != x.shape or gain.numel() != x.shape[1] or (copy is not None and copy.shape != x.shape) \
             or (bias is not None and (bias.dtype != torch.float32 or bias.numel() != x.shape[1])):
         raise KernelError("norm_add: shapes do not fit")
-    conv_w = conv_state = conv_slots = None
-    taps = 0
-    if conv is not None:
-        conv_w, conv_state, conv_slots = conv
-        _dev(conv_w, conv_state, conv_slots)
-        _want(conv_w, torch.float32, "convolution weights")
-        _want(conv_slots, torch.int32, "sequence slots")
-        taps = conv_w.shape[0]
-        if next_gain is None or layer or not norm_add_conv_fits(x.shape[1], taps) or conv_w.shape[1] != x.shape[1] \
-                or conv_state.dtype != copy.dtype or conv_state.dim() != 3 or conv_state.shape[1:] != (taps - 1, x.shape[1]) \
-                or conv_slots.numel() != x.shape[0]:
-            raise KernelError("norm_add: the convolution's weights, kept rows or slots do not fit the step")
     _check("elementwise", library("elementwise").rocml_norm_add(
         _ptr(x), _ptr(y), x.shape[0], x.shape[1], _ptr(gain), _ptr(bias), float(eps), 1 if layer else 0, _ptr(copy),
         _code(copy) if copy is not None else 0, _ptr(partials), n_splits, split_stride, 1 if replace else 0, _ptr(next_gain),
-        float(next_eps), _ptr(conv_w), _ptr(conv_state), 0 if conv_state is None else conv_state.shape[0], _ptr(conv_slots), taps,
-        _stream()))
-
-
-def norm_add_conv_fits(n: int, taps: int) -> bool:
-    """Whether ``norm_add`` takes a convolution of so many taps over rows of ``n`` values."""
-    return bool(library("elementwise").rocml_norm_add_conv_fits(int(n), int(taps)))
+        float(next_eps), _stream()))
 
 
 ADDED_CONV_MAX_TAPS = 16

@@ -149,11 +149,7 @@ class NormHint:
 @dataclass(frozen=True)
 class FullNormHint(NormHint):
     """The same norm, for a consumer that wants the norm's whole output (not an operand that still lacks its rows' scale):
-    a kernel that completes the stream may write ``x / sqrt(mean(x^2) + eps) * gain`` in the compute type beside it.
-    ``conv``: what the consumer really reads is that output ``h`` plus its causal convolution over the sequence, and in this
-    step (one token per sequence) the kernel may form that too: ``(weights [taps, width], kept rows [slots, taps - 1, width],
-    slots of the step's sequences)``."""
-    conv: Optional[Tuple[torch.Tensor, torch.Tensor, torch.Tensor]] = None
+    a kernel that completes the stream may write ``x / sqrt(mean(x^2) + eps) * gain`` in the compute type beside it."""
 
 
 class Norm(Part):

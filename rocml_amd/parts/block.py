@@ -109,10 +109,9 @@ class PreNormBlock(ConvInput, Part):
     takes_pending = True      # forward() may be handed a stream that still lacks deferred sums
     takes_next_norm = True    # forward() accepts the hint of the norm that reads the stream after it
 
-    def entry_hint(self, step, cache=None):
+    def entry_hint(self, step):
         """The norm this block reads the residual stream with first, for the product that completes
-        the stream before it, if the block's mixer can apply the norm's scale itself in this step.
-        ``cache``: the block's view in this step."""
+        the stream before it, if the block's mixer can apply the norm's scale itself in this step."""
         if self.input_conv is not None:
             return None               # the convolution needs the normed rows themselves
         return self._hint(step, self.mixer_norm, self.mixer)
@@ -378,12 +377,11 @@ class SandwichNormBlock(ConvInput, Part):
     compute type; the sublayer writes its result to a buffer of the block; one kernel then norms that buffer and
     adds it to the 32-bit stream (it takes a product's K pieces in place of the buffer) and, in the same pass over
     the row, forms the norm that reads the stream next: the feed-forward's first norm behind the mixer, the next
-    layer's first norm behind the feed-forward when that layer is of this kind (``entry_hint``), in a step of one token
-    per sequence together with the convolution on that layer's input.  The norms are root-mean-square norms with a gain."""
+    layer's first norm behind the feed-forward when that layer is of this kind (``entry_hint``).  The norms are
+    root-mean-square norms with a gain."""
     takes_pending = False
     takes_next_norm = True
-    # in step.memo: (stream, gain, operand, whether the convolution on it is in it) of a norm that the kernel before formed
-    _READY = "sandwich_norm.operand"
+    _READY = "sandwich_norm.operand"      # in step.memo: (stream, gain, operand) of a norm that the kernel before formed
 
     def __init__(self, spec: BlockSpec, ctx: BuildContext):
         if spec.mixer_out_norm is None or (spec.ffn is not None and (spec.ffn_norm is None or spec.ffn_out_norm is None)):
@@ -418,15 +416,13 @@ class SandwichNormBlock(ConvInput, Part):
             (self.ffn.activation_bytes(n_tokens) if self.ffn is not None else 0) + \
             (self.input_conv.activation_bytes(n_tokens) if self.input_conv is not None else 0)
 
-    def entry_hint(self, step, cache=None):
-        """The norm this block reads the stream with first, for the kernel that completes the stream before it (and
-        the convolution on its output, where that kernel can form it).  ``cache``: the block's view in this step."""
+    def entry_hint(self, step):
+        """The norm this block reads the stream with first, for the kernel that completes the stream before it."""
         norm = self.children["mixer_norm"]
         gain = getattr(norm, "gain", None)
         if gain is None or not hasattr(norm, "eps") or getattr(norm, "centred", False):
             return None
-        conv = None if self.input_conv is None else self.input_conv.in_norm(step, self._views(cache)[1])
-        return FullNormHint(gain, float(norm.eps), self.hidden, conv=conv)
+        return FullNormHint(gain, float(norm.eps), self.hidden)
 
     def _sublayer(self, step, x, norm, run, out_norm, following, conv_view=None) -> None:
         """``following``: a ``FullNormHint`` of the norm that reads the stream after this sublayer, or None.
@@ -437,12 +433,10 @@ class SandwichNormBlock(ConvInput, Part):
         gain = getattr(norm, "gain", None)
         if ready is not None and gain is not None and ready[0] == x.data_ptr() and ready[1] == gain.data_ptr():
             xn = ready[2]           # the kernel that completed the stream formed this norm on its way
-            convolved = ready[3]
         else:
             xn = ws.get("block.xn", tuple(x.shape), self.dtype)
             norm.forward(x, xn)
-            convolved = False
-        if conv_view is not None and not convolved:
+        if conv_view is not None:
             xn = self.input_conv.forward(step, xn, conv_view[0])
         y = ws.get("block.sublayer", tuple(x.shape), torch.float32)
         rs.overwrite = rs.defer_overwrite = True
@@ -454,8 +448,8 @@ class SandwichNormBlock(ConvInput, Part):
             # (the sublayer is done with its operand: the buffer takes the next one)
             nxt = ws.get("block.xn", tuple(x.shape), self.dtype)
             ops.norm_add(x, y, out_norm.gain, None, out_norm.eps, layer=False, partials=partials, replace=replace, copy=nxt,
-                         next_gain=following.gain, next_eps=following.eps, conv=following.conv)
-            step.memo[self._READY] = (x.data_ptr(), following.gain.data_ptr(), nxt, following.conv is not None)
+                         next_gain=following.gain, next_eps=following.eps)
+            step.memo[self._READY] = (x.data_ptr(), following.gain.data_ptr(), nxt)
         else:
             ops.norm_add(x, y, out_norm.gain, None, out_norm.eps, layer=False, partials=partials, replace=replace)
 

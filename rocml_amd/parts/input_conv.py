@@ -1,8 +1,7 @@
 """What a layer's mixer reads, plus a short causal convolution over it: ``h_t + sum_j w[:, j] h_(t - taps + 1 + j)`` per
 channel, zeros before a sequence's start.  ``h`` is the layer's first norm in the compute type; the sums are 32-bit and the
 result is rounded to the compute type.  A sequence keeps its last ``taps - 1`` rows of ``h`` (in the compute type, which
-holds them exactly).  In a step of one token per sequence the kernel that forms the norm may form the convolution as well
-(``FullNormHint.conv``): the same arithmetic on the same rounded numbers."""
+holds them exactly).  A prompt step and a step of one token run the same kernel."""
 from __future__ import annotations
 
 from typing import Dict, Optional
@@ -34,12 +33,6 @@ class InputConv(Part):
 
     def activation_bytes(self, n_tokens: int) -> int:
         return n_tokens * self.hidden * (2 if self.dtype == torch.bfloat16 else 4)
-
-    def in_norm(self, step, view):
-        """What the kernel that forms the norm needs to form the convolution too, or None where it cannot."""
-        if step.max_new != 1 or view is None or not ops.norm_add_conv_fits(self.hidden, self.taps):
-            return None
-        return self.w, view.state, step.seq_slots
 
     def forward(self, step, h: torch.Tensor, view) -> torch.Tensor:
         out = step.workspace.get("block.conv", tuple(h.shape), self.dtype)

@@ -131,11 +131,9 @@ _COSTS: Dict[str, Tuple[str, Callable]] = {
     "sigmoid_gate": ("output gate", lambda y, gate, **kw: (2 * _nbytes(y) + gate.numel() * 4, 4 * y.numel())),
     "qk_span_stats": ("q/k norm factors", lambda qkv, q_width, k_width, bias, eps, out: (
         qkv.shape[0] * (q_width + k_width) * qkv.element_size() + _nbytes(out), 2 * qkv.shape[0] * (q_width + k_width))),
-    "norm_add": (lambda *a, **kw: "sublayer norm, residual sum, the next norm and its convolution" if kw.get("conv") is not None
-                 else "sublayer norm, residual sum and the next norm" if kw.get("next_gain") is not None
+    "norm_add": (lambda *a, **kw: "sublayer norm, residual sum and the next norm" if kw.get("next_gain") is not None
                  else "sublayer norm and residual sum", lambda x, y, gain, bias, eps, **kw: (
-        2 * _nbytes(x) + _nbytes(kw.get("copy"), kw.get("partials")) + (0 if kw.get("replace") else _nbytes(y))
-        + (0 if kw.get("conv") is None else _nbytes(kw["conv"][0]) + 2 * (kw["conv"][0].shape[0] - 1) * _nbytes(kw["copy"])), 8 * x.numel())),
+        2 * _nbytes(x) + _nbytes(kw.get("copy"), kw.get("partials")) + (0 if kw.get("replace") else _nbytes(y)), 8 * x.numel())),
     "added_conv": ("convolution on the mixer's input", lambda h, w, state, cu, slots, counts, out: (
         _nbytes(h, out, w) + (0 if state is None else 2 * slots.numel() * state.shape[1] * state.shape[2] * state.element_size()),
         2 * w.shape[0] * h.numel())),

@@ -1,5 +1,5 @@
 """Each mechanism of the Kakalorn layers alone, kernel against the plain functions: the convolution added to a mixer's
-input carried through pieces and slots, by itself and inside the norm that precedes it; the recurrence whose forget gate
+input carried through pieces and slots; the recurrence whose forget gate
 writes, with gates at both ends; the head norm without a gate; windows with kept first positions, learned sinks and keys
 as values, with one key made to stand out at every edge (prompt and single-token kernels, plain and matrix-core, page
 borders, rotations of a part of the head); latent rows and queries that turn in pairs of neighbours with slowed
@@ -94,37 +94,6 @@ def test_convolution_over_many_sequences_whose_runs_differ():
     out = torch.empty(len(rows), n, device=DEV)
     ops.added_conv(h.to(DEV), w.t().contiguous().to(DEV), state, cu, slots, counts, out)
     _close(out, want, 1e-6)
-
-
-@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("n,taps,splits", [(36, 2, 0), (256, 3, 2), (1024, 4, 3), (2052, 4, 0), (4096, 4, 5), (4096, 2, 1)])
-def test_convolution_inside_the_norm_before_it(n, taps, splits, dtype):
-    """A step of one token per sequence: the kernel that completes the stream and forms the next norm forms the convolution
-    too, bit for bit what the two kernels one after the other give, and moves the kept rows."""
-    from rocml_amd import ops
-    g = _gen(n + taps)
-    B, slots = 5, _i32([6, 0, 3, 2, 5])
-    x, y = torch.randn(B, n, generator=g).to(DEV), torch.randn(B, n, generator=g).to(DEV)
-    gain, gain2 = (1 + 0.2 * torch.randn(2, n, generator=g)).to(DEV)
-    w = torch.randn(taps, n, generator=g).to(DEV)
-    state = torch.randn(7, taps - 1, n, generator=g).to(dtype).to(DEV)
-    partials = torch.randn(splits, B, n, generator=g).to(DEV) if splits else None
-    assert ops.norm_add_conv_fits(n, taps)
-    x1, s1, h1, c1 = x.clone(), state.clone(), torch.empty(B, n, dtype=dtype, device=DEV), torch.empty(B, n, dtype=dtype, device=DEV)
-    kw = dict(partials=partials, replace=bool(splits), next_gain=gain2, next_eps=1e-5)
-    ops.norm_add(x1, y.clone(), gain, None, 1e-6, False, copy=h1, **kw)
-    ops.added_conv(h1, w, s1, _i32(list(range(B + 1))), slots, [1] * B, c1)
-    x2, s2, c2 = x.clone(), state.clone(), torch.empty(B, n, dtype=dtype, device=DEV)
-    ops.norm_add(x2, y.clone(), gain, None, 1e-6, False, copy=c2, conv=(w, s2, slots), **kw)
-    assert torch.equal(x1, x2) and torch.equal(s1, s2) and torch.equal(c1, c2)
-    # and against the plain functions
-    z = partials.sum(0) if splits else y
-    new = x.cpu().double() + plain.norm(z.cpu().double(), gain.cpu().double(), 1e-6)
-    h = plain.norm(new, gain2.cpu().double(), 1e-5)
-    past = state[slots.long()].cpu().double()
-    want = h + torch.einsum("bkn,kn->bn", torch.cat([past, h[:, None]], dim=1), w.cpu().double())
-    _close(c2, want, 1e-5 if dtype == torch.float32 else 1e-2)
-    assert not ops.norm_add_conv_fits(4100, 4) and not ops.norm_add_conv_fits(256, 5) and not ops.norm_add_conv_fits(70, 4)
 
 
 @pytest.mark.parametrize("dk,dv,H", [(1, 1, 2), (6, 12, 3), (20, 36, 3), (33, 9, 2), (64, 64, 3), (128, 130, 2), (256, 16, 2), (24, 40, 160)])
