@@ -255,14 +255,16 @@ class KVGroup(PagedGroup):
         h, d = request.n_kv_heads, request.head_dim
         dv = d if getattr(request, "v_head_dim", None) is None else request.v_head_dim
         self.k = torch.zeros((n_lines, self.n_pages, h, self.page_size, d), dtype=geo.dtype, device=geo.device)
-        self.v = torch.zeros((n_lines, self.n_pages, h, dv, self.page_size), dtype=geo.dtype, device=geo.device)
+        hv = h if getattr(request, "n_v_heads", None) is None else request.n_v_heads
+        self.v = torch.zeros((n_lines, self.n_pages, hv, dv, self.page_size), dtype=geo.dtype, device=geo.device)
 
     @staticmethod
     def planned_bytes(request: KVCacheRequest, n_lines: int, geo: Geometry) -> int:
         size = torch.empty((), dtype=geo.dtype).element_size()
         dv = request.head_dim if getattr(request, "v_head_dim", None) is None else request.v_head_dim
+        hv = request.n_kv_heads if getattr(request, "n_v_heads", None) is None else request.n_v_heads
         return (n_lines * PagedGroup.pool_pages(PagedGroup.span_of(request), geo, getattr(request, "keep_first", 0)) * geo.page_size
-                * request.n_kv_heads * (request.head_dim + dv) * size)
+                * (request.n_kv_heads * request.head_dim + hv * dv) * size)
 
     def view(self, line: int, step) -> "CacheLineView":
         return CacheLineView(group=self, line=line, k=self.k[line], v=self.v[line],
@@ -270,7 +272,7 @@ class KVGroup(PagedGroup):
 
     def bytes_per_token(self) -> int:
         r = self.request
-        return self.n_lines * r.n_kv_heads * (r.head_dim + self.v.shape[3]) * self.k.element_size()
+        return self.n_lines * (r.n_kv_heads * r.head_dim + self.v.shape[2] * self.v.shape[3]) * self.k.element_size()
 
 
 class LatentGroup(PagedGroup):

@@ -143,6 +143,14 @@ def _register_builtin() -> None:
         to_spec=lambda cfg: cfg.to_model_spec(),
         checkpoint_names=kakalorn.checkpoint_names,
         unused_tensors=kakalorn.unused_tensors))
+    from . import nazulorn
+    register_architecture(Architecture(
+        name=nazulorn.ARCHITECTURE,
+        read_config=nazulorn.NazulornConfig.from_dict,
+        to_spec=lambda cfg: cfg.to_model_spec(),
+        checkpoint_names=nazulorn.checkpoint_names,
+        unused_tensors=nazulorn.unused_tensors,
+        refine_config=lambda cfg, shapes: cfg.with_shapes(shapes)))
 
 
 _register_builtin()

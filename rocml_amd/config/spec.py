@@ -152,6 +152,26 @@ class LatentAttentionSpec:
 
 
 @dataclass(frozen=True)
+class DifferentialAttentionSpec:
+    """Softmax attention with two maps per head over the same values.  ``q`` has ``n_heads * 2 * head_dim`` rows and ``k``
+    ``n_kv_heads * 2 * head_dim``, head by head ``[map 1, map 2]``; ``v`` has ``n_kv_heads * v_head_dim``.  Each map is an attention of its
+    own (rotated as ``position`` says, scaled by ``scale``, under ``window``); with ``a1``, ``a2`` their outputs and
+    ``lam = exp(sum(lq1 lk1)) - exp(sum(lq2 lk2)) + diff`` (one number for the layer, from four learned vectors of ``head_dim``), the
+    head's output is ``o = a1 - lam a2`` divided by its root mean square (``eps`` inside the root), times ``1 - diff``."""
+    hidden: int
+    n_heads: int
+    n_kv_heads: int
+    head_dim: int
+    v_head_dim: int
+    scale: float
+    diff: float
+    eps: float
+    window: Optional[int] = None
+    position: Optional[RopeSpec] = None
+    kind: str = "differential_attention"
+
+
+@dataclass(frozen=True)
 class GatedMlpSpec:
     """Dense gated feed-forward: ``down(act(g) * (u + up_offset))`` with ``g = gate(x)``,
     ``u = up(x)``.  ``limit``: ``g`` is cut off above at ``limit`` and ``u`` is held inside
@@ -187,7 +207,10 @@ class RoutedExpertsSpec:
     scores for the choice (of groups and of experts) only; the weights use the scores without it.
     ``group_score`` ``"top2_sum"``: a group's score is the sum of its two largest (corrected) scores instead of
     its largest.  ``shared_intermediate``: one more expert of that size runs for every token and is added, with
-    ``shared_gate`` times ``sigmoid(W_sg h)`` (one number per token)."""
+    ``shared_gate`` times ``sigmoid(W_sg h)`` (one number per token).  ``activation``, ``limit``, ``up_offset``: as in ``GatedMlpSpec``, for the
+    experts and (with ``shared_limit`` as its limit) the shared one.  ``identity``: behind the ``n_experts`` the router knows so many
+    more, whose output is their input and which have no matrices; scores, choice and weights do not tell them apart.
+    ``weight_scale``: the weights are multiplied by it in the end."""
     hidden: int
     n_experts: int
     top: int
@@ -202,6 +225,11 @@ class RoutedExpertsSpec:
     group_score: str = "max"
     shared_intermediate: Optional[int] = None
     shared_gate: bool = False
+    limit: Optional[float] = None
+    up_offset: float = 0.0
+    shared_limit: Optional[float] = None
+    identity: int = 0
+    weight_scale: float = 1.0
 
 
 @dataclass(frozen=True)
@@ -296,6 +324,23 @@ class Hgrn2Spec:
 
 
 @dataclass(frozen=True)
+class GatedLinearAttentionSpec:
+    """Linear attention with a decay per token and key channel (gated linear attention): ``q = W_q h``, ``k = W_k h``, ``v = W_v h``;
+    ``alpha = sigmoid(W_a2 (W_a1 h) + b)^(1 / tau)`` with an inner width of ``decay_rank``; per head
+    ``S <- diag(alpha) S + k v^T``, ``o = S^T q head_dim^(-1/2)`` with the new ``S``.  Every head's output is normed over ``v_head_dim`` with
+    one gain for all heads, the heads side by side are multiplied by ``silu(W_g h)`` and projected back.  The state
+    (``head_dim x v_head_dim`` per head) is 32-bit."""
+    hidden: int
+    n_heads: int
+    head_dim: int
+    v_head_dim: int
+    decay_rank: int
+    tau: float
+    eps: float
+    kind: str = "gated_linear_attention"
+
+
+@dataclass(frozen=True)
 class TokenSideSpec:
     """A per-token input that depends on the token's id: with ``e`` the columns ``column0 ..
     column0 + dim - 1`` of the token's row of the model's table ``table``, the result is
@@ -357,13 +402,15 @@ class TokenPositionTableSpec:
 class NormLinearHeadSpec:
     """The model's output: a norm of the wanted rows of the residual stream, then their
     product with a ``[vocab, hidden]`` matrix; ``tied``: that matrix is the input's table.
-    ``softcap``: the logits ``z`` become ``softcap * tanh(z / softcap)``."""
+    ``scale``: the logits are multiplied by it.  ``softcap``: the logits ``z`` become ``softcap * tanh(z / softcap)`` (behind the
+    scale)."""
     vocab: int
     hidden: int
     norm: NormSpec
     tied: bool
     kind: str = "norm_linear"
     softcap: Optional[float] = None
+    scale: float = 1.0
 
 
 @dataclass(frozen=True)
@@ -381,7 +428,12 @@ class BlockSpec:
     ``x += mixer_out_norm(mixer(mixer_norm(x))); x += ffn_out_norm(ffn(ffn_norm(x)))``: a norm before
     and one after every sublayer.  ``input_conv``: what the mixer reads, ``h``, is first replaced by ``h`` plus
     a causal convolution of so many taps over it per channel (no bias); the last ``input_conv - 1`` rows of
-    ``h`` are part of a sequence's state (only in ``pre_norm`` and ``sandwich_norm``)."""
+    ``h`` are part of a sequence's state (only in ``pre_norm`` and ``sandwich_norm``).
+
+    ``linked_streams`` keeps ``streams`` copies ``x_1 .. x_s`` of the stream (hyper-connections): a sublayer reads
+    ``norm(sum_s in[s] x_s)``, and with ``y`` its output every copy becomes ``sum_s mix[s, t] x_s + branch_scale * out[t] * y``; ``in``,
+    ``out`` and ``mix`` are learned numbers of the layer, for each of its sublayers.  A run of such layers starts with copies equal to
+    the stream and leaves their sum as the stream."""
     mixer: Any
     ffn: Any
     mixer_norm: Any
@@ -393,6 +445,8 @@ class BlockSpec:
     mixer_out_norm: Optional[Any] = None
     ffn_out_norm: Optional[Any] = None
     input_conv: Optional[int] = None
+    streams: int = 1
+    branch_scale: float = 1.0
 
 
 @dataclass(frozen=True)
@@ -430,6 +484,7 @@ class ModelSpec:
     pass_offsets: int = 0                   # rows of the table that schedule entries add to the stream
     tables: Tuple[Any, ...] = ()            # matrices that parts of several layers read (``TableSpec``)
     logit_softcap: Optional[float] = None   # the default head's soft cap on the logits
+    logit_scale: float = 1.0                # the default head's factor on the logits
 
     def embedding_spec(self) -> Any:
         return self.embedding if self.embedding is not None else \
@@ -437,7 +492,8 @@ class ModelSpec:
 
     def head_spec(self) -> Any:
         return self.head if self.head is not None else \
-            NormLinearHeadSpec(self.vocab, self.hidden, self.final_norm, self.tie_lm_head, softcap=self.logit_softcap)
+            NormLinearHeadSpec(self.vocab, self.hidden, self.final_norm, self.tie_lm_head, softcap=self.logit_softcap,
+                               scale=self.logit_scale)
 
     def validate(self) -> None:
         from ..errors import ConfigError

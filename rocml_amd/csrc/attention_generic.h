@@ -19,7 +19,9 @@
 //    and the running sum at 1;
 //  * sinks[h]: with sink, the term is exp(sinks[h]) instead: the running maximum starts there;
 //  * softcap: the scaled score s becomes softcap * tanh(s / softcap), before the mask and the slope;
-//  * keep_first: with a window, the first keep_first positions are seen whatever their distance.
+//  * keep_first: with a window, the first keep_first positions are seen whatever their distance;
+//  * key_heads_per_value: so many neighbouring key heads share one value head (the value cache then has fewer heads).
+// The output may be of another type than the queries (TO).
 #pragma once
 #include "common.h"
 
@@ -57,6 +59,7 @@ struct AttnExtra {
     const float* sinks;     // [Hq] or null
     float softcap;          // 0: none
     int keep_first;         // 0: none
+    int key_heads_per_value = 1;
 };
 
 __device__ __forceinline__ int attn_first_key(int pos, int window, int chunk) {
@@ -64,9 +67,9 @@ __device__ __forceinline__ int attn_first_key(int pos, int window, int chunk) {
     return window > 0 ? max(0, pos - window + 1) : 0;
 }
 
-template <typename T>
+template <typename T, typename TO = T>
 __global__ void __launch_bounds__(AG_BLOCK)
-attn_generic_kernel(const T* __restrict__ q, T* __restrict__ out, const T* __restrict__ kcache,
+attn_generic_kernel(const T* __restrict__ q, TO* __restrict__ out, const T* __restrict__ kcache,
                     const T* __restrict__ vcache, const int* __restrict__ block_table, int bt_width,
                     const int* __restrict__ token_seq, const int* __restrict__ token_pos, int hq,
                     int hkv, int d, int page_size, float scale, int window, AttnExtra ex) {
@@ -83,6 +86,7 @@ attn_generic_kernel(const T* __restrict__ q, T* __restrict__ out, const T* __res
     int n_kept = min(ex.keep_first, lo), n_seen = n_kept + pos - lo + 1;
     auto key_of = [&](int i) { return i < n_kept ? i : lo + i - n_kept; };
     int dv = ex.dv;
+    int hv = hkv / ex.key_heads_per_value, vh = kvh / ex.key_heads_per_value;
     float slope = ex.slopes ? ex.slopes[h] : 0.f;
     const T* qrow = q + ((size_t)t * hq + h) * d;
     for (int e = tid; e < d; e += AG_BLOCK) qs[e] = Elem<T>::load(qrow + e);
@@ -124,7 +128,7 @@ attn_generic_kernel(const T* __restrict__ q, T* __restrict__ out, const T* __res
                 for (int jj = 0; jj < n_keys; ++jj) {
                     int key = key_of(c0 + jj);
                     int page = pages[key / page_size];
-                    const T* vcol = vcache + ((size_t)page * hkv + kvh) * dv * page_size + key % page_size;
+                    const T* vcol = vcache + ((size_t)page * hv + vh) * dv * page_size + key % page_size;
                     a = fmaf(ps[jj], Elem<T>::load(vcol + (size_t)e * page_size), a);
                 }
             }
@@ -133,10 +137,10 @@ attn_generic_kernel(const T* __restrict__ q, T* __restrict__ out, const T* __res
         m = m_new;
         __syncthreads();                         // ps is rewritten by the next chunk
     }
-    T* orow = out + ((size_t)t * hq + h) * dv;
+    TO* orow = out + ((size_t)t * hq + h) * dv;
 #pragma unroll
     for (int r = 0; r < AG_MAX_D_PER_THREAD; ++r) {
         int e = tid + r * AG_BLOCK;
-        if (e < dv) Elem<T>::store(orow + e, acc[r] / l);
+        if (e < dv) Elem<TO>::store(orow + e, acc[r] / l);
     }
 }

@@ -3,6 +3,7 @@
 // Norm statistics, angles and the SiLU are computed in 32-bit (angles in 64-bit) whatever
 // the storage type is.
 #include "common.h"
+#include "gated_activation.h"
 
 ROCML_LAST_ERROR_FN(elementwise)
 
@@ -217,15 +218,7 @@ ROCML_EXPORT int rocml_rmsnorm(float* x, const float* gain, void* out, int out_d
 // (rocml-kernels/kernels/silu_mul.hip:12-20).  Gate and up halves lie side by side in a row.
 // With `interleaved` a row holds (gate_0, up_0, gate_1, up_1, ...), the order the fused product
 // epilogue wants its weight rows in.
-// act: 0 silu, 1 relu (max(g, 0)), 2 gelu with the tanh form 0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))),
-// 3 g sigmoid(1.702 g).
-__device__ __forceinline__ float gate_activation(float g, int act) {
-    if (act == 1) return fmaxf(g, 0.f);
-    if (act == 3) return g / (1.0f + expf(-1.702f * g));      // g sigmoid(1.702 g)
-    if (act == 2) return 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
-    return g / (1.0f + expf(-g));
-}
-
+// act: as gate_activation says.
 // out[i] = act(x[i]) without a gate: the activations above, or 4: max(x, 0)^2.
 template <typename TO>
 __global__ void activate_kernel(const float* __restrict__ x, TO* __restrict__ out, long long total, int act) {
@@ -252,39 +245,35 @@ ROCML_EXPORT int rocml_activate(const float* x, void* out, int out_dtype, long l
     return 0;
 }
 
-// limit > 0: g is cut off above at limit and u is held inside [-limit, limit] first; up_offset is
-// added to u (after the limit).
+// limit and up_offset: as gated_value says.  ld: numbers between the starts of two tokens' rows (they may be columns of a
+// wider matrix).
 template <typename TI, typename TO>
-__global__ void swiglu_kernel(const TI* __restrict__ gu, TO* __restrict__ out, int inter,
+__global__ void swiglu_kernel(const TI* __restrict__ gu, int ld, TO* __restrict__ out, int inter,
                               long long total, int interleaved, int act, float limit, float up_offset) {
     long long idx = (long long)blockIdx.x * EW_BLOCK + threadIdx.x;
     if (idx >= total) return;
     long long t = idx / inter;
     int i = (int)(idx - t * inter);
-    const TI* row = gu + (size_t)t * 2 * inter;
+    const TI* row = gu + (size_t)t * ld;
     float g = Elem<TI>::load(row + (interleaved ? 2 * i : i));
     float u = Elem<TI>::load(row + (interleaved ? 2 * i + 1 : inter + i));
-    if (limit > 0.f) {
-        g = fminf(g, limit);
-        u = fminf(fmaxf(u, -limit), limit);
-    }
-    Elem<TO>::store(out + idx, gate_activation(g, act) * (u + up_offset));
+    Elem<TO>::store(out + idx, gated_value(g, u, act, limit, up_offset));
 }
 
-ROCML_EXPORT int rocml_swiglu(const void* gu, int in_dtype, void* out, int out_dtype, int n_tokens,
+ROCML_EXPORT int rocml_swiglu(const void* gu, int in_dtype, int ld, void* out, int out_dtype, int n_tokens,
                               int inter, int interleaved, int act, float limit, float up_offset, hipStream_t stream) {
-    ROCML_REQUIRE(n_tokens >= 0 && inter > 0, "swiglu: bad sizes T=%d I=%d", n_tokens, inter);
+    ROCML_REQUIRE(n_tokens >= 0 && inter > 0 && ld >= 2 * inter, "swiglu: bad sizes T=%d I=%d ld=%d", n_tokens, inter, ld);
     ROCML_REQUIRE(act >= 0 && act <= 3, "swiglu: unknown activation %d (0 silu, 1 relu, 2 gelu_tanh, 3 sigmoid_1702)", act);
     ROCML_REQUIRE(limit >= 0.f, "swiglu: the limit must not be negative (0: none)");
     long long total = (long long)n_tokens * inter;
     if (total == 0) return 0;
     int grid = ceil_div(total, EW_BLOCK);
     if (in_dtype == ROCML_F32 && out_dtype == ROCML_F32)
-        swiglu_kernel<float, float><<<grid, EW_BLOCK, 0, stream>>>((const float*)gu, (float*)out, inter, total, interleaved, act, limit, up_offset);
+        swiglu_kernel<float, float><<<grid, EW_BLOCK, 0, stream>>>((const float*)gu, ld, (float*)out, inter, total, interleaved, act, limit, up_offset);
     else if (in_dtype == ROCML_F32 && out_dtype == ROCML_BF16)
-        swiglu_kernel<float, bf16_t><<<grid, EW_BLOCK, 0, stream>>>((const float*)gu, (bf16_t*)out, inter, total, interleaved, act, limit, up_offset);
+        swiglu_kernel<float, bf16_t><<<grid, EW_BLOCK, 0, stream>>>((const float*)gu, ld, (bf16_t*)out, inter, total, interleaved, act, limit, up_offset);
     else if (in_dtype == ROCML_BF16 && out_dtype == ROCML_BF16)
-        swiglu_kernel<bf16_t, bf16_t><<<grid, EW_BLOCK, 0, stream>>>((const bf16_t*)gu, (bf16_t*)out, inter, total, interleaved, act, limit, up_offset);
+        swiglu_kernel<bf16_t, bf16_t><<<grid, EW_BLOCK, 0, stream>>>((const bf16_t*)gu, ld, (bf16_t*)out, inter, total, interleaved, act, limit, up_offset);
     else
         return rocml_fail("swiglu: unsupported dtype pair in=%d out=%d", in_dtype, out_dtype);
     ROCML_CHECK_LAUNCH("swiglu");
@@ -346,7 +335,8 @@ __global__ void qk_norm_rope_append_kernel(
     const int* __restrict__ block_table, int bt_width, const int* __restrict__ token_seq,
     const int* __restrict__ token_pos, int page_size, int write_kv, int n_splits, long long split_stride,
     int rows_per_token, int pairing, int first_row, const float* __restrict__ bias, int dv,
-    float qt_coef, int qt_every, const float* __restrict__ span_inv, int span_self, int v_col0) {
+    float qt_coef, int qt_every, const float* __restrict__ span_inv, int span_self, int v_col0, int hv) {
+    // hv: value heads (as many as key heads, or fewer where several key heads share one).
     // v_col0: first value column (behind the q and k rows, or at the first k row: values that are the projected keys).
     // span_inv (may be null): [T, 2], the norm's factor of a token's whole q row and whole k row; the gains then
     // have one number per column of the q (k) projection, and a head takes its own part of them.  span_self: the
@@ -489,7 +479,7 @@ __global__ void qk_norm_rope_append_kernel(
         if (page < 0) return;
         if (kind == 2) {
             // values are stored transposed inside a page: [page, Hkv, Dv, page_size]
-            TO* vdst = vcache + ((size_t)page * hkv + head) * dv * page_size + pos % page_size;
+            TO* vdst = vcache + ((size_t)page * hv + head) * dv * page_size + pos % page_size;
 #pragma unroll
             for (int j = 0; j < QK_PER_LANE; ++j) {
                 int e = lane + j * WAVE;
@@ -638,7 +628,8 @@ ROCML_EXPORT int rocml_qk_norm_rope_append(
     void* kcache, void* vcache, int out_dtype, const int* block_table, int bt_width,
     const int* token_seq, const int* token_pos, int page_size, int write_kv, int n_splits,
     long long split_stride, const float* bias, int dv, float qt_coef, int qt_every, const float* span_inv, int span_self,
-    int v_is_k, hipStream_t stream) {
+    int v_is_k, int hv, hipStream_t stream) {
+    // hv (0: hkv): value heads, when several key heads share one
     // v_is_k: the rows hold no value columns, a value is the projected key before norm and rotation (dv = d)
     // span_self: the norm spans a token's whole q row and whole k row as with span_inv, and the kernel forms the
     // factors itself (a step of few tokens)
@@ -656,9 +647,10 @@ ROCML_EXPORT int rocml_qk_norm_rope_append(
                   "qk_norm_rope_append: partial sums must be 32-bit with a positive stride");
     ROCML_REQUIRE(d <= QK_MAX_PER_LANE * WAVE, "qk_norm_rope_append: head_dim %d exceeds %d", d,
                   QK_MAX_PER_LANE * WAVE);
-    ROCML_REQUIRE(!v_is_k || dv == d, "qk_norm_rope_append: values that are the keys have the keys' size");
+    if (hv <= 0) hv = hkv;
+    ROCML_REQUIRE(!v_is_k || (dv == d && hv == hkv), "qk_norm_rope_append: values that are the keys have the keys' size and number");
     const int v_col0 = (v_is_k ? hq : hq + hkv) * d;
-    ROCML_REQUIRE(ld >= v_col0 + hkv * dv || (!write_kv && ld >= hq * d),
+    ROCML_REQUIRE(ld >= v_col0 + hv * dv || (!write_kv && ld >= hq * d),
                   "qk_norm_rope_append: row stride %d too small", ld);
     ROCML_REQUIRE(rot >= 0 && rot <= d && rot % 2 == 0, "qk_norm_rope_append: rot_dim %d must be even and <= %d", rot, d);
     ROCML_REQUIRE(pairing == 0 || pairing == 1, "qk_norm_rope_append: pairing %d (0: halves, 1: neighbours)", pairing);
@@ -677,7 +669,7 @@ ROCML_EXPORT int rocml_qk_norm_rope_append(
     // (without q_out the q rows are left to the caller: the prefill attention that reads the
     // projection prepares its queries itself)
     int first_row = q_out ? 0 : hq;
-    int rows_per_token = hq - first_row + (write_kv ? (v_tiled ? hkv : 2 * hkv) : 0);
+    int rows_per_token = hq - first_row + (write_kv ? (v_tiled ? hkv : hkv + hv) : 0);
     long long rows = (long long)n_tokens * rows_per_token;
     int widest = d > dv ? d : dv;
     int per_lane = widest <= 64 ? 1 : widest <= 128 ? 2 : widest <= 256 ? 4 : 8;     // head values per lane
@@ -693,7 +685,7 @@ ROCML_EXPORT int rocml_qk_norm_rope_append(
     qk_norm_rope_append_kernel<TI, TO, N, LP><<<grid, EW_BLOCK, lds, stream>>>(                 \
         (const TI*)qkv, ld, n_tokens, hq, hkv, d, q_gain, k_gain, eps, cos_t, sin_t, rot,       \
         (TO*)q_out, (TO*)kcache, (TO*)vcache, block_table, bt_width, token_seq, token_pos,      \
-        page_size, write_kv, n_splits, split_stride, rows_per_token, pairing, first_row, bias, dv, qt_coef, qt_every, span_inv, span_self, v_col0)
+        page_size, write_kv, n_splits, split_stride, rows_per_token, pairing, first_row, bias, dv, qt_coef, qt_every, span_inv, span_self, v_col0, hv)
 #define LAUNCH_ROWS(TI, TO, N)                                                                  \
     qk_norm_rope_rows_kernel<TI, TO, N, MANY><<<grid, EW_BLOCK, 0, stream>>>(                   \
         (const TI*)qkv, ld, n_tokens, hq, hkv, d, q_gain, k_gain, eps, rot ? cos_t : nullptr,   \
@@ -707,9 +699,9 @@ ROCML_EXPORT int rocml_qk_norm_rope_append(
         else if (per_lane == 4) { if (local_pair) LAUNCH_N(TI, TO, 4, true); else LAUNCH_N(TI, TO, 4, false); } \
         else { if (local_pair) LAUNCH_N(TI, TO, 8, true); else LAUNCH_N(TI, TO, 8, false); }    \
         if (v_tiled) {                                                                          \
-            dim3 vgrid(ceil_div(n_tokens, VT_TOKENS), hkv, ceil_div(dv, VT_VALUES));            \
+            dim3 vgrid(ceil_div(n_tokens, VT_TOKENS), hv, ceil_div(dv, VT_VALUES));            \
             v_append_tile_kernel<TI, TO><<<vgrid, EW_BLOCK, 0, stream>>>(                       \
-                (const TI*)qkv, ld, n_tokens, v_col0, hkv, dv, (TO*)vcache, block_table,\
+                (const TI*)qkv, ld, n_tokens, v_col0, hv, dv, (TO*)vcache, block_table,\
                 bt_width, token_seq, token_pos, page_size, bias);                               \
         }                                                                                       \
     }

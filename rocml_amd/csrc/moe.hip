@@ -8,6 +8,7 @@
 // pairs of one expert are neighbours; the experts' products work on rows in that order (a tile of
 // MOE_TM rows never spans two experts) and the weighted sum reads them back through `place`.
 #include "common.h"
+#include "gated_activation.h"
 
 ROCML_LAST_ERROR_FN(moe)
 
@@ -36,7 +37,8 @@ __device__ __forceinline__ void wave_argmax(float& v, int& i) {
 __global__ void __launch_bounds__(RT_BLOCK)
 moe_route_kernel(const float* __restrict__ logits, int n_tokens, int n_experts, int top, int group_count, int group_keep,
                  float sum_eps, int* __restrict__ chosen, float* __restrict__ weight, const float* __restrict__ bias,
-                 int sigmoid, const float* __restrict__ correction, int group_top2, int ld) {
+                 int sigmoid, const float* __restrict__ correction, int group_top2, int ld, float weight_scale) {
+    // weight_scale: every weight is multiplied by it in the end
     // ld: numbers between the starts of two tokens' logits (the logits may be the leading columns of a wider matrix)
     // bias (may be null): one number per expert, added to the logits first
     extern __shared__ float rt_smem[];          // [waves][n_experts]
@@ -143,13 +145,13 @@ moe_route_kernel(const float* __restrict__ logits, int n_tokens, int n_experts, 
     }
     if (live && lane < top) {
         chosen[(size_t)t * top + lane] = mine_e;
-        weight[(size_t)t * top + lane] = mine_w / (total + sum_eps);
+        weight[(size_t)t * top + lane] = mine_w / (total + sum_eps) * weight_scale;
     }
 }
 
 ROCML_EXPORT int rocml_moe_route(const float* logits, int n_tokens, int n_experts, int top, int group_count, int group_keep,
                                  float sum_eps, int* chosen, float* weight, const float* bias, int sigmoid,
-                                 const float* correction, int group_top2, int ld, hipStream_t stream) {
+                                 const float* correction, int group_top2, int ld, float weight_scale, hipStream_t stream) {
     ROCML_REQUIRE(ld >= n_experts, "moe_route: rows of %d numbers for %d experts", ld, n_experts);
     ROCML_REQUIRE(n_tokens >= 0 && n_experts > 0 && n_experts <= RT_MAX_PER_LANE * WAVE, "moe_route: %d experts (1 to %d)", n_experts,
                   RT_MAX_PER_LANE * WAVE);
@@ -162,7 +164,7 @@ ROCML_EXPORT int rocml_moe_route(const float* logits, int n_tokens, int n_expert
     size_t lds = (size_t)(RT_BLOCK / WAVE) * n_experts * sizeof(float);
     moe_route_kernel<<<ceil_div(n_tokens, RT_BLOCK / WAVE), RT_BLOCK, lds, stream>>>(logits, n_tokens, n_experts, top, group_count,
                                                                                      group_keep, sum_eps, chosen, weight, bias,
-                                                                                     sigmoid, correction, group_top2, ld);
+                                                                                     sigmoid, correction, group_top2, ld, weight_scale);
     ROCML_CHECK_LAUNCH("moe_route");
     return 0;
 }
@@ -172,7 +174,7 @@ ROCML_EXPORT int rocml_moe_route(const float* logits, int n_tokens, int n_expert
 // place[pair] = its place; tiles[2 i] and tiles[2 i + 1] are the expert and the first place of
 // tile i, n_tiles[0] their number.  Which of an expert's places a pair gets is decided by atomic
 // counters and may differ from run to run; every row of the products is computed by itself, so no
-// result depends on it.
+// result depends on it.  A pair whose choice is n_experts or more (an expert without matrices) has no place: place = -1.
 constexpr int PL_BLOCK = 1024;
 
 __global__ void __launch_bounds__(PL_BLOCK)
@@ -184,7 +186,10 @@ moe_plan_kernel(const int* __restrict__ chosen, int n_pairs, int n_experts, int*
     int* cursor = pl_smem + n_experts;
     for (int e = threadIdx.x; e < n_experts; e += PL_BLOCK) count[e] = 0;
     __syncthreads();
-    for (int p = threadIdx.x; p < n_pairs; p += PL_BLOCK) atomicAdd(&count[chosen[p]], 1);
+    for (int p = threadIdx.x; p < n_pairs; p += PL_BLOCK) {
+        int e = chosen[p];
+        if (e < n_experts) atomicAdd(&count[e], 1);
+    }
     __syncthreads();
     if (threadIdx.x == 0) {
         int at = 0, nt = 0;
@@ -203,7 +208,12 @@ moe_plan_kernel(const int* __restrict__ chosen, int n_pairs, int n_experts, int*
     }
     __syncthreads();
     for (int p = threadIdx.x; p < n_pairs; p += PL_BLOCK) {
-        int at = atomicAdd(&cursor[chosen[p]], 1);
+        int e = chosen[p];
+        if (e >= n_experts) {
+            place[p] = -1;
+            continue;
+        }
+        int at = atomicAdd(&cursor[e], 1);
         order[at] = p;
         place[p] = at;
     }
@@ -226,8 +236,8 @@ ROCML_EXPORT int rocml_moe_plan(const int* chosen, int n_pairs, int n_experts, i
 // For every place r of expert e: out[r, :] = W_e a(r), W_e = w + e * w_expert_stride ([N, K],
 // rows ldw apart).  a(r) is row order[r] / top of `a` when `order` is given (the rows of the
 // step's tokens, gathered) and row r otherwise (rows already in the plan's order).  DUAL: a second
-// matrix w2 of the same shape, and out[r, j] = act(W_e a)[j] * (W2_e a)[j] with act = silu (a gated
-// feed-forward's first two products and its activation in one pass).  Block (x, y): columns
+// matrix w2 of the same shape, and out[r, j] = act((W_e a)[j]) * ((W2_e a)[j] + up_offset) (a gated
+// feed-forward's first two products and its activation in one pass; act, limit and up_offset as in gated_activation.h).  Block (x, y): columns
 // 64 x .. 64 x + 63 of tile y; blocks beyond the plan's number of tiles leave at once.
 struct MoeGemmArgs {
     const void* a;
@@ -244,9 +254,9 @@ struct MoeGemmArgs {
     const int* offsets;
     const int* tiles;
     const int* n_tiles;
+    int act;
+    float limit, up_offset;
 };
-
-__device__ __forceinline__ float moe_silu(float z) { return z / (1.0f + expf(-z)); }
 
 // Any sizes and types, fused multiply-add in 32-bit: the whole 32-bit path and shapes the
 // matrix-core kernel refuses.  64 x 64 outputs at a time (a tile's rows in MOE_TM / 64 passes), 4 x 4
@@ -316,7 +326,7 @@ moe_gemm_plain_kernel(MoeGemmArgs g) {
         for (int j = 0; j < 4; ++j) {
             int gn = n0 + tx * 4 + j;
             if (gn >= g.n) continue;
-            float v = DUAL ? moe_silu(acc[i][j]) * acc2[DUAL ? i : 0][j] : acc[i][j];
+            float v = DUAL ? gated_value(acc[i][j], acc2[DUAL ? i : 0][j], g.act, g.limit, g.up_offset) : acc[i][j];
             Elem<TO>::store((TO*)g.out + (size_t)r * g.ldo + gn, v);
         }
     }
@@ -436,7 +446,7 @@ moe_gemm_mfma_kernel(MoeGemmArgs g) {
             for (int e = 0; e < 4; ++e) {
                 int gn = n0 + nt * 16 + (lane >> 4) * 4 + e;
                 if (gn >= g.n) continue;
-                float v = DUAL ? moe_silu(acc[nt][mt][e]) * acc2[nt * D2][mt * D2][e] : acc[nt][mt][e];
+                float v = DUAL ? gated_value(acc[nt][mt][e], acc2[nt * D2][mt * D2][e], g.act, g.limit, g.up_offset) : acc[nt][mt][e];
                 Elem<TO>::store((TO*)g.out + (size_t)r * g.ldo + gn, v);
             }
         }
@@ -445,7 +455,7 @@ moe_gemm_mfma_kernel(MoeGemmArgs g) {
 ROCML_EXPORT int rocml_moe_gemm(const void* a, int a_dtype, int lda, int a_rows, const int* order, int top, const void* w,
                                 const void* w2, int w_dtype, long long w_expert_stride, int ldw, int n_experts, void* out,
                                 int out_dtype, int ldo, int n_pairs, int n, int k, const int* offsets, const int* tiles,
-                                const int* n_tiles, int max_tiles, int plain, hipStream_t stream) {
+                                const int* n_tiles, int max_tiles, int plain, int act, float limit, float up_offset, hipStream_t stream) {
     ROCML_REQUIRE(n_pairs >= 0 && n > 0 && k > 0 && n_experts > 0 && top >= 1, "moe_gemm: bad sizes pairs=%d n=%d k=%d", n_pairs, n, k);
     ROCML_REQUIRE(lda >= k && ldw >= k && ldo >= n && w_expert_stride >= (long long)(n - 1) * ldw + k,
                   "moe_gemm: strides do not fit the shapes (lda=%d ldw=%d ldo=%d)", lda, ldw, ldo);
@@ -453,8 +463,9 @@ ROCML_EXPORT int rocml_moe_gemm(const void* a, int a_dtype, int lda, int a_rows,
     ROCML_REQUIRE(order ? (long long)a_rows * top >= n_pairs : a_rows >= n_pairs, "moe_gemm: %d rows for %d pairs", a_rows, n_pairs);
     ROCML_REQUIRE(max_tiles >= ceil_div(n_pairs, MOE_TM) && max_tiles >= 1 && max_tiles < 65536, "moe_gemm: room for %d tiles", max_tiles);
     ROCML_REQUIRE(a_dtype == w_dtype, "moe_gemm: activations and weights must share their type");
+    ROCML_REQUIRE(act >= 0 && act <= 3 && limit >= 0.f, "moe_gemm: unknown activation %d or negative limit %g", act, (double)limit);
     if (n_pairs == 0) return 0;
-    MoeGemmArgs g{a, lda, order, top, w, w2, w_expert_stride, ldw, out, ldo, n, k, offsets, tiles, n_tiles};
+    MoeGemmArgs g{a, lda, order, top, w, w2, w_expert_stride, ldw, out, ldo, n, k, offsets, tiles, n_tiles, act, limit, up_offset};
     dim3 grid(ceil_div(n, 64), max_tiles);
     bool dual = w2 != nullptr;
     bool mfma = !plain && a_dtype == ROCML_BF16 && k % 8 == 0 && lda % 8 == 0 && ldw % 8 == 0 && w_expert_stride % 8 == 0;
@@ -489,26 +500,81 @@ ROCML_EXPORT int rocml_moe_gemm(const void* a, int a_dtype, int lda, int a_rows,
 }
 
 // ---- the weighted sum -------------------------------------------------------------------
-// out[t, :] (+)= sum_c weight[t, c] * y[place[t * top + c], :], choices in order (32-bit).
+// out[t, :] (+)= sum_c weight[t, c] * y[place[t * top + c], :], choices in order (32-bit).  A choice without a place is an
+// expert whose output is its input: the token's row of h ([T, n] in the compute type) stands for it.
+template <typename TH>
 __global__ void __launch_bounds__(256)
 moe_combine_kernel(const float* __restrict__ y, const int* __restrict__ place, const float* __restrict__ weight,
-                   float* __restrict__ out, int top, int n, long long total, int accumulate) {
+                   const TH* __restrict__ h, float* __restrict__ out, int top, int n, long long total, int accumulate) {
     long long idx = (long long)blockIdx.x * 256 + threadIdx.x;
     if (idx >= total) return;
     long long t = idx / n;
     int i = (int)(idx - t * n);
     float sum = 0.f;
-    for (int c = 0; c < top; ++c) sum = fmaf(weight[t * top + c], y[(size_t)place[t * top + c] * n + i], sum);
+    for (int c = 0; c < top; ++c) {
+        int at = place[t * top + c];
+        if (at >= 0) sum = fmaf(weight[t * top + c], y[(size_t)at * n + i], sum);
+        else if (h) sum = fmaf(weight[t * top + c], Elem<TH>::load(h + idx), sum);
+    }
     out[idx] = accumulate ? out[idx] + sum : sum;
 }
 
-ROCML_EXPORT int rocml_moe_combine(const float* y, const int* place, const float* weight, float* out, int n_tokens, int top,
-                                   int n, int accumulate, hipStream_t stream) {
+// The same for rows that are whole 16-byte pieces: four values a thread, and up to eight choices' rows on their way at a time.
+template <typename TH>
+__global__ void __launch_bounds__(256)
+moe_combine_vec_kernel(const float* __restrict__ y, const int* __restrict__ place, const float* __restrict__ weight,
+                       const TH* __restrict__ h, float* __restrict__ out, int top, int n, long long total4, int accumulate) {
+    long long idx = (long long)blockIdx.x * 256 + threadIdx.x;
+    if (idx >= total4) return;
+    int n4 = n / 4;
+    long long t = idx / n4;
+    int i = (int)(idx - t * n4) * 4;
+    float4 sum = {0.f, 0.f, 0.f, 0.f};
+    float own[4] = {0.f, 0.f, 0.f, 0.f};
+    if (h) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) own[e] = Elem<TH>::load(h + t * n + i + e);
+    }
+    float4 before = {0.f, 0.f, 0.f, 0.f};
+    if (accumulate) before = *(const float4*)(out + idx * 4);
+    for (int c0 = 0; c0 < top; c0 += 8) {
+        float4 v[8];
+        float w[8];
+        int at[8];
+#pragma unroll
+        for (int c = 0; c < 8; ++c) {
+            int cc = min(c0 + c, top - 1);
+            at[c] = place[t * top + cc];
+            w[c] = weight[t * top + cc];
+            v[c] = at[c] >= 0 ? *(const float4*)(y + (size_t)at[c] * n + i) : float4{own[0], own[1], own[2], own[3]};
+        }
+#pragma unroll
+        for (int c = 0; c < 8; ++c) {
+            if (c0 + c >= top) continue;
+            sum.x = fmaf(w[c], v[c].x, sum.x); sum.y = fmaf(w[c], v[c].y, sum.y);
+            sum.z = fmaf(w[c], v[c].z, sum.z); sum.w = fmaf(w[c], v[c].w, sum.w);
+        }
+    }
+    if (accumulate) { sum.x += before.x; sum.y += before.y; sum.z += before.z; sum.w += before.w; }
+    *(float4*)(out + idx * 4) = sum;
+}
+
+ROCML_EXPORT int rocml_moe_combine(const float* y, const int* place, const float* weight, const void* h, int h_dtype, float* out,
+                                   int n_tokens, int top, int n, int accumulate, hipStream_t stream) {
     ROCML_REQUIRE(n_tokens >= 0 && top >= 1 && n > 0, "moe_combine: bad sizes T=%d top=%d n=%d", n_tokens, top, n);
     ROCML_REQUIRE(y && place && weight && out, "moe_combine: missing arguments");
+    ROCML_REQUIRE(h_dtype == ROCML_F32 || h_dtype == ROCML_BF16, "moe_combine: unknown dtype code %d", h_dtype);
     long long total = (long long)n_tokens * n;
     if (total == 0) return 0;
-    moe_combine_kernel<<<ceil_div(total, 256), 256, 0, stream>>>(y, place, weight, out, top, n, total, accumulate);
+    if (n % 4 == 0 && (((uintptr_t)y | (uintptr_t)out) & 15) == 0) {
+        int grid = ceil_div(total / 4, 256);
+        if (h_dtype == ROCML_BF16) moe_combine_vec_kernel<bf16_t><<<grid, 256, 0, stream>>>(y, place, weight, (const bf16_t*)h, out, top, n, total / 4, accumulate);
+        else moe_combine_vec_kernel<float><<<grid, 256, 0, stream>>>(y, place, weight, (const float*)h, out, top, n, total / 4, accumulate);
+    } else {
+        int grid = ceil_div(total, 256);
+        if (h_dtype == ROCML_BF16) moe_combine_kernel<bf16_t><<<grid, 256, 0, stream>>>(y, place, weight, (const bf16_t*)h, out, top, n, total, accumulate);
+        else moe_combine_kernel<float><<<grid, 256, 0, stream>>>(y, place, weight, (const float*)h, out, top, n, total, accumulate);
+    }
     ROCML_CHECK_LAUNCH("moe_combine");
     return 0;
 }

@@ -1155,7 +1155,8 @@ ROCML_EXPORT int rocml_gated_part_norm(const float* y, const float* z, int ldz, 
 // ---- recurrences with a decay per key channel ---------------------------------------------
 // Per head a state S [dk, dv] that starts at zero, decays row by row and takes the outer product of the
 // token's key and value: S <- diag(w_t) S + k_t v_t^T.  Two ways to read it:
-//   after the update (a retention):        o_t = S_t^T q_t, with w_t one constant per head;
+//   after the update:                      o_t = S_t^T q_t, with w_t one constant per head (a retention) or per token and
+//                                          channel (gated linear attention);
 //   before it, with a bonus on the token:  o_t = (S_(t-1) + diag(u) k_t v_t^T)^T q_t, with w_t per token and channel.
 // A third form writes what it forgets: there is no key, S_t = diag(1 - g_t) S_(t-1) + g_t v_t^T = S_(t-1) + diag(g_t)
 // (v_t^T - S_(t-1)) and o_t = S_t^T silu(q_t), with g_t = (1 - l) sigmoid(-(x_t + b)) from logits x and, per channel, a bias
@@ -1189,6 +1190,7 @@ struct DecayScanArgs {
     const float* gate_bias;                    // bias gate_bias; q is raw and passes silu (there is no key and no other decay)
     float* state; const int* cu_seqlens; const int* seq_slots;
     float* out; int n_heads; int dk; int dv;
+    float out_scale;                           // every output is multiplied by it (a scale of the queries)
 };
 
 // The sigmoid form a / (1 + e^x) by one hardware exponential and one hardware reciprocal: both are good to an ulp or so, and
@@ -1197,20 +1199,22 @@ __device__ __forceinline__ float ds_over_one_plus_exp(float a, float x) {
     return a * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(x * 1.4426950408889634f));
 }
 
-enum DecayMode : int { DECAY_HEAD = 0, DECAY_BONUS = 1, DECAY_GATE = 2 };
+enum DecayMode : int { DECAY_HEAD = 0, DECAY_BONUS = 1, DECAY_GATE = 2, DECAY_TOKEN = 3 };
 
 // R: entries of a column per lane (dk <= 16 R).  CPL: columns per lane.  DECAY_BONUS: a decay per token and channel and a
 // bonus, the state read before its update; DECAY_HEAD: one decay per head, the state read after it; DECAY_GATE: the
-// forget gate that writes (its g in place of the key), the state read after it.
+// forget gate that writes (its g in place of the key), the state read after it; DECAY_TOKEN: a decay per token and channel,
+// the state read after its update.
 // A token's row in LDS has a fixed layout, whatever dk: q, k (and the decays) padded to 16 R numbers each, the block's
 // 16 CPL values, and with DECAY_HEAD the token's decay (the head's, or one for the rows beyond the sequence's last
-// token, which then leave the state as it is: with DECAY_BONUS their decays are one and their keys zero, with DECAY_GATE their g is).  A lane reads its
+// token, which then leave the state as it is: with DECAY_BONUS and DECAY_TOKEN their decays are one and their keys zero, with DECAY_GATE their g is).  A lane reads its
 // R numbers of each part as whole vectors at fixed offsets, without a bound to check.
 template <int R, int CPL, int MODE>
 __global__ void __launch_bounds__(DS_THREADS)
 decay_scan_kernel(DecayScanArgs a) {
     constexpr bool BONUS = MODE == DECAY_BONUS, GATE = MODE == DECAY_GATE, HEAD = MODE == DECAY_HEAD;
-    constexpr int ARRAYS = BONUS ? 3 : 2;
+    constexpr bool TOKEN = MODE == DECAY_TOKEN, ROWS = BONUS || TOKEN;      // ROWS: the decays are rows of their own
+    constexpr int ARRAYS = ROWS ? 3 : 2;
     constexpr int DKP = DS_LANES * R;
     constexpr int TILE = DS_GROUPS * CPL;                            // columns of a block
     constexpr int ROW = ARRAYS * DKP + TILE + (HEAD ? 4 : 0);
@@ -1324,6 +1328,17 @@ decay_scan_kernel(DecayScanArgs a) {
                 }
                 sums[p] = sum;
             }
+        } else if constexpr (TOKEN) {
+#pragma unroll
+            for (int p = 0; p < CPL; ++p) {
+                float sum = 0.f;
+#pragma unroll
+                for (int r = 0; r < R; ++r) {
+                    s[p][r] = fmaf(ww[r], s[p][r], kk[r] * vv[p]);
+                    sum = fmaf(s[p][r], qq[r], sum);
+                }
+                sums[p] = sum;
+            }
         } else {
 #pragma unroll
             for (int p = 0; p < CPL; ++p) {
@@ -1395,7 +1410,7 @@ decay_scan_kernel(DecayScanArgs a) {
                 kk[r] = in ? ds_over_one_plus_exp(1.f - low[r], kk[r] + shift[r]) : 0.f;
             }
         }
-        if constexpr (BONUS) {
+        if constexpr (ROWS) {
             row_part(ww, a.w + t * a.ldw + a.w_col0 + head0);
             if (a.w_offset) {
                 float shift[R];
@@ -1412,7 +1427,7 @@ decay_scan_kernel(DecayScanArgs a) {
         float out_val = sums[0];
 #pragma unroll
         for (int p = 1; p < CPL; ++p) out_val = l == p ? sums[p] : out_val;
-        if (l < CPL && col0 + l < a.dv) a.out[t * a.n_heads * a.dv + (size_t)h * a.dv + col0 + l] = out_val;
+        if (l < CPL && col0 + l < a.dv) a.out[t * a.n_heads * a.dv + (size_t)h * a.dv + col0 + l] = out_val * a.out_scale;
         keep_state();
         return;
     }
@@ -1433,7 +1448,7 @@ decay_scan_kernel(DecayScanArgs a) {
 #pragma unroll
                 for (int j = 0; j < DS_CHUNK; ++j) {
                     float val = next[m][j];
-                    if (BONUS && is_logit[m]) val = expf(-expf(val + offset[m]));
+                    if (ROWS && is_logit[m]) val = expf(-expf(val + offset[m]));
                     if constexpr (GATE) {
                         // silu(q) = q / (1 + e^-q), and g = (1 - l) / (1 + e^(x + b))
                         if (form[m]) {
@@ -1464,7 +1479,7 @@ decay_scan_kernel(DecayScanArgs a) {
                         float4 k4 = *(const float4*)(tok + DKP + 4 * r4);
                         qq[4 * r4] = q4.x; qq[4 * r4 + 1] = q4.y; qq[4 * r4 + 2] = q4.z; qq[4 * r4 + 3] = q4.w;
                         kk[4 * r4] = k4.x; kk[4 * r4 + 1] = k4.y; kk[4 * r4 + 2] = k4.z; kk[4 * r4 + 3] = k4.w;
-                        if constexpr (BONUS) {
+                        if constexpr (ROWS) {
                             float4 w4 = *(const float4*)(tok + 2 * DKP + 4 * r4);
                             ww[4 * r4] = w4.x; ww[4 * r4 + 1] = w4.y; ww[4 * r4 + 2] = w4.z; ww[4 * r4 + 3] = w4.w;
                         }
@@ -1474,7 +1489,7 @@ decay_scan_kernel(DecayScanArgs a) {
                     for (int r = 0; r < R; ++r) {
                         qq[r] = tok[r];
                         kk[r] = tok[DKP + r];
-                        if constexpr (BONUS) ww[r] = tok[2 * DKP + r];
+                        if constexpr (ROWS) ww[r] = tok[2 * DKP + r];
                     }
                 }
                 const float* vals = ds_rows + (j0 + jj) * ROW + ARRAYS * DKP;
@@ -1496,7 +1511,7 @@ decay_scan_kernel(DecayScanArgs a) {
             for (int i = 1; i < NV; ++i) out_val = l == i ? acc[i] : out_val;
             int jj = l / CPL, p = l - jj * CPL;
             if (l < NV && j0 + jj < here && col0 + p < a.dv)
-                a.out[(size_t)(first + t0 + j0 + jj) * a.n_heads * a.dv + (size_t)h * a.dv + col0 + p] = out_val;
+                a.out[(size_t)(first + t0 + j0 + jj) * a.n_heads * a.dv + (size_t)h * a.dv + col0 + p] = out_val * a.out_scale;
         }
         __syncthreads();                         // the rows are rewritten by the next chunk
     }
@@ -1506,7 +1521,8 @@ decay_scan_kernel(DecayScanArgs a) {
 template <int R, int CPL>
 static void launch_decay_scan_cols(const DecayScanArgs& a, int n_seqs, hipStream_t stream) {
     dim3 grid(n_seqs, a.n_heads, ceil_div(a.dv, DS_GROUPS * CPL));
-    if (a.bonus) decay_scan_kernel<R, CPL, DECAY_BONUS><<<grid, DS_THREADS, 0, stream>>>(a);
+    if (a.w && !a.bonus) decay_scan_kernel<R, CPL, DECAY_TOKEN><<<grid, DS_THREADS, 0, stream>>>(a);
+    else if (a.bonus) decay_scan_kernel<R, CPL, DECAY_BONUS><<<grid, DS_THREADS, 0, stream>>>(a);
     else if (a.gate_lower) decay_scan_kernel<R, CPL, DECAY_GATE><<<grid, DS_THREADS, 0, stream>>>(a);
     else decay_scan_kernel<R, CPL, DECAY_HEAD><<<grid, DS_THREADS, 0, stream>>>(a);
 }
@@ -1526,21 +1542,21 @@ ROCML_EXPORT int rocml_decay_scan(const float* q, int ldq, int q_col0, const flo
                                   const float* head_decay, const float* bonus, const float* gate_lower, const float* gate_bias,
                                   float* state, int n_slots, const int* cu_seqlens,
                                   const int* seq_slots, int n_seqs, int n_tokens, float* out, int n_heads, int dk, int dv,
-                                  hipStream_t stream) {
+                                  float out_scale, hipStream_t stream) {
     ROCML_REQUIRE(n_tokens >= 0 && n_seqs >= 0 && n_slots > 0 && n_heads > 0 && dk > 0 && dv > 0, "decay_scan: bad sizes T=%d B=%d H=%d",
                   n_tokens, n_seqs, n_heads);
     ROCML_REQUIRE(dk <= 16 * DS_LANES, "decay_scan: a key size of %d exceeds %d", dk, 16 * DS_LANES);
     ROCML_REQUIRE(q && k && v && state && cu_seqlens && seq_slots && out, "decay_scan: missing arguments");
-    ROCML_REQUIRE((w != nullptr) + (head_decay != nullptr) + (gate_lower != nullptr) == 1 && (w != nullptr) == (bonus != nullptr) &&
+    ROCML_REQUIRE((w != nullptr) + (head_decay != nullptr) + (gate_lower != nullptr) == 1 && (!bonus || w) &&
                       (gate_lower != nullptr) == (gate_bias != nullptr),
-                  "decay_scan: a decay per token and channel with a bonus, one decay per head without, or a forget gate's lower bound and bias");
+                  "decay_scan: a decay per token and channel (with a bonus or without), one decay per head, or a forget gate's lower bound and bias");
     ROCML_REQUIRE(!w_offset || w, "decay_scan: an offset goes with decays given as logits");
     ROCML_REQUIRE(q_col0 >= 0 && k_col0 >= 0 && v_col0 >= 0 && ldq >= q_col0 + n_heads * dk && ldk >= k_col0 + n_heads * dk &&
                       ldv >= v_col0 + n_heads * dv && (!w || (w_col0 >= 0 && ldw >= w_col0 + n_heads * dk)),
                   "decay_scan: a row stride is too small for its columns");
     if (n_tokens == 0 || n_seqs == 0) return 0;
     DecayScanArgs a{q, ldq, q_col0, k, ldk, k_col0, v, ldv, v_col0, w, ldw, w_col0, w_offset, head_decay, bonus, gate_lower, gate_bias, state, cu_seqlens,
-                    seq_slots, out, n_heads, dk, dv};
+                    seq_slots, out, n_heads, dk, dv, out_scale};
     int r = ceil_div(dk, DS_LANES);
     if (r <= 1) launch_decay_scan<1>(a, n_seqs, stream);
     else if (r <= 2) launch_decay_scan<2>(a, n_seqs, stream);
@@ -1548,6 +1564,71 @@ ROCML_EXPORT int rocml_decay_scan(const float* q, int ldq, int q_col0, const flo
     else if (r <= 8) launch_decay_scan<8>(a, n_seqs, stream);
     else launch_decay_scan<16>(a, n_seqs, stream);
     ROCML_CHECK_LAUNCH("decay_scan");
+    return 0;
+}
+
+// ---- decays from a low-rank product --------------------------------------------------------
+// decay[t, c] = sigmoid(z)^(1 / tau) with z = bias[c] + sum_r w[r, c] * low[t, r]: the second of two small matrices, the
+// sigmoid and the root in one pass, all 32-bit.  low is `rank` columns (from low_col0 on) of rows of ldl 32-bit numbers, w is
+// [rank, n] (neighbouring channels side by side).  A block takes 256 channels and LD_TOKENS tokens, whose rows of `low` lie in LDS.
+constexpr int LD_TOKENS = 8;
+constexpr int LD_RANK = 64;      // numbers of a token's row in LDS at a time
+
+template <typename TW, int TB>
+__global__ void __launch_bounds__(RC_BLOCK)
+low_rank_decay_kernel(const float* __restrict__ low, int ldl, int low_col0, const TW* __restrict__ w, const float* __restrict__ bias,
+                      float inv_tau, float* __restrict__ decay, int n_tokens, int n, int rank) {
+    __shared__ float rows[TB][LD_RANK];
+    int c = blockIdx.x * RC_BLOCK + threadIdx.x;
+    int t0 = blockIdx.y * TB;
+    float z[TB];
+#pragma unroll
+    for (int j = 0; j < TB; ++j) z[j] = 0.f;
+    for (int r0 = 0; r0 < rank; r0 += LD_RANK) {
+        int here = min(LD_RANK, rank - r0);
+        if (r0 > 0) __syncthreads();
+        for (int i = threadIdx.x; i < TB * here; i += RC_BLOCK) {
+            int j = i / here, r = i - j * here;
+            rows[j][r] = t0 + j < n_tokens ? low[(size_t)(t0 + j) * ldl + low_col0 + r0 + r] : 0.f;
+        }
+        __syncthreads();
+        if (c < n) {
+#pragma unroll 8
+            for (int r = 0; r < here; ++r) {
+                float wv = Elem<TW>::load(w + (size_t)(r0 + r) * n + c);
+#pragma unroll
+                for (int j = 0; j < TB; ++j) z[j] = fmaf(wv, rows[j][r], z[j]);
+            }
+        }
+    }
+    if (c >= n) return;
+    float b = bias ? bias[c] : 0.f;
+#pragma unroll
+    for (int j = 0; j < TB; ++j) {
+        if (t0 + j >= n_tokens) continue;
+        float v = z[j] + b;
+        // log sigmoid(v) = min(v, 0) - log(1 + e^-|v|)
+        float logs = fminf(v, 0.f) - log1pf(expf(-fabsf(v)));
+        decay[(size_t)(t0 + j) * n + c] = expf(logs * inv_tau);
+    }
+}
+
+ROCML_EXPORT int rocml_low_rank_decay(const float* low, int ldl, int low_col0, const void* w, int w_dtype, const float* bias, float tau,
+                                      float* decay, int n_tokens, int n, int rank, hipStream_t stream) {
+    ROCML_REQUIRE(n_tokens >= 0 && n > 0 && rank > 0 && low_col0 >= 0 && ldl >= low_col0 + rank && tau > 0.f && low && w && decay,
+                  "low_rank_decay: bad arguments T=%d n=%d rank=%d ld=%d tau=%g", n_tokens, n, rank, ldl, (double)tau);
+    ROCML_REQUIRE(w_dtype == ROCML_F32 || w_dtype == ROCML_BF16, "low_rank_decay: unknown dtype code %d", w_dtype);
+    if (n_tokens == 0) return 0;
+    ROCML_REQUIRE(n_tokens <= 65535 * LD_TOKENS, "low_rank_decay: %d tokens are too many", n_tokens);
+    // few tokens: one a block, so that their channels spread over the chip
+    bool few = n_tokens <= 64;
+    dim3 grid(ceil_div(n, RC_BLOCK), few ? n_tokens : ceil_div(n_tokens, LD_TOKENS));
+    float inv = 1.0f / tau;
+#define LRD(TW_, TB_) low_rank_decay_kernel<TW_, TB_><<<grid, RC_BLOCK, 0, stream>>>(low, ldl, low_col0, (const TW_*)w, bias, inv, decay, n_tokens, n, rank)
+    if (w_dtype == ROCML_BF16) { if (few) LRD(bf16_t, 1); else LRD(bf16_t, LD_TOKENS); }
+    else { if (few) LRD(float, 1); else LRD(float, LD_TOKENS); }
+#undef LRD
+    ROCML_CHECK_LAUNCH("low_rank_decay");
     return 0;
 }
 

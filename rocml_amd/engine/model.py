@@ -55,12 +55,10 @@ class DecoderModel:
     def kernel_families(self):
         """The kernel libraries this model's steps launch from: the ones every model needs and those
         its parts name (``kernel_families``), so that a fresh checkout compiles what the model uses."""
-        families = list(ops.MODEL_FAMILIES)
+        wanted = set(ops.MODEL_FAMILIES)
         for part in [self.embedding, self.head] + self.blocks:
-            for f in getattr(part, "kernel_families", ()):
-                if f not in families:
-                    families.append(f)
-        return tuple(families)
+            wanted.update(getattr(part, "kernel_families", ()))
+        return tuple(f for f in ops.FAMILIES if f in wanted)
 
     @property
     def embed(self) -> Optional[torch.Tensor]:

@@ -29,10 +29,10 @@ _SIGNATURES = {
     "elementwise": {
         "rocml_embed_gather": [_P, _I, _P, _P, _I, _I, _I, _F, _P, _P, _I, _P],
         "rocml_rmsnorm": [_P, _P, _P, _I, _P, _I, _I, _F, _P, _I, _LL, _P],
-        "rocml_swiglu": [_P, _I, _P, _I, _I, _I, _I, _I, _F, _F, _P],
+        "rocml_swiglu": [_P, _I, _I, _P, _I, _I, _I, _I, _I, _F, _F, _P],
         "rocml_rope_table": [_P, _P, _P, _P, _I, _I, _F, _P],
         "rocml_qk_norm_rope_append": [_P, _I, _I, _I, _I, _I, _I, _P, _P, _F, _P, _P, _I, _I, _P, _P, _P,
-                                      _I, _P, _I, _P, _P, _I, _I, _I, _LL, _P, _I, _F, _I, _P, _I, _I, _P],
+                                      _I, _P, _I, _P, _P, _I, _I, _I, _LL, _P, _I, _F, _I, _P, _I, _I, _I, _P],
         "rocml_qk_span_stats": [_P, _I, _I, _I, _I, _I, _P, _F, _P, _P],
         "rocml_norm_add": [_P, _P, _I, _I, _P, _P, _F, _I, _P, _I, _P, _I, _LL, _I, _P, _F, _P],
         "rocml_added_conv": [_P, _P, _I, _I, _I, _P, _I, _P, _I, _P, _P, _I, _P, _P],
@@ -62,17 +62,18 @@ _SIGNATURES = {
         "rocml_mlstm_scan": [_P, _I, _I, _I, _I, _I, _I, _P, _P, _F, _F, _F, _P, _P, _P, _I, _P, _P, _I, _I, _P, _I, _I, _I, _P],
         "rocml_mlstm_tile": [],
         "rocml_head_norm_gate": [_P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _F, _I, _P],
-        "rocml_decay_scan": [_P, _I, _I, _P, _I, _I, _P, _I, _I, _P, _I, _I, _P, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _P, _I, _I, _I, _P],
+        "rocml_decay_scan": [_P, _I, _I, _P, _I, _I, _P, _I, _I, _P, _I, _I, _P, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _P, _I, _I, _I, _F, _P],
+        "rocml_low_rank_decay": [_P, _I, _I, _P, _I, _P, _F, _P, _I, _I, _I, _P],
         "rocml_rotate_rows": [_P, _I, _I, _I, _I, _I, _I, _P, _P, _F, _I, _F, _P],
         "rocml_shift_mix": [_P, _I, _I, _I, _P, _I, _P, _I, _P, _P, _P, _I, _P, _P],
         "rocml_tanh": [_P, _P, _I, _LL, _P],
         "rocml_double_exp_decay": [_P, _P, _I, _I, _P],
     },
     "moe": {
-        "rocml_moe_route": [_P, _I, _I, _I, _I, _I, _F, _P, _P, _P, _I, _P, _I, _I, _P],
+        "rocml_moe_route": [_P, _I, _I, _I, _I, _I, _F, _P, _P, _P, _I, _P, _I, _I, _F, _P],
         "rocml_moe_plan": [_P, _I, _I, _P, _P, _P, _P, _P, _I, _P],
-        "rocml_moe_gemm": [_P, _I, _I, _I, _P, _I, _P, _P, _I, _LL, _I, _I, _P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _P],
-        "rocml_moe_combine": [_P, _P, _P, _P, _I, _I, _I, _I, _P],
+        "rocml_moe_gemm": [_P, _I, _I, _I, _P, _I, _P, _P, _I, _LL, _I, _I, _P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _I, _F, _F, _P],
+        "rocml_moe_combine": [_P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _P],
     },
     "gemm": {
         "rocml_gemm": [_P, _I, _I, _P, _I, _I, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P, _P, _LL, _P, _I, _F, _I, _P],
@@ -89,12 +90,23 @@ _SIGNATURES = {
         "rocml_attention_prefill_fused": [_P, _I, _P, _F, _P, _P, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _F, _I,
                                           _P, _I, _P, _P],
     },
+    "streams": {
+        "rocml_stream_links": [_P, _I, _P, _P, _I, _LL, _I, _P, _P, _P, _P, _P, _P, _F, _P, _I, _I, _I, _I, _P],
+    },
+    "diff_attention": {
+        "rocml_diff_attention_sizes_ok": [_I, _I, _I],
+        "rocml_diff_attention_max_group": [],
+        "rocml_diff_attention": [_P, _P, _P, _P, _I, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _F, _F, _F, _P, _I, _P, _P, _I, _P],
+        "rocml_diff_attention_decode": [_P, _I, _I, _LL, _P, _P, _I, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _F, _I, _F, _F, _F, _I,
+                                        _P, _LL, _P],
+    },
     "sampling": {
         "rocml_sample": [_P, _P, _I, _I, _P, _P, _P, _P, _P, _P, _I, _P, _I, _P, _P],
         "rocml_argmax": [_P, _I, _I, _P, _P, _P],
     },
 }
 
+FAMILIES = _build.FAMILIES
 _libs: Dict[str, ctypes.CDLL] = {}
 
 
@@ -114,8 +126,8 @@ def library(family: str) -> ctypes.CDLL:
     return lib
 
 
-MODEL_FAMILIES = ("elementwise", "gemm", "attention")   # what every model's step needs; sampling comes with generation,
-                                                        # and a part with kernels of another family names it (``kernel_families``)
+MODEL_FAMILIES = ("elementwise", "gemm")    # what every model's step needs; sampling comes with generation,
+                                            # and a part with kernels of another family names it (``kernel_families``)
 
 
 def prepare(families=tuple(_SIGNATURES)) -> None:
@@ -247,19 +259,22 @@ GATE_ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2, "sigmoid_1702": 3}    
 
 def swiglu(gate_up: torch.Tensor, out: torch.Tensor, interleaved: bool = False, activation: str = "silu",
            limit: Optional[float] = None, up_offset: float = 0.0) -> None:
-    """``out = act(gate) * (up + up_offset)``.  ``gate_up`` rows hold the gate half then the up half, or
-    (gate, up) pairs when ``interleaved``; ``activation`` is one of ``GATE_ACTIVATIONS``.  ``limit``:
+    """``out = act(gate) * (up + up_offset)``.  ``gate_up`` rows (which may be a column range of a wider matrix) hold the gate half
+    then the up half, or (gate, up) pairs when ``interleaved``; ``activation`` is one of ``GATE_ACTIVATIONS``.  ``limit``:
     the gate is cut off above at ``limit`` and the up value is held inside ``[-limit, limit]`` first."""
     if limit is not None and not limit > 0:
         raise KernelError(f"the limit of a gated activation must be positive, got {limit}")
     if activation not in GATE_ACTIVATIONS:
         raise KernelError(f"unknown activation {activation!r}; known: {sorted(GATE_ACTIVATIONS)}")
-    _dev(gate_up, out)
+    _dev(out)
+    if not gate_up.is_cuda:
+        raise KernelError("kernel arguments must be GPU tensors; this library has no CPU path")
     n_tokens, inter = out.shape
-    if gate_up.shape != (n_tokens, 2 * inter):
-        raise KernelError(f"gate/up is {tuple(gate_up.shape)}, expected {(n_tokens, 2 * inter)}")
+    if gate_up.shape != (n_tokens, 2 * inter) or gate_up.stride(1) != 1:
+        raise KernelError(f"gate/up is {tuple(gate_up.shape)}, expected {(n_tokens, 2 * inter)} with unit inner stride")
+    ld = gate_up.stride(0) if n_tokens > 1 else max(gate_up.stride(0), 2 * inter)
     _check("elementwise", library("elementwise").rocml_swiglu(
-        _ptr(gate_up), _code(gate_up), _ptr(out), _code(out), n_tokens, inter, 1 if interleaved else 0,
+        _ptr(gate_up), _code(gate_up), ld, _ptr(out), _code(out), n_tokens, inter, 1 if interleaved else 0,
         GATE_ACTIVATIONS[activation], 0.0 if limit is None else float(limit), float(up_offset), _stream()))
 
 
@@ -304,7 +319,7 @@ def qk_norm_rope_append(qkv: torch.Tensor, n_heads: int, n_kv_heads: int, head_d
                         token_seq: torch.Tensor, token_pos: torch.Tensor, write_kv: bool = True,
                         n_splits: int = 1, pairing: str = "halves", bias: Optional[torch.Tensor] = None,
                         v_head_dim: Optional[int] = None, q_temp=None, span_inv: Optional[torch.Tensor] = None,
-                        span_self: bool = False, values_are_keys: bool = False) -> None:
+                        span_self: bool = False, values_are_keys: bool = False, n_v_heads: Optional[int] = None) -> None:
     """``qkv`` is ``[T, ld]`` with q, k, v side by side (k and v may be absent when
     ``write_kv`` is false).  Keys are ``[pages, Hkv, page_size, D]``, values
     ``[pages, Hkv, D, page_size]``.  ``pairing``: which two values of the rotated width turn
@@ -318,7 +333,9 @@ def qk_norm_rope_append(qkv: torch.Tensor, n_heads: int, n_kv_heads: int, head_d
     factors of a norm over a token's whole q row and whole k row (``qk_span_stats``); the gains then
     have one number per column of the q and of the k projection.  ``span_self``: the same norm, its
     factors formed inside the kernel (for steps of few tokens).  ``values_are_keys``: ``qkv`` holds no value columns, a
-    value is the projected key (with its bias) before norm and rotation."""
+    value is the projected key (with its bias) before norm and rotation.  ``n_v_heads``: the number of value heads when it is not
+    the key heads' (several key heads share one)."""
+    hv = n_kv_heads if n_v_heads is None else int(n_v_heads)
     qt_coef, qt_every = (0.0, 0) if q_temp is None else (float(q_temp[0]), int(q_temp[1]))
     if q_temp is not None and qt_every <= 0:
         raise KernelError(f"the period of the query's stretch must be positive, got {qt_every}")
@@ -336,7 +353,7 @@ def qk_norm_rope_append(qkv: torch.Tensor, n_heads: int, n_kv_heads: int, head_d
     if bias is not None:
         _want(bias, torch.float32, "projection bias")
         # (rows may be wider than the projection: a product shared with other mixers, whose columns follow)
-        if bias.numel() > ld or bias.numel() < n_heads * head_dim + (n_kv_heads * (head_dim + (0 if values_are_keys else dv)) if write_kv else 0):
+        if bias.numel() > ld or bias.numel() < n_heads * head_dim + (n_kv_heads * head_dim + (0 if values_are_keys else hv * dv) if write_kv else 0):
             raise KernelError(f"the bias has {bias.numel()} values for rows of {ld}")
     whole = span_inv is not None or span_self
     if span_inv is not None:
@@ -363,7 +380,7 @@ def qk_norm_rope_append(qkv: torch.Tensor, n_heads: int, n_kv_heads: int, head_d
         if k_cache is None or v_cache is None or block_table is None:
             raise KernelError("appending to the cache needs the cache and the block table")
         if k_cache.shape[1:] != (n_kv_heads, k_cache.shape[2], head_dim) \
-                or v_cache.shape != (k_cache.shape[0], n_kv_heads, dv, k_cache.shape[2]):
+                or v_cache.shape != (k_cache.shape[0], hv, dv, k_cache.shape[2]):
             raise KernelError(f"cache shape {tuple(k_cache.shape)} does not fit {n_kv_heads} heads of {head_dim}")
         if q_out is not None and k_cache.dtype != q_out.dtype:
             raise KernelError("cache and q output must share their type")
@@ -374,7 +391,7 @@ def qk_norm_rope_append(qkv: torch.Tensor, n_heads: int, n_kv_heads: int, head_d
         eps, _ptr(cos), _ptr(sin), rot_dim if cos is not None else 0, ROPE_PAIRINGS[pairing], _ptr(q_out), _ptr(k_cache),
         _ptr(v_cache), _code(q_out if q_out is not None else k_cache), _ptr(block_table), bt_width, _ptr(token_seq),
         _ptr(token_pos), page_size, 1 if write_kv else 0, n_splits, split_stride, _ptr(bias), dv, qt_coef, qt_every,
-        _ptr(span_inv), 1 if span_self else 0, 1 if values_are_keys else 0, _stream()))
+        _ptr(span_inv), 1 if span_self else 0, 1 if values_are_keys else 0, hv, _stream()))
 
 
 def qk_span_stats(qkv: torch.Tensor, q_width: int, k_width: int, bias: Optional[torch.Tensor], eps: float,
@@ -1326,15 +1343,15 @@ def decay_scan(q: torch.Tensor, q_col0: int, k: torch.Tensor, k_col0: int, v: to
                n_heads: int, head_dim: int, v_head_dim: int, head_decay: Optional[torch.Tensor] = None,
                decay: Optional[torch.Tensor] = None, decay_col0: int = 0, bonus: Optional[torch.Tensor] = None,
                decay_offset: Optional[torch.Tensor] = None, gate_lower: Optional[torch.Tensor] = None,
-               gate_bias: Optional[torch.Tensor] = None) -> None:
+               gate_bias: Optional[torch.Tensor] = None, out_scale: float = 1.0) -> None:
     """A recurrence whose state per head, ``S [dk, dv]``, decays row by row, over the step's tokens, per sequence in
     order: ``S <- diag(w_t) S + k_t v_t^T``.  With ``head_decay`` (one number per head) ``w_t`` is that constant and
     the output reads the new state, ``o_t = S_t^T q_t``; with ``decay`` (per token and key channel, columns
-    ``decay_col0 ..`` of a 32-bit matrix) and ``bonus`` ``u [H * dk]`` the output reads the state before the update,
-    ``o_t = (S_(t-1) + diag(u) k_t v_t^T)^T q_t``.  With ``decay_offset`` (``[H * dk]``) ``decay`` holds logits ``x`` and the
+    ``decay_col0 ..`` of a 32-bit matrix) alone it reads the new state too, and with ``bonus`` ``u [H * dk]`` beside it the
+    state before the update, ``o_t = (S_(t-1) + diag(u) k_t v_t^T)^T q_t``.  With ``decay_offset`` (``[H * dk]``) ``decay`` holds logits ``x`` and the
     decay is ``exp(-exp(x + decay_offset))``.  With ``gate_lower`` ``l`` and ``gate_bias`` ``b`` (``[H * dk]`` each) ``k`` holds the
     logits of a forget gate ``f = l + (1 - l) sigmoid(k + b)`` that decides what is written too, ``S <- diag(f) S + (1 - f) v^T``,
-    ``o = S^T silu(q)`` with the new state.  q, k, v are column ranges of 32-bit matrices ``[T, ld]``;
+    ``o = S^T silu(q)`` with the new state.  ``out_scale`` multiplies every output.  q, k, v are column ranges of 32-bit matrices ``[T, ld]``;
     ``state [slots, H, dv, dk]``; ``out [T, H * dv]``; all 32-bit."""
     _dev(q, k, v, state, cu_seqlens, seq_slots, out, head_decay, decay, bonus, decay_offset, gate_lower, gate_bias)
     for t, what in ((q, "queries"), (k, "keys"), (v, "values"), (state, "recurrent state"), (out, "recurrence output")):
@@ -1345,9 +1362,9 @@ def decay_scan(q: torch.Tensor, q_col0: int, k: torch.Tensor, k_col0: int, v: to
     if out.shape != (n_tokens, n_heads * v_head_dim) or cu_seqlens.numel() != n_seqs + 1 \
             or any(t.dim() != 2 or t.shape[0] != n_tokens for t in (q, k, v)):
         raise KernelError("recurrence inputs, output or tables do not fit the step")
-    if sum(t is not None for t in (head_decay, decay, gate_lower)) != 1 or (decay is None) != (bonus is None) \
+    if sum(t is not None for t in (head_decay, decay, gate_lower)) != 1 or (decay is None and bonus is not None) \
             or (gate_lower is None) != (gate_bias is None):
-        raise KernelError("the recurrence takes one decay per head, a decay per token and channel together with a bonus, or a "
+        raise KernelError("the recurrence takes one decay per head, a decay per token and channel (with a bonus or without), or a "
                           "forget gate's lower bound and bias")
     if decay_offset is not None and decay is None:
         raise KernelError("an offset of the decays' logits goes with decays per token")
@@ -1363,7 +1380,21 @@ def decay_scan(q: torch.Tensor, q_col0: int, k: torch.Tensor, k_col0: int, v: to
         0 if decay is None else decay.shape[1], decay_col0, _ptr(decay_offset), _ptr(head_decay), _ptr(bonus), _ptr(gate_lower),
         _ptr(gate_bias), _ptr(state),
         state.shape[0],
-        _ptr(cu_seqlens), _ptr(seq_slots), n_seqs, n_tokens, _ptr(out), n_heads, head_dim, v_head_dim, _stream()))
+        _ptr(cu_seqlens), _ptr(seq_slots), n_seqs, n_tokens, _ptr(out), n_heads, head_dim, v_head_dim, float(out_scale), _stream()))
+
+
+def low_rank_decay(low: torch.Tensor, low_col0: int, w: torch.Tensor, bias: Optional[torch.Tensor], tau: float, out: torch.Tensor) -> None:
+    """``out[t, c] = sigmoid(z)^(1 / tau)`` with ``z = bias[c] + sum_r w[r, c] * low[t, low_col0 + r]``, all in 32-bit: ``low`` a
+    32-bit matrix, ``w [rank, n]`` in 32-bit or bfloat16, ``out [T, n]``."""
+    _dev(low, w, bias, out)
+    _want(low, torch.float32, "the small product")
+    _want(out, torch.float32, "decays")
+    rank, n = w.shape
+    if low.dim() != 2 or out.shape != (low.shape[0], n) or low.shape[1] < low_col0 + rank \
+            or (bias is not None and (bias.dtype != torch.float32 or bias.numel() != n)):
+        raise KernelError(f"low_rank_decay: low {tuple(low.shape)}, w {tuple(w.shape)} or bias do not fit decays {tuple(out.shape)}")
+    _check("recurrent", library("recurrent").rocml_low_rank_decay(_ptr(low), low.shape[1], low_col0, _ptr(w), _code(w), _ptr(bias), float(tau),
+                                                                _ptr(out), low.shape[0], n, rank, _stream()))
 
 
 def rotate_rows(buf: torch.Tensor, col0: int, n_heads: int, head_dim: int, rot_dim: int, cos: Optional[torch.Tensor],
@@ -1431,10 +1462,10 @@ def moe_max_tiles(n_pairs: int, n_experts: int) -> int:
 
 def moe_route(logits: torch.Tensor, top: int, groups, sum_eps: float, chosen: torch.Tensor, weight: torch.Tensor,
               bias: Optional[torch.Tensor] = None, sigmoid: bool = False, correction: Optional[torch.Tensor] = None,
-              group_top2: bool = False) -> None:
+              group_top2: bool = False, weight_scale: float = 1.0) -> None:
     """Softmax over all experts, the ``top`` best (of the experts of the ``groups[1]`` best of
     ``groups[0]`` equal groups of neighbours, a group's score being its largest, if ``groups`` is
-    given), weights = chosen scores / (their sum + ``sum_eps``).  ``chosen`` int32, ``weight`` float32,
+    given), weights = chosen scores / (their sum + ``sum_eps``) * ``weight_scale``.  ``chosen`` int32, ``weight`` float32,
     both ``[T, top]``.  ``bias``: 32-bit, one number per expert, added to the logits first.  ``sigmoid``: an
     expert's score is ``sigmoid(logit)`` instead of the softmax.  ``correction``: 32-bit, one number per expert,
     added to the scores for the choice of groups and experts only.  ``group_top2``: a group's score is the sum of
@@ -1456,11 +1487,13 @@ def moe_route(logits: torch.Tensor, top: int, groups, sum_eps: float, chosen: to
     _check("moe", library("moe").rocml_moe_route(_ptr(logits), n_tokens, n_experts, top, count, keep, float(sum_eps),
                                                  _ptr(chosen), _ptr(weight), _ptr(bias), 1 if sigmoid else 0,
                                                  _ptr(correction), 1 if group_top2 else 0,
-                                                 logits.stride(0) if n_tokens > 1 else max(logits.stride(0), n_experts), _stream()))
+                                                 logits.stride(0) if n_tokens > 1 else max(logits.stride(0), n_experts), float(weight_scale),
+                                                 _stream()))
 
 
 def moe_plan(chosen: torch.Tensor, n_experts: int, plan: torch.Tensor):
-    """Sorts the (token, choice) pairs by expert.  ``plan`` is int32 scratch of at least
+    """Sorts the (token, choice) pairs by expert; a choice of ``n_experts`` or more (an expert without matrices) gets no place
+    (``place`` -1).  ``plan`` is int32 scratch of at least
     ``moe_plan_words(pairs, experts)`` words; returns its views
     ``(offsets [E + 1], order [pairs], place [pairs], tiles [2 * max_tiles], n_tiles [1], max_tiles)``."""
     _dev(chosen, plan)
@@ -1486,11 +1519,14 @@ def moe_plan_words(n_pairs: int, n_experts: int) -> int:
 
 
 def moe_gemm(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, plan, top: int, gather: bool,
-             w2: Optional[torch.Tensor] = None, plain: bool = False) -> None:
+             w2: Optional[torch.Tensor] = None, plain: bool = False, activation: str = "silu", limit: Optional[float] = None,
+             up_offset: float = 0.0) -> None:
     """The products of all experts over the plan's order: row ``r`` of ``out`` (a place of expert
     ``e``) is ``w[e] @ a_r``, with ``a_r`` the row of the pair's token when ``gather`` (``a`` holds the
-    step's tokens) and row ``r`` of ``a`` otherwise.  With ``w2``: ``silu(w[e] a_r) * (w2[e] a_r)``.
-    ``w`` is ``[experts, n, k]``."""
+    step's tokens) and row ``r`` of ``a`` otherwise.  With ``w2``: ``act(w[e] a_r) * (w2[e] a_r + up_offset)``, gate and up values held
+    under ``limit`` first (as in ``swiglu``).  ``w`` is ``[experts, n, k]``."""
+    if activation not in GATE_ACTIVATIONS or (limit is not None and not limit > 0):
+        raise KernelError(f"unknown activation {activation!r} or a limit that is not positive; known: {sorted(GATE_ACTIVATIONS)}")
     offsets, order, place, tiles, n_tiles, max_tiles = plan
     _dev(a, w, w2, out)
     n_experts, n, k = w.shape
@@ -1502,17 +1538,148 @@ def moe_gemm(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, plan, top: int
     _check("moe", library("moe").rocml_moe_gemm(
         _ptr(a), _code(a), a.shape[1], a.shape[0], _ptr(order) if gather else None, top, _ptr(w), _ptr(w2), _code(w), n * k, k,
         n_experts, _ptr(out), _code(out), n, n_pairs, n, k, _ptr(offsets), _ptr(tiles), _ptr(n_tiles), max_tiles,
-        1 if plain else 0, _stream()))
+        1 if plain else 0, GATE_ACTIVATIONS[activation], 0.0 if limit is None else float(limit), float(up_offset), _stream()))
 
 
-def moe_combine(y: torch.Tensor, plan, weight: torch.Tensor, out: torch.Tensor, accumulate: bool = False) -> None:
-    """``out[t] (+)= sum_c weight[t, c] * y[place[t * top + c]]`` (32-bit, choices in order)."""
+def moe_combine(y: torch.Tensor, plan, weight: torch.Tensor, out: torch.Tensor, accumulate: bool = False,
+                own: Optional[torch.Tensor] = None) -> None:
+    """``out[t] (+)= sum_c weight[t, c] * y[place[t * top + c]]`` (32-bit, choices in order).  A choice without a place is an expert
+    whose output is its input: ``own[t]`` (the experts' input) stands for its row."""
     offsets, order, place, tiles, n_tiles, max_tiles = plan
     _dev(y, weight, out)
     for t, what in ((y, "expert outputs"), (weight, "expert weights"), (out, "feed-forward output")):
         _want(t, torch.float32, what)
     n_tokens, top = weight.shape
+    _dev(own)
+    if own is not None and own.shape != out.shape:
+        raise KernelError("moe_combine: the experts' input differs in shape from the output")
     if y.shape != (n_tokens * top, out.shape[1]) or out.shape[0] != n_tokens:
         raise KernelError("moe_combine: sizes differ")
-    _check("moe", library("moe").rocml_moe_combine(_ptr(y), _ptr(place), _ptr(weight), _ptr(out), n_tokens, top, out.shape[1],
+    _check("moe", library("moe").rocml_moe_combine(_ptr(y), _ptr(place), _ptr(weight), _ptr(own), 0 if own is None else _code(own), _ptr(out), n_tokens, top, out.shape[1],
                                                    1 if accumulate else 0, _stream()))
+
+
+# ---- streams -----------------------------------------------------------------------------
+MAX_STREAMS = 16
+
+
+def stream_links(src: torch.Tensor, n_streams: int, y: Optional[torch.Tensor] = None, mix: Optional[torch.Tensor] = None,
+                 w_out: Optional[torch.Tensor] = None, partials: Optional[torch.Tensor] = None, replace: bool = False,
+                 dst: Optional[torch.Tensor] = None, total: Optional[torch.Tensor] = None, w_in: Optional[torch.Tensor] = None,
+                 gain: Optional[torch.Tensor] = None, eps: float = 0.0, normed: Optional[torch.Tensor] = None) -> None:
+    """What lies between two sublayers of a residual path of ``n_streams`` streams, in one pass (32-bit).  ``src`` is ``[T, S, n]``, or
+    ``[T, n]`` for S equal streams.  With a sublayer's output ``y [T, n]`` (and the K pieces ``partials`` of the product that made it,
+    added in split order; with ``replace`` they are all of it) the streams are formed anew,
+    ``new_t = sum_s mix[s, t] x_s + w_out[t] y``, and stored in ``dst`` (which may be ``src``).  ``total``: their sum, ``[T, n]``.
+    ``normed``: ``rms(sum_t w_in[t] new_t) * gain`` in its own type, what the next sublayer reads."""
+    _dev(src, y, mix, w_out, partials, dst, total, w_in, gain, normed)
+    if not 1 <= n_streams <= MAX_STREAMS:
+        raise KernelError(f"{n_streams} streams; 1 to {MAX_STREAMS} are supported")
+    rows, n = src.shape[0], src.shape[-1]
+    if src.dim() not in (2, 3) or (src.dim() == 3 and src.shape[1] != n_streams):
+        raise KernelError(f"the streams are {tuple(src.shape)}, expected [T, {n_streams}, n] or [T, n]")
+    for t, shape, what in ((src, tuple(src.shape), "streams"), (y, (rows, n), "sublayer output"), (mix, (n_streams, n_streams), "mix"),
+                           (w_out, (n_streams,), "output weights"), (dst, (rows, n_streams, n), "new streams"), (total, (rows, n), "sum of the streams"),
+                           (w_in, (n_streams,), "input weights"), (gain, (n,), "norm gain")):
+        if t is not None and (t.dtype != torch.float32 or tuple(t.shape) != shape):
+            raise KernelError(f"stream_links: {what} must be 32-bit {shape}, got {t.dtype} {tuple(t.shape)}")
+    if normed is not None and tuple(normed.shape) != (rows, n):
+        raise KernelError("stream_links: the next sublayer's input must be [T, n]")
+    n_splits = stride = 0
+    if partials is not None:
+        _want(partials, torch.float32, "partial sums")
+        if partials.dim() != 3 or tuple(partials.shape[1:]) != (rows, n):
+            raise KernelError("stream_links: partial sums must be [splits, T, n]")
+        n_splits, stride = partials.shape[0], rows * n
+    elif replace:
+        raise KernelError("stream_links: nothing to replace the sublayer's output with")
+    _check("streams", library("streams").rocml_stream_links(
+        _ptr(src), 1 if src.dim() == 2 else n_streams, _ptr(y), _ptr(partials), n_splits, stride, 1 if replace else 0, _ptr(mix), _ptr(w_out),
+        _ptr(dst), _ptr(total), _ptr(w_in), _ptr(gain), float(eps), _ptr(normed), 0 if normed is None else _code(normed), rows, n, n_streams,
+        _stream()))
+
+
+# ---- attention with two maps per head ------------------------------------------------------
+def diff_attention_sizes_ok(dtype: torch.dtype, head_dim: int, v_head_dim: int, page: int) -> bool:
+    """Whether the matrix-core kernels take these head sizes (the plain kernel takes any up to 1024)."""
+    return dtype == torch.bfloat16 and bool(library("diff_attention").rocml_diff_attention_sizes_ok(head_dim, v_head_dim, page))
+
+
+def diff_attention_decode_fits(dtype: torch.dtype, n_heads: int, n_kv_heads: int, head_dim: int, v_head_dim: int, page: int) -> bool:
+    """Whether ``diff_attention_decode`` takes a layer."""
+    return diff_attention_sizes_ok(dtype, head_dim, v_head_dim, page) \
+        and n_heads // n_kv_heads <= library("diff_attention").rocml_diff_attention_max_group()
+
+
+def _diff_cache_checks(k_cache, v_cache, n_kv_heads: int, head_dim: int, v_head_dim: int, dtype) -> int:
+    page = k_cache.shape[2]
+    if k_cache.dtype != dtype or k_cache.shape[1:] != (2 * n_kv_heads, page, head_dim) or v_cache.dtype != dtype \
+            or v_cache.shape != (k_cache.shape[0], n_kv_heads, v_head_dim, page):
+        raise KernelError(f"cache {tuple(k_cache.shape)} / {tuple(v_cache.shape)} does not fit two maps of {n_kv_heads} heads of {head_dim} / {v_head_dim}")
+    return page
+
+
+def diff_attention(q: torch.Tensor, out: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
+                   token_seq: torch.Tensor, token_pos: torch.Tensor, n_heads: int, n_kv_heads: int, head_dim: int, v_head_dim: int,
+                   scale: float, map_weight: float, out_scale: float, eps: float, cu_seqlens: torch.Tensor, q_counts: Sequence[int],
+                   window: Optional[int] = None, maps: Optional[torch.Tensor] = None, plain: bool = False, max_len: int = 0) -> None:
+    """Attention with two softmax maps per head over one value head: ``a1 - map_weight * a2`` per head, divided by its root mean square
+    (``eps`` inside the root), times ``out_scale``.  ``q [T, 2 H * dim]`` with the query rows in the order (key/value head, map, head of
+    the group), keys ``[pages, 2 G, page, dim]`` (a head's two maps side by side), values ``[pages, G, v_dim, page]``, all in the compute
+    type and in the cache already; ``out [T, H * v_dim]``.  ``maps``: 32-bit ``[T, 2 H * v_dim]`` for the plain path (``plain``, 32-bit, or sizes the
+    matrix-core kernels refuse).  ``q_counts`` (host): query tokens of each sequence; ``max_len`` is what a profile prices the call with."""
+    _dev(q, out, k_cache, v_cache, block_table, token_seq, token_pos, cu_seqlens, maps)
+    n_tokens = q.shape[0]
+    if q.shape != (n_tokens, 2 * n_heads * head_dim) or out.shape != (n_tokens, n_heads * v_head_dim) or out.dtype != q.dtype:
+        raise KernelError("attention with two maps: queries are [T, 2 * heads * dim], the output [T, heads * value size], of one type")
+    page = _diff_cache_checks(k_cache, v_cache, n_kv_heads, head_dim, v_head_dim, q.dtype)
+    for t, what in ((block_table, "block table"), (token_seq, "token sequence table"), (token_pos, "token position table"),
+                    (cu_seqlens, "sequence offsets")):
+        _want(t, torch.int32, what)
+    n_seqs = cu_seqlens.numel() - 1
+    if token_seq.numel() != n_tokens or token_pos.numel() != n_tokens or len(q_counts) != n_seqs or block_table.shape[0] < n_seqs:
+        raise KernelError("one sequence index and position per token, one count and block table row per sequence are needed")
+    if maps is not None and (maps.dtype != torch.float32 or maps.numel() < n_tokens * 2 * n_heads * v_head_dim):
+        raise KernelError("the maps' outputs need 32-bit room for [T, 2 * heads * value size]")
+    counts = (ctypes.c_int * n_seqs)(*[int(c) for c in q_counts])
+    _check("diff_attention", library("diff_attention").rocml_diff_attention(
+        _ptr(q), _ptr(out), _ptr(k_cache), _ptr(v_cache), _code(q), _ptr(block_table), block_table.shape[1], _ptr(token_seq), _ptr(token_pos),
+        n_tokens, n_heads, n_kv_heads, head_dim, v_head_dim, page, float(scale), 0 if window is None else int(window), float(map_weight),
+        float(out_scale), float(eps), _ptr(cu_seqlens), n_seqs, counts, _ptr(maps), 1 if plain else 0, _stream()))
+
+
+def diff_attention_decode(qkv: torch.Tensor, out: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
+                          token_pos: torch.Tensor, n_heads: int, n_kv_heads: int, head_dim: int, v_head_dim: int, scale: float,
+                          map_weight: float, out_scale: float, eps: float, cos: Optional[torch.Tensor], sin: Optional[torch.Tensor],
+                          window: Optional[int] = None, n_splits: int = 1, workspace: Optional[torch.Tensor] = None, max_len: int = 0) -> None:
+    """A decode step's attention with two maps per head straight from the projection ``qkv`` (32-bit ``[T, ld]`` or its K pieces
+    ``[splits, T, ld]``; rows hold ``2 H`` query heads in the order of ``diff_attention``, ``2 G`` key heads and ``G`` value heads): rotation of
+    the leading values of every q and k head (tables ``[T, rot / 2]``), append of the new keys and value, and attention in one launch.
+    Token ``t`` is the one token of the step's sequence ``t``.  ``workspace`` (for ``n_splits`` above one) must not overlap ``qkv``."""
+    _dev(qkv, out, k_cache, v_cache, block_table, token_pos, cos, sin, workspace)
+    _want(qkv, torch.float32, "projection output")
+    splits, stride = 1, 0
+    if qkv.dim() == 3:
+        splits, stride = qkv.shape[0], qkv.shape[1] * qkv.shape[2]
+        qkv = qkv[0]
+    n_tokens, ld = qkv.shape
+    if out.shape != (n_tokens, n_heads * v_head_dim):
+        raise KernelError("attention with two maps: the output is [T, heads * value size]")
+    page = _diff_cache_checks(k_cache, v_cache, n_kv_heads, head_dim, v_head_dim, out.dtype)
+    if not diff_attention_decode_fits(out.dtype, n_heads, n_kv_heads, head_dim, v_head_dim, page):
+        raise KernelError("the single-token kernel for two maps does not take this layer")
+    rot = 0
+    if cos is not None:
+        _want(cos, torch.float32, "rotation table")
+        rot = 2 * cos.shape[-1]
+        if cos.shape != (n_tokens, rot // 2) or rot > head_dim or sin is None or sin.shape != cos.shape or sin.dtype != cos.dtype:
+            raise KernelError(f"rotation tables must be float32 {(n_tokens, head_dim // 2)} or narrower")
+    _want(block_table, torch.int32, "block table")
+    _want(token_pos, torch.int32, "token position table")
+    if token_pos.numel() != n_tokens or block_table.shape[0] < n_tokens:
+        raise KernelError("one position and one block table row per token are needed")
+    ws_ptr, ws_bytes = (None, 0) if workspace is None else (workspace.data_ptr(), workspace.numel() * workspace.element_size())
+    _check("diff_attention", library("diff_attention").rocml_diff_attention_decode(
+        _ptr(qkv), ld, splits, stride, _ptr(cos), _ptr(sin), rot, _ptr(out), _ptr(k_cache), _ptr(v_cache), _ptr(block_table),
+        block_table.shape[1], _ptr(token_pos), n_tokens, n_heads, n_kv_heads, head_dim, v_head_dim, page, float(scale),
+        0 if window is None else int(window), float(map_weight), float(out_scale), float(eps), int(n_splits), ws_ptr, ws_bytes, _stream()))

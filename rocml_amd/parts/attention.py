@@ -38,6 +38,7 @@ from .residual import stream
 
 class Attention(Mixer):
     adds_only = True
+    kernel_families = ("attention",)
     FUSED_PREFILL_MIN_TOKENS = 1024
     SPAN_STATS_MIN_TOKENS = 64         # from so many tokens on, a kernel of its own forms the factors of a whole-row norm of q and k
 
@@ -124,7 +125,7 @@ class Attention(Mixer):
         self.sinks: Optional[torch.Tensor] = None
         self.conv_w: Optional[torch.Tensor] = None
         if self.conv is not None:
-            self.kernel_families = ("recurrent",)
+            self.kernel_families = ("attention", "recurrent")
 
     def param_specs(self) -> Dict[str, ParamSpec]:
         s = self.spec

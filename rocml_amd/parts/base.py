@@ -58,13 +58,15 @@ class KVCacheRequest:
     ``v_head_dim``: size of a value head when it is not ``head_dim``.  ``chunk``: positions are
     cut into blocks of so many, counted from 0, and no query looks back beyond the start of its
     own block (so earlier blocks' pages can be given back).  ``keep_first``: with a window, the first so
-    many positions stay visible whatever their distance (their pages are kept)."""
+    many positions stay visible whatever their distance (their pages are kept).  ``n_v_heads``: the number of value heads when
+    it is not the key heads' (several key heads share one)."""
     n_kv_heads: int
     head_dim: int
     window: Optional[int] = None
     v_head_dim: Optional[int] = None
     chunk: Optional[int] = None
     keep_first: int = 0
+    n_v_heads: Optional[int] = None
 
 
 @dataclass(frozen=True)
@@ -150,6 +152,13 @@ class NormHint:
 class FullNormHint(NormHint):
     """The same norm, for a consumer that wants the norm's whole output (not an operand that still lacks its rows' scale):
     a kernel that completes the stream may write ``x / sqrt(mean(x^2) + eps) * gain`` in the compute type beside it."""
+
+
+@dataclass(frozen=True)
+class LinkHint(NormHint):
+    """The same norm over a weighted sum of the stream's copies: what the kernel that completes the copies needs to form the
+    next sublayer's input (``weights``: one number per copy)."""
+    weights: torch.Tensor
 
 
 class Norm(Part):

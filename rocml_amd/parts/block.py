@@ -10,6 +10,8 @@
 ``sublayer_norm`` norms a sublayer's output alone: ``x += norm(mixer(x))``, ``x += norm(ffn(x))`` and, if the
 layer has one, ``x += norm(side(x))``; the sublayers read the stream itself.
 
+``linked_streams`` keeps several copies of the stream; see ``LinkedStreamsBlock``.
+
 A block may put a short causal convolution between its first norm and its mixer (``InputConv``).  The rows it keeps
 are state of the block's own, beside what the mixer keeps: the block's cache request is then composite, ``(mixer,
 convolution)``.  A schedule entry that reads another entry's cache line shares the mixer's part and keeps its own
@@ -24,7 +26,7 @@ import torch
 
 from ..config.spec import BlockSpec
 from ..errors import ConfigError
-from .base import BuildContext, CompositeRequest, CompositeView, FullNormHint, ParamSpec, Part
+from .base import BuildContext, CompositeRequest, CompositeView, FullNormHint, LinkHint, ParamSpec, Part
 from .input_conv import InputConv
 from .registry import build_feed_forward, build_mixer, build_norm, register_block
 from .residual import stream
@@ -87,6 +89,7 @@ class PreNormBlock(ConvInput, Part):
         self.ffn = self.children.get("ffn")
         self.graph_safe = all(getattr(c, "graph_safe", True) for c in self.children.values())
         self.prompt_graph_safe = all(getattr(c, "prompt_graph_safe", False) for c in self.children.values())
+        self.kernel_families = tuple(f for c in self.children.values() for f in getattr(c, "kernel_families", ()))
 
     def param_specs(self) -> Dict[str, ParamSpec]:
         return {f"{name}.{p}": spec for name, child in self.children.items()
@@ -475,3 +478,125 @@ class SandwichNormBlock(ConvInput, Part):
 
 
 register_block("sandwich_norm", SandwichNormBlock)
+
+
+class LinkedStreamsBlock(Part):
+    """Hyper-connections: the layer works on ``streams`` copies of the stream.  A sublayer reads ``norm(sum_s in[s] x_s)``; behind
+    it every copy becomes ``sum_s mix[s, t] x_s + branch_scale * out[t] * y``, all from the old copies.  The copies are 32-bit
+    (``[tokens, streams, hidden]``) and live in a buffer from the first layer of a run of such layers to its last.  The sublayer
+    writes its result to a buffer of the block; one kernel then forms all copies anew (taking a product's K pieces in place of
+    the buffer) and, in the same pass over the row, the next sublayer's input: the feed-forward's behind the mixer, the next
+    layer's behind the feed-forward (``entry_hint``).  The run's first layer reads the plain stream as so many equal copies; its
+    last layer, the one that no layer of this kind follows, writes the copies' sum to the stream instead of the copies."""
+    takes_pending = False
+    takes_next_norm = True
+    _OPEN = "linked_streams.open"         # in step.memo: (the copies, the gain whose norm is formed, its output)
+
+    def __init__(self, spec: BlockSpec, ctx: BuildContext):
+        _no_input_conv(spec)
+        if not 1 <= spec.streams <= ops.MAX_STREAMS:
+            raise ConfigError(f"{spec.streams} copies of the stream; 1 to {ops.MAX_STREAMS} are supported")
+        self.dtype = ctx.dtype
+        self.hidden = spec.mixer_norm.size
+        self.streams = spec.streams
+        self.branch_scale = float(spec.branch_scale)
+        self.children = {"mixer_norm": build_norm(spec.mixer_norm, ctx),
+                         "mixer": build_mixer(spec.mixer, ctx)}
+        if spec.ffn is not None:
+            self.children["ffn_norm"] = build_norm(spec.ffn_norm, ctx)
+            self.children["ffn"] = build_feed_forward(spec.ffn, ctx)
+        self.mixer = self.children["mixer"]
+        self.ffn = self.children.get("ffn")
+        for name in ("mixer_norm", "ffn_norm"):
+            norm = self.children.get(name)
+            if norm is not None and (not hasattr(norm, "gain") or not hasattr(norm, "eps") or getattr(norm, "centred", False)):
+                raise ConfigError("a block with copies of the stream needs root-mean-square norms before its sublayers")
+        self.graph_safe = all(getattr(c, "graph_safe", True) for c in self.children.values())
+        self.prompt_graph_safe = all(getattr(c, "prompt_graph_safe", False) for c in self.children.values())
+        self.kernel_families = ("streams",) + tuple(f for c in self.children.values() for f in getattr(c, "kernel_families", ()))
+        self.links: Dict[str, tuple] = {}        # sublayer -> (in, mix, branch_scale * out)
+
+    def param_specs(self) -> Dict[str, ParamSpec]:
+        specs = PreNormBlock.param_specs(self)
+        s = self.streams
+        for name in ("mixer", "ffn"):
+            if name in self.children:
+                specs[f"{name}_link.in"] = ParamSpec((s,), role="gain", init="gain")
+                specs[f"{name}_link.out"] = ParamSpec((s,), role="gain", init="gain")
+                specs[f"{name}_link.mix"] = ParamSpec((s, s), role="gain", init="normal")
+        return specs
+
+    def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
+        PreNormBlock.bind(self, tensors)
+        for name in ("mixer", "ffn"):
+            if name in self.children:
+                link = name + "_link."
+                self.links[name] = (tensors[link + "in"], tensors[link + "mix"], (tensors[link + "out"] * self.branch_scale).contiguous())
+
+    cache_request = PreNormBlock.cache_request
+    input_conv = None
+    flops = PreNormBlock.flops
+
+    def activation_bytes(self, n_tokens: int) -> int:
+        size = 2 if self.dtype == torch.bfloat16 else 4
+        return n_tokens * self.hidden * (size + 4 + 4 * self.streams) + self.mixer.activation_bytes(n_tokens) + \
+            (self.ffn.activation_bytes(n_tokens) if self.ffn is not None else 0)
+
+    def entry_hint(self, step):
+        return self._hint("mixer")
+
+    def _hint(self, name: str) -> LinkHint:
+        norm = self.children[name + "_norm"]
+        return LinkHint(norm.gain, float(norm.eps), self.hidden, self.links[name][0])
+
+    def _read(self, step, x, hint: LinkHint):
+        """``(source of the copies, the first sublayer's input)``: prepared by the layer before, or formed here at the start of
+        a run."""
+        found = step.memo.pop(self._OPEN, None)
+        if found is not None:
+            copies, gain, xn = found
+            if copies.shape[1] != self.streams or gain != hint.gain.data_ptr():
+                raise ConfigError("layers with copies of the stream that follow each other keep the same number of copies")
+            return copies, xn
+        xn = step.workspace.get("block.xn", tuple(x.shape), self.dtype)
+        ops.stream_links(x, self.streams, w_in=hint.weights, gain=hint.gain, eps=hint.eps, normed=xn)
+        return x, xn
+
+    def _update(self, step, x, source, y, name: str, following):
+        """The copies behind a sublayer and the input of what reads them next (``following``, a ``LinkHint``), or their sum."""
+        ws = step.workspace
+        _, mix, w_out = self.links[name]
+        # (a product cut along K may have left its pieces for this kernel to add: all of y, or what y still lacks)
+        pending = ws.take_pending_or_whole(y)
+        partials, replace = pending if pending is not None else (None, False)
+        if following is None:
+            ops.stream_links(source, self.streams, y=y, mix=mix, w_out=w_out, partials=partials, replace=replace, total=x)
+            return None, None
+        copies = ws.get("block.streams", (x.shape[0], self.streams, self.hidden), torch.float32)
+        xn = ws.get("block.xn", tuple(x.shape), self.dtype)        # (the sublayer is done with its operand)
+        ops.stream_links(source, self.streams, y=y, mix=mix, w_out=w_out, partials=partials, replace=replace, dst=copies,
+                         w_in=following.weights, gain=following.gain, eps=following.eps, normed=xn)
+        return copies, xn
+
+    def forward(self, step, x: torch.Tensor, cache, owns_cache: bool, next_norm=None) -> None:
+        ws = step.workspace
+        rs = stream(step)
+        ws.flush_pending()
+        rs.row_scale = rs.next_norm = None
+        following = next_norm if isinstance(next_norm, LinkHint) else None
+        try:
+            source, xn = self._read(step, x, self._hint("mixer"))
+            y = ws.get("block.sublayer", tuple(x.shape), torch.float32)
+            rs.overwrite = rs.defer_overwrite = True
+            self.mixer.forward(step, xn, y, cache, owns_cache)
+            copies, xn = self._update(step, x, source, y, "mixer", following if self.ffn is None else self._hint("ffn"))
+            if self.ffn is not None:
+                self.ffn.forward(step, xn, y)
+                copies, xn = self._update(step, x, copies, y, "ffn", following)
+            if following is not None:
+                step.memo[self._OPEN] = (copies, following.gain.data_ptr(), xn)
+        finally:
+            rs.overwrite = rs.defer_overwrite = False
+
+
+register_block("linked_streams", LinkedStreamsBlock)

@@ -2,7 +2,7 @@
 the output matrix (rocml/src/forward/chunk_forward.rs:170-184 does both for the last row only).
 A tied output matrix is the embedding's table itself, one buffer
 (rocml/src/weights/mod.rs:48-62 loads it twice).  With a soft cap the logits ``z`` become
-``cap * tanh(z / cap)``."""
+``cap * tanh(z / cap)``.  A factor on the logits is folded into the norm's gain (and bias), in 32-bit."""
 from __future__ import annotations
 
 from typing import Dict, Optional
@@ -26,6 +26,7 @@ class NormLinearHead(Head):
         self.softcap = getattr(spec, "softcap", None)
         if self.softcap is not None and not self.softcap > 0:
             raise ConfigError(f"the soft cap of the logits must be positive, got {self.softcap}")
+        self.scale = float(getattr(spec, "scale", 1.0))
         self.dtype = ctx.dtype
         self.norm = build_norm(spec.norm, ctx)
         self.matrix: Optional[torch.Tensor] = None
@@ -41,6 +42,12 @@ class NormLinearHead(Head):
     def bind(self, tensors: Dict[str, torch.Tensor], shared: Optional[torch.Tensor] = None) -> None:
         prefix = "final_norm."
         self.norm.bind({k[len(prefix):]: v for k, v in tensors.items() if k.startswith(prefix)})
+        if self.scale != 1.0:
+            if getattr(self.norm, "gain", None) is None:
+                raise ConfigError("a factor on the logits needs a norm with a gain before the output matrix")
+            self.norm.gain = self.norm.gain * self.scale
+            if getattr(self.norm, "bias", None) is not None:
+                self.norm.bias = self.norm.bias * self.scale
         if self.tied:
             if shared is None or tuple(shared.shape) != (self.vocab, self.hidden):
                 raise ConfigError("a tied output matrix needs an embedding with a [vocab, hidden] table")

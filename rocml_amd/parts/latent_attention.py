@@ -44,6 +44,7 @@ from .residual import stream
 
 class LatentAttention(Mixer):
     adds_only = True
+    kernel_families = ("attention",)
     # A prompt step of at least so many tokens expands keys and values per head for the positions its
     # queries see and runs the attention kernels for separate heads: a (query, key) pair then costs
     # 2 (head_dim + rot_dim) + 2 v_head_dim operations instead of 2 (kv_rank + rot_dim) + 2 kv_rank.
