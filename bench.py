@@ -2,7 +2,7 @@
 """Decode and prefill speed of the Qwen3 shapes with random bfloat16 weights on one MI355X.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--model qwen3-8b|qwen3-14b|qwen3-32b]
-    python bench.py --design dokulix|felovik|sogavik|roravik|kakalorn [--design-size 2b|8b|14b] [--layers N]
+    python bench.py --design dokulix|felovik|sogavik|roravik|kakalorn|nazulorn [--design-size 2b|8b|14b] [--layers N]
 
 The default run is the Qwen3-8B shape.  A step is one decode step of a batch of 8 sequences,
 each with a 2,048-token random prompt in the cache (context length 4,096): the engine's step
@@ -43,6 +43,10 @@ another's rows, windowed attention whose values are its keys, with kept first po
 forget gate writes, in turn; a convolution on every mixer's input, a norm before and after every sublayer, squared-rectifier
 feed-forwards) beside the two closest designs at equal size: Dokulix (latent attention, biased attention with a sink, dense
 feed-forwards) and Roravik (a recurrence with a decay, norms before and after every sublayer).
+``--design nazulorn`` measures a Nazulorn model (windowed attention with two maps per head and gated linear attention in
+turn, four copies of the stream, routed experts of which some are identities with a shared expert in every layer) beside Roravik
+(routed experts with a shared expert, a windowed attention, recurrences with a decay) and Kakalorn (a windowed attention, a
+recurrence with a decay per token and channel).
 
 The workloads follow the reference's bench (rocml-cli/src/cmd_bench.rs:79-243): synthetic
 prompts, greedy, no stop token, warm-up first; times are taken around synchronised steps.
@@ -89,7 +93,8 @@ def felovik_config(z: dict, n_layers: int):
 
 
 # the closest models each design is measured beside
-COMPANIONS = {"dokulix": ("qwen3",), "felovik": ("qwen3",), "sogavik": ("felovik",), "roravik": ("felovik",), "kakalorn": ("dokulix", "roravik")}
+COMPANIONS = {"dokulix": ("qwen3",), "felovik": ("qwen3",), "sogavik": ("felovik",), "roravik": ("felovik",), "kakalorn": ("dokulix", "roravik"),
+              "nazulorn": ("roravik", "kakalorn")}
 
 
 def design_configs(size: dict, n_layers: int, design: str = "dokulix"):
@@ -101,6 +106,13 @@ def design_configs(size: dict, n_layers: int, design: str = "dokulix"):
         mine = kakalorn_config(z["vocab"], z["width"], z["heads"], z["kv_heads"], z["dim"], z["window"], 4, z["heads"], z["dim"],
                                z["rot_dim"], z["q_rank"], z["kv_rank"], z["width"] // 128, 128, z["ff"], n_layers)
         return mine, design_configs(z, n_layers, "dokulix")[0], design_configs(z, n_layers, "roravik")[0]
+    if design == "nazulorn":
+        from rocml_amd.config.catalog import nazulorn_config
+        # the companions' projection sizes: as many heads, each with two maps of half the size over values of the whole size; recurrence
+        # heads of 64 x 128 with an inner width equal to the model's; experts and shared expert as Roravik's
+        mine = nazulorn_config(z["vocab"], z["width"], z["heads"], z["kv_heads"], z["dim"] // 2, z["dim"], z["window"], z["width"] // 128, 64, 128,
+                               32, 2, 4, z["ff"] // 4, z["ff"] // 2, n_layers)
+        return mine, design_configs(z, n_layers, "roravik")[0], design_configs(z, n_layers, "kakalorn")[0]
     if design == "sogavik":
         from rocml_amd.config.catalog import sogavik_config
         return (sogavik_config(z["vocab"], z["width"], z["heads"], z["kv_heads"], z["dim"], z["window"], z["width"] // 128, 128,

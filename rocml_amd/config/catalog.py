@@ -222,6 +222,35 @@ CATALOG += [
     ModelEntry("kakalorn-2b", kakalorn_config(32768, 2048, 16, 8, 128, 1024, 4, 16, 128, 64, 768, 512, 16, 128, 6144, 24)),
 ]
 
+
+
+def nazulorn_config(vocab, width, heads, kv_heads, dim, vdim, window, rec_heads, rec_dim, rec_vdim, experts, identity, top, expert_ff,
+                    shared_ff, n_layers, streams=4, decay_rank=16, factor=4.0, original=4096, max_positions=None):
+    """A Nazulorn configuration: windowed attention with two maps per head and gated linear attention in turn, routed experts
+    (some of them identities) with a shared expert in every layer, ``streams`` copies of the stream."""
+    rot = {"base": 10000.0, "dims": dim, "scaling": {"factor": factor, "original": original, "fast": 32.0, "slow": 1.0}}
+    attention = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5, "diff": 0.8, "mask": {"size": window},
+                 "rot": rot}
+    recurrence = {"heads": rec_heads, "dim": rec_dim, "vdim": rec_vdim, "tau": 8.0, "decay_rank": decay_rank}
+    mlp = {"kind": "moe", "expert": {"ff": expert_ff, "limit": 7.0}, "shared": {"ff": shared_ff, "limit": 10.0},
+           "router": {"experts": experts, "identity": identity, "top": top, "scale": 2.5}}
+    layers = [{"type": "attention", "mixer": attention, "mlp": mlp} if i % 2 == 0 else {"type": "gla", "mixer": recurrence, "mlp": mlp}
+              for i in range(n_layers)]
+    cfg = {"architecture": "Nazulorn", "vocab": vocab, "width": width, "streams": streams, "norm": {"eps": 1e-6}, "embedding": {"scale": 2.0},
+           "residual_mult": 0.25, "logit_scale": 0.125, "layers": layers}
+    if max_positions is not None:
+        cfg["max_positions"] = max_positions
+    return cfg
+
+
+# The seventh architecture: a test-sized model and the layer sizes of a 2B-class model (random weights; no
+# checkpoint of this design exists).
+CATALOG += [
+    ModelEntry("nazulorn-tiny", nazulorn_config(352, 96, 4, 2, 16, 40, 40, 3, 16, 32, 6, 2, 2, 48, 64, 4, streams=2, decay_rank=8),
+               default_ctx=512, init_norm_jitter=True),
+    ModelEntry("nazulorn-2b", nazulorn_config(32768, 2048, 16, 8, 64, 128, 1024, 16, 64, 128, 32, 2, 4, 1536, 3072, 24)),
+]
+
 _BY_NAME = {e.name: e for e in CATALOG}
 
 

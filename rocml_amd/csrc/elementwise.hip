@@ -581,6 +581,46 @@ qk_norm_rope_rows_kernel(
     }
 }
 
+// Prompts: q and k rows without a norm (nor a stretch or biases), in 16-byte pieces, whatever the head size: a thread takes
+// four neighbouring pairs (e, e + rot/2) of a row, or four values beyond the rotated part.  d and rot are multiples of 8.
+template <typename TO>
+__global__ void __launch_bounds__(EW_BLOCK)
+rope_rows_vec_kernel(const float* __restrict__ qkv, int ld, int hq, int hkv, int d, const float* __restrict__ cos_t,
+                     const float* __restrict__ sin_t, int rot, TO* __restrict__ q_out, TO* __restrict__ kcache,
+                     const int* __restrict__ block_table, int bt_width, const int* __restrict__ token_seq,
+                     const int* __restrict__ token_pos, int page_size, int rows_per_token, int first_row, long long total) {
+    long long idx = (long long)blockIdx.x * EW_BLOCK + threadIdx.x;
+    if (idx >= total) return;
+    const int half = rot / 2, pair_units = rot / 8, units = pair_units + (d - rot) / 4;
+    long long row = idx / units;
+    int unit = (int)(idx - row * units);
+    int t = (int)(row / rows_per_token), r = first_row + (int)(row - (long long)t * rows_per_token);
+    bool pairs = unit < pair_units;
+    int e = pairs ? unit * 4 : rot + (unit - pair_units) * 4;
+    const float* src = qkv + (size_t)t * ld + (size_t)r * d + e;
+    float4 lo = *(const float4*)src, hi = lo, c = lo, s = lo;
+    if (pairs) {
+        hi = *(const float4*)(src + half);
+        c = *(const float4*)(cos_t + (size_t)t * half + e);
+        s = *(const float4*)(sin_t + (size_t)t * half + e);
+    }
+    TO* dst;
+    if (r < hq) {
+        dst = q_out + ((size_t)t * hq + r) * d + e;
+    } else {
+        int pos = token_pos[t];
+        int page = block_table[(size_t)token_seq[t] * bt_width + pos / page_size];
+        if (page < 0) return;
+        dst = kcache + (((size_t)page * hkv + (r - hq)) * page_size + pos % page_size) * d + e;
+    }
+    if (!pairs) {
+        store4(dst, lo.x, lo.y, lo.z, lo.w);
+        return;
+    }
+    store4(dst, lo.x * c.x - hi.x * s.x, lo.y * c.y - hi.y * s.y, lo.z * c.z - hi.z * s.z, lo.w * c.w - hi.w * s.w);
+    store4(dst + half, lo.x * s.x + hi.x * c.x, lo.y * s.y + hi.y * c.y, lo.z * s.z + hi.z * c.z, lo.w * s.w + hi.w * c.w);
+}
+
 // Values of many tokens at once (prompts): a block takes 64 consecutive tokens of the packed
 // batch, one key/value head and 32 of its values, stages them in LDS and writes them transposed.
 // In the transposed page a token is one 2- or 4-byte column; written token by token every store
@@ -679,6 +719,13 @@ ROCML_EXPORT int rocml_qk_norm_rope_append(
     // many rows, none of them values: several rows per wave
     bool many_rows = local_pair && per_lane <= 4 && n_splits == 1 && n_tokens >= VT_TOKENS && (v_tiled || !write_kv) && !span_self;
     constexpr int MANY = 4;
+    // the same for rows without a norm, of any size that is a multiple of 8
+    uintptr_t aligned = (uintptr_t)qkv | (uintptr_t)q_out | (uintptr_t)kcache | (uintptr_t)cos_t | (uintptr_t)sin_t;
+    bool plain_rows = in_dtype == ROCML_F32 && !many_rows && !q_gain && !k_gain && !bias && qt_every == 0 && n_splits == 1 &&
+                      n_tokens >= VT_TOKENS && (v_tiled || !write_kv) && d % 8 == 0 && rot % 8 == 0 && pairing == 0 && ld % 4 == 0 &&
+                      (aligned & 15) == 0;
+    long long pieces = (long long)n_tokens * rows_per_token * (cos_t ? rot / 8 + (d - rot) / 4 : d / 4);
+    plain_rows = plain_rows && pieces < (1ll << 31) * EW_BLOCK;
     int grid = many_rows ? ceil_div(rows, QK_WAVES * MANY) : ceil_div(rows, QK_WAVES);
     size_t lds = local_pair ? 0 : (size_t)QK_WAVES * d * sizeof(float);
 #define LAUNCH_N(TI, TO, N, LP)                                                                 \
@@ -693,7 +740,11 @@ ROCML_EXPORT int rocml_qk_norm_rope_append(
         token_pos, page_size, rows_per_token, first_row, bias, qt_coef, qt_every, span_inv)
 #define LAUNCH(TI, TO)                                                                          \
     {                                                                                           \
-        if (many_rows) { if (per_lane == 2) LAUNCH_ROWS(TI, TO, 2); else LAUNCH_ROWS(TI, TO, 4); } \
+        if (plain_rows) {                                                                       \
+            rope_rows_vec_kernel<TO><<<ceil_div(pieces, EW_BLOCK), EW_BLOCK, 0, stream>>>(      \
+                (const float*)qkv, ld, hq, hkv, d, cos_t, sin_t, cos_t ? rot : 0, (TO*)q_out, (TO*)kcache, block_table, bt_width, \
+                token_seq, token_pos, page_size, rows_per_token, first_row, pieces);            \
+        } else if (many_rows) { if (per_lane == 2) LAUNCH_ROWS(TI, TO, 2); else LAUNCH_ROWS(TI, TO, 4); } \
         else if (per_lane == 1) LAUNCH_N(TI, TO, 1, false);                                     \
         else if (per_lane == 2) { if (local_pair) LAUNCH_N(TI, TO, 2, true); else LAUNCH_N(TI, TO, 2, false); } \
         else if (per_lane == 4) { if (local_pair) LAUNCH_N(TI, TO, 4, true); else LAUNCH_N(TI, TO, 4, false); } \

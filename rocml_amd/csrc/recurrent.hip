@@ -1607,9 +1607,11 @@ low_rank_decay_kernel(const float* __restrict__ low, int ldl, int low_col0, cons
     for (int j = 0; j < TB; ++j) {
         if (t0 + j >= n_tokens) continue;
         float v = z[j] + b;
-        // log sigmoid(v) = min(v, 0) - log(1 + e^-|v|)
-        float logs = fminf(v, 0.f) - log1pf(expf(-fabsf(v)));
-        decay[(size_t)(t0 + j) * n + c] = expf(logs * inv_tau);
+        // log2 sigmoid(v) = min(v, 0) log2(e) - log2(1 + e^-|v|), by hardware exponentials and logarithm: where e^-|v| is
+        // next to nothing against 1, what its sum rounds off is below the decay's own rounding next to 1
+        float logs = fminf(v, 0.f) * 1.4426950408889634f
+                     - __builtin_amdgcn_logf(1.0f + __builtin_amdgcn_exp2f(-fabsf(v) * 1.4426950408889634f));
+        decay[(size_t)(t0 + j) * n + c] = __builtin_amdgcn_exp2f(logs * inv_tau);
     }
 }
 

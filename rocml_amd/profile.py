@@ -66,6 +66,26 @@ def _attention_cost(q, out, k_cache, v_cache, block_table, token_seq, token_pos,
     return _nbytes(q, out) + kv, 2 * n_heads * (head_dim + dv) * n_tokens * keys_per_query
 
 
+def _diff_attention_cost(q, out, k_cache, v_cache, block_table, token_seq, token_pos, n_heads, n_kv_heads, head_dim, v_head_dim,
+                         *a, **kw) -> Tuple[int, int]:
+    n_tokens, n_seqs = q.shape[0], block_table.shape[0]
+    counts = a[5] if len(a) > 5 else kw["q_counts"]
+    max_new, max_len, window = max(counts), kw.get("max_len", 0), kw.get("window")
+    keys_per_query, read_len = max(1, max_len - max_new // 2), max_len
+    if window:
+        keys_per_query, read_len = min(keys_per_query, window), min(max_len, max_new + window)
+    kv = n_seqs * read_len * n_kv_heads * (2 * head_dim + v_head_dim) * k_cache.element_size()
+    return _nbytes(q, out) + kv, 4 * n_heads * (head_dim + v_head_dim) * n_tokens * keys_per_query
+
+
+def _diff_decode_cost(qkv, out, k_cache, v_cache, block_table, token_pos, n_heads, n_kv_heads, head_dim, v_head_dim, *a, **kw) -> Tuple[int, int]:
+    n_seqs, seen = out.shape[0], kw.get("max_len", 0)
+    if kw.get("window"):
+        seen = min(seen, kw["window"])
+    kv = n_seqs * seen * n_kv_heads * (2 * head_dim + v_head_dim) * k_cache.element_size()
+    return _nbytes(qkv, out) + kv, 4 * n_heads * (head_dim + v_head_dim) * n_seqs * seen
+
+
 def _gemm_batched_cost(x, x_head_stride, w, out, out_head_stride, **kw) -> Tuple[int, int]:
     heads, n, k = w.shape
     rows = x.shape[0]
@@ -168,7 +188,14 @@ _COSTS: Dict[str, Tuple[str, Callable]] = {
         min(w.shape[0], out.shape[0]) * w.shape[1] * w.shape[2] * w.element_size() * (2 if w2 is not None else 1)
         + out.shape[0] * (w.shape[2] * a.element_size() + w.shape[1] * out.element_size()),
         2 * out.shape[0] * w.shape[1] * w.shape[2] * (2 if w2 is not None else 1))),
-    "moe_combine": ("weighted sum of experts", lambda y, plan, weight, out, **kw: (_nbytes(y, out), 2 * y.numel())),
+    "moe_combine": ("weighted sum of experts", lambda y, plan, weight, out, **kw: (_nbytes(y, out, kw.get("own")), 2 * y.numel())),
+    "stream_links": ("copies of the stream and the next norm", lambda src, n_streams, y=None, partials=None, replace=False, dst=None, total=None,
+                     normed=None, **kw: (_nbytes(src, partials, dst, total, normed) + (0 if replace else _nbytes(y)),
+                                         2 * (n_streams + 2) * n_streams * src.shape[0] * src.shape[-1])),
+    "diff_attention": ("attention (two maps)", _diff_attention_cost),
+    "diff_attention_decode": ("attention (two maps, rotation, append)", _diff_decode_cost),
+    "low_rank_decay": ("decays from a low-rank product", lambda low, c0, w, bias, tau, out: (
+        out.shape[0] * w.shape[0] * 4 + _nbytes(w, bias, out), 2 * out.numel() * w.shape[0], PEAK_FLOPS[torch.float32])),
     "decay_scan": ("recurrence with a decay per channel (32-bit vector work)",
                    lambda q, q0, k, k0, v, v0, state, cu, slots, out, n_heads, head_dim, v_head_dim, **kw: (
                        out.shape[0] * n_heads * ((3 if kw.get("decay") is not None else 2) * head_dim + v_head_dim) * 4 + _nbytes(out)

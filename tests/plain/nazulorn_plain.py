@@ -71,8 +71,10 @@ def frequencies(rot: Dict) -> Tuple[List[float], float]:
     return out, 0.1 * math.log(sc["factor"]) + 1.0
 
 
-def rotate(x: torch.Tensor, rot: Dict) -> torch.Tensor:
+def rotate(x: torch.Tensor, rot: Optional[Dict]) -> torch.Tensor:
     """``x [T, heads, d]``: the first ``dims`` numbers of every head turn in pairs ``(i, i + dims/2)``; the rest stays."""
+    if rot is None:
+        return x
     n = rot["dims"]
     f, factor = frequencies(rot)
     angle = torch.arange(x.shape[0], dtype=torch.float64)[:, None] * torch.tensor(f, dtype=torch.float64)[None, :]
@@ -109,10 +111,10 @@ def combine_maps(a1: torch.Tensor, a2: torch.Tensor, weight, diff: float, eps: f
 
 def differential_attention(h: torch.Tensor, p: Dict[str, torch.Tensor], m: Dict, eps: float) -> torch.Tensor:
     T, H, G, d, dv = h.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
-    q = rotate((h @ p["q"].T).view(T, H * 2, d), m["rot"]).view(T, H, 2, d)
-    k = rotate((h @ p["k"].T).view(T, G * 2, d), m["rot"]).view(T, G, 2, d)
+    q = rotate((h @ p["q"].T).view(T, H * 2, d), m.get("rot")).view(T, H, 2, d)
+    k = rotate((h @ p["k"].T).view(T, G * 2, d), m.get("rot")).view(T, G, 2, d)
     v = (h @ p["v"].T).view(T, G, dv)
-    seen = window_seen(T, m["mask"]["size"])
+    seen = window_seen(T, m["mask"]["size"] if m.get("mask") is not None else T)
     weight = map_weight(p, m["diff"])
     out = []
     for a in range(H):
@@ -151,9 +153,10 @@ def gated_linear_attention(h: torch.Tensor, p: Dict[str, torch.Tensor], m: Dict,
 
 
 # ---- experts -------------------------------------------------------------------------------
-def expert(h: torch.Tensor, gate: torch.Tensor, up: torch.Tensor, down: torch.Tensor, limit: float) -> torch.Tensor:
-    g = torch.clamp(h @ gate.T, max=limit)
-    u = torch.clamp(h @ up.T, min=-limit, max=limit)
+def expert(h: torch.Tensor, gate: torch.Tensor, up: torch.Tensor, down: torch.Tensor, limit: Optional[float]) -> torch.Tensor:
+    g, u = h @ gate.T, h @ up.T
+    if limit is not None:
+        g, u = torch.clamp(g, max=limit), torch.clamp(u, min=-limit, max=limit)
     return (g * torch.sigmoid(1.702 * g) * (u + 1.0)) @ down.T
 
 
@@ -168,7 +171,7 @@ def choose_experts(logits: torch.Tensor, correction: torch.Tensor, top: int, sca
 
 def experts(h: torch.Tensor, p: Dict[str, torch.Tensor], m: Dict) -> torch.Tensor:
     r = m["router"]
-    chosen, w = choose_experts(h @ p["router"].T, p["correction"], r["top"], r["scale"])
+    chosen, w = choose_experts(h @ p["router"].T, p["correction"], r["top"], 1.0 if r.get("scale") is None else r["scale"])
     y = torch.zeros_like(h)
     for t in range(h.shape[0]):
         for c in range(r["top"]):
