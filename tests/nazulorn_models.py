@@ -95,7 +95,8 @@ CFG_E = config(160, 64, 3, 1.2, 0.6, 0.8, [
     gla(2, 200, 24, 4.0, 70, moe(9, 3, 6, 16, 1.3, 1.0, (16, 1.0))),
 ])
 
-CONFIGS = {"A": (CFG_A, 61), "B": (CFG_B, 62), "C": (CFG_C, 63), "D": (CFG_D, 64), "E": (CFG_E, 65)}
+# (C's seed: no choice between its one expert and the identity is close for the tests' requests, which attention would spread)
+CONFIGS = {"A": (CFG_A, 61), "B": (CFG_B, 62), "C": (CFG_C, 98), "D": (CFG_D, 64), "E": (CFG_E, 65)}
 
 
 def written(cfg: Dict) -> Dict:
