@@ -1570,48 +1570,68 @@ ROCML_EXPORT int rocml_decay_scan(const float* q, int ldq, int q_col0, const flo
 // ---- decays from a low-rank product --------------------------------------------------------
 // decay[t, c] = sigmoid(z)^(1 / tau) with z = bias[c] + sum_r w[r, c] * low[t, r]: the second of two small matrices, the
 // sigmoid and the root in one pass, all 32-bit.  low is `rank` columns (from low_col0 on) of rows of ldl 32-bit numbers, w is
-// [rank, n] (neighbouring channels side by side).  A block takes 256 channels and LD_TOKENS tokens, whose rows of `low` lie in LDS.
-constexpr int LD_TOKENS = 8;
+// [rank, n] (neighbouring channels side by side).  A block takes 256 CPT channels and TB tokens, whose rows of `low` lie in LDS with
+// the tokens side by side: a read of four of them serves CPT channels of a thread.
+constexpr int LD_TOKENS = 8, LD_CHANNELS = 2;
 constexpr int LD_RANK = 64;      // numbers of a token's row in LDS at a time
 
-template <typename TW, int TB>
+template <typename TW, int TB, int CPT>
 __global__ void __launch_bounds__(RC_BLOCK)
 low_rank_decay_kernel(const float* __restrict__ low, int ldl, int low_col0, const TW* __restrict__ w, const float* __restrict__ bias,
                       float inv_tau, float* __restrict__ decay, int n_tokens, int n, int rank) {
-    __shared__ float rows[TB][LD_RANK];
-    int c = blockIdx.x * RC_BLOCK + threadIdx.x;
+    __shared__ __attribute__((aligned(16))) float rows[LD_RANK][TB];
+    int c0 = blockIdx.x * RC_BLOCK * CPT + threadIdx.x;
     int t0 = blockIdx.y * TB;
-    float z[TB];
+    float z[CPT][TB];
 #pragma unroll
-    for (int j = 0; j < TB; ++j) z[j] = 0.f;
+    for (int p = 0; p < CPT; ++p)
+#pragma unroll
+        for (int j = 0; j < TB; ++j) z[p][j] = 0.f;
     for (int r0 = 0; r0 < rank; r0 += LD_RANK) {
         int here = min(LD_RANK, rank - r0);
         if (r0 > 0) __syncthreads();
         for (int i = threadIdx.x; i < TB * here; i += RC_BLOCK) {
             int j = i / here, r = i - j * here;
-            rows[j][r] = t0 + j < n_tokens ? low[(size_t)(t0 + j) * ldl + low_col0 + r0 + r] : 0.f;
+            rows[r][j] = t0 + j < n_tokens ? low[(size_t)(t0 + j) * ldl + low_col0 + r0 + r] : 0.f;
         }
         __syncthreads();
-        if (c < n) {
-#pragma unroll 8
-            for (int r = 0; r < here; ++r) {
-                float wv = Elem<TW>::load(w + (size_t)(r0 + r) * n + c);
+#pragma unroll 4
+        for (int r = 0; r < here; ++r) {
+            float wv[CPT];
 #pragma unroll
-                for (int j = 0; j < TB; ++j) z[j] = fmaf(wv, rows[j][r], z[j]);
+            for (int p = 0; p < CPT; ++p) wv[p] = Elem<TW>::load(w + (size_t)(r0 + r) * n + min(c0 + p * RC_BLOCK, n - 1));
+            float tok[TB];
+            if constexpr (TB % 4 == 0) {
+#pragma unroll
+                for (int j = 0; j < TB; j += 4) {
+                    float4 v = *(const float4*)&rows[r][j];
+                    tok[j] = v.x; tok[j + 1] = v.y; tok[j + 2] = v.z; tok[j + 3] = v.w;
+                }
+            } else {
+#pragma unroll
+                for (int j = 0; j < TB; ++j) tok[j] = rows[r][j];
             }
+#pragma unroll
+            for (int p = 0; p < CPT; ++p)
+#pragma unroll
+                for (int j = 0; j < TB; ++j) z[p][j] = fmaf(wv[p], tok[j], z[p][j]);
         }
     }
-    if (c >= n) return;
-    float b = bias ? bias[c] : 0.f;
 #pragma unroll
-    for (int j = 0; j < TB; ++j) {
-        if (t0 + j >= n_tokens) continue;
-        float v = z[j] + b;
-        // log2 sigmoid(v) = min(v, 0) log2(e) - log2(1 + e^-|v|), by hardware exponentials and logarithm: where e^-|v| is
-        // next to nothing against 1, what its sum rounds off is below the decay's own rounding next to 1
-        float logs = fminf(v, 0.f) * 1.4426950408889634f
-                     - __builtin_amdgcn_logf(1.0f + __builtin_amdgcn_exp2f(-fabsf(v) * 1.4426950408889634f));
-        decay[(size_t)(t0 + j) * n + c] = __builtin_amdgcn_exp2f(logs * inv_tau);
+    for (int p = 0; p < CPT; ++p) {
+        int c = c0 + p * RC_BLOCK;
+        if (c >= n) continue;
+        float b = bias ? bias[c] : 0.f;
+#pragma unroll
+        for (int j = 0; j < TB; ++j) {
+            if (t0 + j >= n_tokens) continue;
+            float v = z[p][j] + b;
+            // log2 sigmoid(v) = min(v, 0) log2(e) - log2(1 + e^-|v|), by hardware exponentials and logarithm: where e^-|v| is
+            // next to nothing against 1, what its sum rounds off is below the decay's own rounding next to 1
+            float logs = fminf(v, 0.f) * 1.4426950408889634f
+                         - __builtin_amdgcn_logf(1.0f + __builtin_amdgcn_exp2f(-fabsf(v) * 1.4426950408889634f));
+            decay[(size_t)(t0 + j) * n + c] = __builtin_amdgcn_exp2f(logs * inv_tau);
+        }
     }
 }
 
@@ -1624,11 +1644,11 @@ ROCML_EXPORT int rocml_low_rank_decay(const float* low, int ldl, int low_col0, c
     ROCML_REQUIRE(n_tokens <= 65535 * LD_TOKENS, "low_rank_decay: %d tokens are too many", n_tokens);
     // few tokens: one a block, so that their channels spread over the chip
     bool few = n_tokens <= 64;
-    dim3 grid(ceil_div(n, RC_BLOCK), few ? n_tokens : ceil_div(n_tokens, LD_TOKENS));
+    dim3 grid(ceil_div(n, few ? RC_BLOCK : RC_BLOCK * LD_CHANNELS), few ? n_tokens : ceil_div(n_tokens, LD_TOKENS));
     float inv = 1.0f / tau;
-#define LRD(TW_, TB_) low_rank_decay_kernel<TW_, TB_><<<grid, RC_BLOCK, 0, stream>>>(low, ldl, low_col0, (const TW_*)w, bias, inv, decay, n_tokens, n, rank)
-    if (w_dtype == ROCML_BF16) { if (few) LRD(bf16_t, 1); else LRD(bf16_t, LD_TOKENS); }
-    else { if (few) LRD(float, 1); else LRD(float, LD_TOKENS); }
+#define LRD(TW_, TB_, CPT_) low_rank_decay_kernel<TW_, TB_, CPT_><<<grid, RC_BLOCK, 0, stream>>>(low, ldl, low_col0, (const TW_*)w, bias, inv, decay, n_tokens, n, rank)
+    if (w_dtype == ROCML_BF16) { if (few) LRD(bf16_t, 1, 1); else LRD(bf16_t, LD_TOKENS, LD_CHANNELS); }
+    else { if (few) LRD(float, 1, 1); else LRD(float, LD_TOKENS, LD_CHANNELS); }
 #undef LRD
     ROCML_CHECK_LAUNCH("low_rank_decay");
     return 0;
